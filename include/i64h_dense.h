@@ -35,7 +35,9 @@ int i64h_device_check(void);
  *   I64H_EPI_SILU_MUL: silu(A W^T) * (A W2^T), laid out as I64H_EPI_GELU_MUL;
  *   I64H_EPI_XIELU: v > 0 ? act_a v^2 + v / 2 : act_b (exp(v) - 1 - v) + v / 2  (the caller passes act_a = softplus(p), act_b = 1/2 + softplus(q)).
  *   I64H_EPI_RELU_SQ: max(v, 0)^2.
- *   bias (may be NULL; fp32 [N], batch stride bias_batch) is added to the sum before any epilogue but the two gate / up ones.
+ *   I64H_EPI_CLAMP_GLU: u = min(A W^T, act_b), w = clamp(A W2^T, -act_b, act_b), u * sigmoid(act_a * u) * (w + 1), laid out as I64H_EPI_GELU_MUL;
+ *   I64H_EPI_ADD: v + E[b][m, n];  I64H_EPI_DECAY: exp(-E[b][m, n] * softplus(v))  (with lde = 0 E is one row for all m).
+ *   bias (may be NULL; fp32 [N], batch stride bias_batch) is added to the sum before any epilogue but the three gate / up ones.
  * group_off (may be NULL; device int32 [batch + 1], ascending): batch b takes the rows [group_off[b], group_off[b + 1]) of a_rows
  *   (of A itself without a_rows) and of C instead of all M rows; M is then the most rows any batch may have (it sizes the launch,
  *   workgroups past a batch's rows leave at once), and the launch needs no count on the host.  Such launches take the 64 x 64 tile form,
@@ -51,6 +53,9 @@ int i64h_device_check(void);
 #define I64H_EPI_SILU_MUL 6
 #define I64H_EPI_XIELU 7
 #define I64H_EPI_RELU_SQ 8
+#define I64H_EPI_CLAMP_GLU 9
+#define I64H_EPI_ADD 10
+#define I64H_EPI_DECAY 11
 #define I64H_SKINNY_ROWS 8
 typedef struct {
     const float* A;
@@ -139,7 +144,7 @@ typedef struct {
 int i64h_latent_prep(const i64h_latent_prep_args* d, void* stream);
 
 /* i64h_latent_attn: row t (sequence slot_ids[t], position p = positions[t]) sees the cached rows j of its sequence with
- * 0 <= p - j < window (window <= 0: every j <= p);  s_j = scale * Q[t, h, :] . row_j;  ordinary softmax over the visible j;
+ * 0 <= p - j < window (window <= 0: every j <= p) and, under a window, the first keep_first positions j < keep_first (<= p);  s_j = scale * Q[t, h, :] . row_j;  ordinary softmax over the visible j;
  * out[t, h, :kv_rank] = sum_j w_j * row_j[:kv_rank].  Scores, weights and sums in fp32.  out fp32 [n, heads, kv_rank].
  * With sink the denominator also holds exp(sink_w[h]) (exp(0) without sink_w): a term without a key and without a value, not scaled.
  * mode 1: one wave per (row, head), fp32 products, any sizes and cache type (of the options below it knows the sink).  Modes 0 / 2 / 3 take the matrix-core form when the cache
@@ -174,6 +179,7 @@ typedef struct {
                             products over 32-column steps that lie wholly inside them are left out */
     const float* sink_w; /* with sink: fp32 [heads], the extra score of head h is sink_w[h] instead of zero (NULL: zero) */
     float softcap;       /* > 0: a score s (after scale and key scale, before any bias) becomes softcap * tanh(s / softcap) */
+    int32_t keep_first;  /* with a window: the first positions of a sequence that stay visible to everyone */
 } i64h_latent_attn_args;
 int i64h_set_latent_attn_decode_form(int32_t on); /* tuning / test knob: 1 (default) = mode 2 launches run the kernel that requests a tile's fragments a tile ahead; 0 = the general matrix-core kernel; same results up to summation order */
 int64_t i64h_latent_attn_workspace_floats(int64_t n, int32_t heads, int32_t kv_rank, int32_t splits);
@@ -212,13 +218,14 @@ int i64h_embed_bigram(const i64h_embed_bigram_args* d, void* stream);
 
 /* ---- multi-stream residual (hyper-connections) with the next sublayer's RMS norm -------------------------------------------------
  * streams fp32 [S, n, W], updated in place, one workgroup per row:
- *   write (y != NULL):  v = y2 ? 0.5 * (rms(y) * yn_w + rms(y2) * y2n_w) : (yn_w ? rms(y) * yn_w : y)
+ *   write (y != NULL):  v = y2 ? (yn_w ? 0.5 * (rms(y) * yn_w + rms(y2) * y2n_w) : y + y2) : (yn_w ? rms(y) * yn_w : y)
  *                       (rms over the W columns with y_eps; weights [W]; a single normed result is the post-norm of a sandwich layer)
  *                       post_w != NULL: v <- norm(v) * post_w, over the W columns with y_eps - the root mean square, or with post_center the
  *                       centred norm (v - mean) / sqrt(mean((v - mean)^2) + y_eps): a norm on a sublayer's result, whatever it is made of
  *                       new_t = sum_s mix[s * S + t] * old_s + out_w[t] * v          (mix == NULL: new_t = old_t + out_w[t] * v)
  *   read  (h != NULL):  u = sum_s in_w[s] * x_s  (in_w == NULL: the plain sum);  h = u / sqrt(mean(u^2) + eps) * norm_w[c % norm_w_len],
- *                       or with h_center the centred norm (u - mean) / sqrt(mean((u - mean)^2) + eps) * norm_w
+ *                       or with h_center the centred norm (u - mean) / sqrt(mean((u - mean)^2) + eps) * norm_w;  norm_b (may be NULL, [W])
+ *                       is added behind the weight
  * rows (may be NULL, read only launches): h[m] is computed from row rows[m] of the streams (the rows whose logits are wanted). */
 typedef struct {
     float* streams;
@@ -244,6 +251,7 @@ typedef struct {
     const float* post_w;
     int32_t post_center;
     int32_t h_center;
+    const float* norm_b;
 } i64h_streams_args;
 int i64h_streams_step(const i64h_streams_args* d, void* stream);
 
@@ -299,6 +307,7 @@ int i64h_ssm_scan(const i64h_ssm_scan_args* d, void* stream);
 
 /* out[t, :] = rms_groups(y[t, :] * silu(z[t, :])) * w: the `width` columns in `groups` equal consecutive parts, each divided by
  * sqrt(mean(part^2) + eps).  z == NULL: no gate.  gate_after: out = rms_groups(y) * w * silu(z), the gate behind the norm.
+ * gate_act 1: sigmoid(z) in the place of silu(z).
  * w_len (0: width) values of w, repeated over the columns (a head norm whose weights all heads share). */
 typedef struct {
     const float* y;
@@ -313,6 +322,7 @@ typedef struct {
     int64_t n;
     int32_t gate_after;
     int32_t w_len;
+    int32_t gate_act;
 } i64h_gate_norm_args;
 int i64h_gate_norm(const i64h_gate_norm_args* d, void* stream);
 
@@ -367,6 +377,8 @@ int i64h_kattn_prep(const i64h_kattn_prep_args* d, void* stream);
  *   s_j = Q[t, h] . k_j * kscale_j + bias[min(p - j, bias_rows - 1) * heads + h]      (bias fp32 [bias_rows, heads], may be NULL)
  *   w_j = exp(s_j) / (sink + sum_i exp(s_i))    (sink = 1: one more score of zero that carries no value; 0: the ordinary softmax)
  *   out[t, h, :] = sum_j w_j * k_j[g, :].   Scores, weights and sums fp32.  out fp32 [n, heads, dim].
+ * With window > 0 (and no chunks) the visible positions are those with p - j < window and, of the older ones, j < keep_first.  sink_w (fp32
+ * [heads], may be NULL; with sink): exp(sink_w[h]) stands in the denominator in the place of exp(0).
  * The matrix-core form carries query and weights as two bf16 terms each (16 mantissa bits; products with the bf16 keys are exact). */
 typedef struct {
     const float* Q;
@@ -393,6 +405,8 @@ typedef struct {
                             [n, heads, vdim + dim] with the query in the last dim columns of a head, out [n, heads, vdim], kscale may be NULL;
                             the workspace is then i64h_kattn_workspace_floats(n, heads, kv_heads, vdim, splits) floats */
     float softcap;       /* > 0: the score Q . k * kscale becomes softcap * tanh(. / softcap) before the bias is added */
+    int32_t window, keep_first;
+    const float* sink_w;
 } i64h_kattn_args;
 int64_t i64h_kattn_workspace_floats(int64_t n, int32_t heads, int32_t kv_heads, int32_t dim, int32_t splits);
 int i64h_kattn(const i64h_kattn_args* d, void* stream);
@@ -494,8 +508,10 @@ int i64h_rot_post(const i64h_rot_post_args* d, void* stream);
  * Per sequence and head a (dim x vdim) matrix S in fp32, head a reading the query / key head a / (heads / kv_heads):
  *   S <- g_t S;   u = beta_t (v_t - S^T k_t);   S <- S + k_t u^T;   o_t = S^T q_t       (the read-out sees the token's own write)
  * q_t = X[t, q_off + j * dim : + dim], k_t likewise at k_off, v_t = X[t, v_off + a * vdim : + vdim]; beta_t = G[t, a], g_t = G[t, heads + a].
+ * F (may be NULL; fp32, row stride ldf): a decay per head AND key channel, F[t, a * dim + d] multiplies row d of S in the place of g_t.
  * i64h_gdn_gates prepares them: q and k of every query / key head divided by sqrt(sum of squares + unit_eps) in place (unit_eps < 0: left as
- * they are), q times q_scale;  G[t, a] = sigmoid(R[t, b_off + a]),  G[t, heads + a] = exp(-exp(A_log[a]) * softplus(R[t, a_off + a] + dt_bias[a])).
+ * they are), q times q_scale;  G[t, a] = sigmoid(R[t, b_off + a]),  G[t, heads + a] = exp(-exp(A_log[a]) * softplus(R[t, a_off + a] + dt_bias[a]))
+ * (a_off < 0: no decay per head is computed - the caller's F holds one per channel, see I64H_EPI_DECAY).
  * state fp32 [slots, heads, vdim, dim] (S transposed; dim <= 256).  All arithmetic fp32, the tokens of a sequence strictly in their order. */
 typedef struct {
     float* X;
@@ -517,6 +533,8 @@ typedef struct {
     float* out;          /* fp32 [n, heads * vdim], row stride ldo */
     int64_t ldo;
     int64_t n;
+    const float* F;
+    int64_t ldf;
 } i64h_gdn_args;
 int i64h_gdn_gates(const i64h_gdn_args* d, void* stream);
 int i64h_gdn_scan(const i64h_gdn_args* d, void* stream);
@@ -525,7 +543,10 @@ int i64h_gdn_scan(const i64h_gdn_args* d, void* stream);
  * Per row t of logits (fp32, row stride ld, E entries):  s = softmax(logits[t]);  choice = s + correction (correction may be NULL);
  * with groups > 1 the E entries form `groups` equal groups of neighbours, a group's score is its largest choice and only the entries of
  * the `keep` best groups can be chosen;  idx[t, :] = the `top` entries with the largest choice (ties: the lower index), in that order;
- * wgt[t, k] = s[idx[t, k]] / (sum_k s[idx[t, k]] + 1e-20) * scale.   E <= 1024, top <= 32. */
+ * wgt[t, k] = s[idx[t, k]] / (sum_k s[idx[t, k]] + 1e-20) * scale.   E <= 1024, top <= 32.
+ * W (bf16 [E, K], with h fp32 of row stride ldh; logits == NULL): the launch computes the logits itself in 32 bits.  bias (fp32 [E], may be
+ * NULL) is added to the logits.  chosen_softmax: the choice falls on the logits (plus correction) as they are and the weights are the softmax
+ * over the chosen logits alone, times scale.  gate_out (fp32 [n], may be NULL; with W): W has one more row, gate_out[t] = sigmoid(h[t] . W[E]). */
 typedef struct {
     const float* logits;
     int64_t ld;
@@ -540,6 +561,9 @@ typedef struct {
     int64_t ldh;
     const void* W;
     int32_t K;
+    const float* bias;
+    int32_t chosen_softmax;
+    float* gate_out;
 } i64h_route_args;
 int i64h_route_topk(const i64h_route_args* d, void* stream);
 
@@ -549,7 +573,7 @@ int i64h_route_topk(const i64h_route_args* d, void* stream);
  *   Linear), pair_row int32 [n, top] (where the pair's row lies, -1 for a non-expert).  The order of rows inside a group is not fixed;
  *   no result depends on it.  One launch of one workgroup; experts <= 4096.
  * i64h_moe_combine: out[t, :] = sum_k wgt[t, k] * (pair_row[t, k] >= 0 ? Y[pair_row[t, k], :] : h[t, :]) + (shared ? shared[t, :] : 0),
- *   summed in the order k = 0 .. top - 1, the shared row last.  Y fp32 [pairs, W]. */
+ *   summed in the order k = 0 .. top - 1, the shared row last.  Y fp32 [pairs, W].  shared_gate (fp32 [n], may be NULL) multiplies the shared row. */
 typedef struct {
     const int32_t* idx;
     int64_t n;
@@ -568,6 +592,7 @@ typedef struct {
     float* out;
     int64_t n;
     int32_t top, W;
+    const float* shared_gate;
 } i64h_moe_combine_args;
 int i64h_moe_combine(const i64h_moe_combine_args* d, void* stream);
 

@@ -532,7 +532,7 @@ def test_mixture_of_experts_alone(dev, name, l, n):
     h = torch.randn(n, cfg["width"], generator=torch.Generator().manual_seed(n + l))
     B = model.buffers(n, 1)
     B.hc.copy_(h)
-    model._moe_ff(B, model.layers[l], n)
+    model._moe_ff(B, model.layers[l], n, B.hc, B.y, B.y2)
     want = R.mixture_ff(w, f"l{l}.mlp.", cfg["layers"][l]["mlp"], h.double())
     assert close(B.y, want, 2e-5)
 
@@ -548,7 +548,7 @@ def test_experts_that_get_no_token_and_one_that_gets_all(dev):
     h = torch.randn(n, 40, generator=torch.Generator().manual_seed(3))
     B = model.buffers(n, 1)
     B.hc.copy_(h)
-    model._moe_ff(B, model.layers[l], n)
+    model._moe_ff(B, model.layers[l], n, B.hc, B.y, B.y2)
     assert B.group_off.tolist() == [0, 0, 0, n, 2 * n, 2 * n]
     want = R.mixture_ff({k: v.double() for k, v in wts.items()}, "l1.mlp.", config_of(name)["layers"][l]["mlp"], h.double())
     assert close(B.y, want, 2e-5)

@@ -262,7 +262,7 @@ class LatentAttn(ctypes.Structure):
     _fields_ = [("Q", _P), ("cache", _P), ("cache_dtype", _I), ("block_table", _P), ("max_blocks_per_seq", _I), ("block_size", _I),
                 ("slot_ids", _P), ("positions", _P), ("window", _I), ("scale", _F), ("out", _P), ("n", _L), ("heads", _I), ("kv_rank", _I),
                 ("rot_dim", _I), ("mode", _I), ("splits", _I), ("workspace", _P), ("row_stride", _I), ("kv_groups", _I), ("chunk", _I), ("kscale", _P),
-                ("bias", _P), ("bias_rows", _I), ("sink", _I), ("key_off", _I), ("sink_w", _P), ("softcap", _F)]
+                ("bias", _P), ("bias_rows", _I), ("sink", _I), ("key_off", _I), ("sink_w", _P), ("softcap", _F), ("keep_first", _I)]
 
 
 class EmbedBigram(ctypes.Structure):
@@ -275,7 +275,7 @@ class Streams(ctypes.Structure):
     """Mirror of i64h_streams_args (include/i64h_dense.h)."""
     _fields_ = [("streams", _P), ("S", _I), ("n", _L), ("W", _I), ("y", _P), ("ldy", _L), ("y2", _P), ("ldy2", _L), ("yn_w", _P), ("y2n_w", _P),
                 ("y_eps", _F), ("mix", _P), ("out_w", _P), ("in_w", _P), ("norm_w", _P), ("norm_w_len", _I), ("eps", _F), ("h", _P), ("rows", _P),
-                ("m_rows", _L), ("post_w", _P), ("post_center", _I), ("h_center", _I)]
+                ("m_rows", _L), ("post_w", _P), ("post_center", _I), ("h_center", _I), ("norm_b", _P)]
 
 
 class CausalConv(ctypes.Structure):
@@ -294,7 +294,7 @@ class SsmScan(ctypes.Structure):
 class GateNorm(ctypes.Structure):
     """Mirror of i64h_gate_norm_args (include/i64h_dense.h)."""
     _fields_ = [("y", _P), ("ldy", _L), ("z", _P), ("ldz", _L), ("w", _P), ("width", _I), ("groups", _I), ("eps", _F), ("out", _P), ("ldo", _L), ("n", _L),
-                ("gate_after", _I), ("w_len", _I)]
+                ("gate_after", _I), ("w_len", _I), ("gate_act", _I)]
 
 
 class MinGruScan(ctypes.Structure):
@@ -314,7 +314,8 @@ class KAttn(ctypes.Structure):
     """Mirror of i64h_kattn_args (include/i64h_dense.h)."""
     _fields_ = [("Q", _P), ("cache", _P), ("cache_dtype", _I), ("kscale", _P), ("block_table", _P), ("max_blocks_per_seq", _I), ("block_size", _I),
                 ("slot_ids", _P), ("positions", _P), ("chunk", _I), ("bias", _P), ("bias_rows", _I), ("sink", _I), ("out", _P), ("n", _L), ("heads", _I),
-                ("kv_heads", _I), ("dim", _I), ("mode", _I), ("splits", _I), ("workspace", _P), ("vdim", _I), ("softcap", _F)]
+                ("kv_heads", _I), ("dim", _I), ("mode", _I), ("splits", _I), ("workspace", _P), ("vdim", _I), ("softcap", _F),
+                ("window", _I), ("keep_first", _I), ("sink_w", _P)]
 
 
 class KvPrep(ctypes.Structure):
@@ -341,7 +342,8 @@ class Gdn(ctypes.Structure):
     """Mirror of i64h_gdn_args (include/i64h_dense.h)."""
     _fields_ = [("X", _P), ("ldx", _L), ("q_off", _I), ("k_off", _I), ("v_off", _I), ("heads", _I), ("kv_heads", _I), ("dim", _I), ("vdim", _I),
                 ("G", _P), ("R", _P), ("ldr", _L), ("b_off", _I), ("a_off", _I), ("A_log", _P), ("dt_bias", _P), ("unit_eps", _F), ("q_scale", _F),
-                ("seg_start", _P), ("nseg", _I), ("positions", _P), ("slot_ids", _P), ("state", _P), ("out", _P), ("ldo", _L), ("n", _L)]
+                ("seg_start", _P), ("nseg", _I), ("positions", _P), ("slot_ids", _P), ("state", _P), ("out", _P), ("ldo", _L), ("n", _L),
+                ("F", _P), ("ldf", _L)]
 
 
 class Gla(ctypes.Structure):
@@ -354,7 +356,7 @@ class Gla(ctypes.Structure):
 class Route(ctypes.Structure):
     """Mirror of i64h_route_args (include/i64h_dense.h)."""
     _fields_ = [("logits", _P), ("ld", _L), ("E", _I), ("correction", _P), ("groups", _I), ("keep", _I), ("top", _I), ("scale", _F), ("idx", _P),
-                ("wgt", _P), ("n", _L), ("h", _P), ("ldh", _L), ("W", _P), ("K", _I)]
+                ("wgt", _P), ("n", _L), ("h", _P), ("ldh", _L), ("W", _P), ("K", _I), ("bias", _P), ("chosen_softmax", _I), ("gate_out", _P)]
 
 
 class MoePlan(ctypes.Structure):
@@ -364,7 +366,7 @@ class MoePlan(ctypes.Structure):
 
 class MoeCombine(ctypes.Structure):
     """Mirror of i64h_moe_combine_args (include/i64h_dense.h)."""
-    _fields_ = [("Y", _P), ("pair_row", _P), ("wgt", _P), ("h", _P), ("shared", _P), ("out", _P), ("n", _L), ("top", _I), ("W", _I)]
+    _fields_ = [("Y", _P), ("pair_row", _P), ("wgt", _P), ("h", _P), ("shared", _P), ("out", _P), ("n", _L), ("top", _I), ("W", _I), ("shared_gate", _P)]
 
 
 _dense: Optional[ctypes.CDLL] = None

@@ -144,17 +144,28 @@ class MoeMlpConfig:
     scale: float = 1.0
     shared_ff: int = 0
     kind: str = "moe"
+    # > 0: the expert's gate is bounded from above by `limit` and its other factor u from both sides, g sigmoid(glu_alpha g) (u + 1)
+    limit: float = 0.0
+    shared_limit: float = 0.0
+    glu_alpha: float = 1.702
+    # fixed by a design: a bias on the router's logits ('router.b'), choice and softmax on the chosen logits alone, a sigmoid gate per token
+    # on the shared expert ('shared.sg')
+    router_bias: bool = False
+    chosen_softmax: bool = False
+    shared_gate: bool = False
 
     @property
     def entries(self) -> int:
         return self.experts + self.identity
 
     @classmethod
-    def from_dict(cls, m: dict) -> "MoeMlpConfig":
+    def from_dict(cls, m: dict, **design) -> "MoeMlpConfig":
         r = m["router"]
         g = r.get("groups") or {}
+        sh = m.get("shared") or {}
         c = cls(ff=int(m["expert"]["ff"]), experts=int(r["experts"]), top=int(r["top"]), identity=int(r.get("identity", 0)), groups=int(g.get("count", 1)),
-                keep=int(g.get("keep", g.get("count", 1))), scale=float(r.get("scale", 1.0)), shared_ff=int((m.get("shared") or {}).get("ff", 0)))
+                keep=int(g.get("keep", g.get("count", 1))), scale=float(r.get("scale", 1.0)), shared_ff=int(sh.get("ff", 0)),
+                limit=float(m["expert"].get("limit") or 0.0), shared_limit=float(sh.get("limit") or 0.0), **design)
         if min(c.ff, c.experts, c.top, c.groups, c.keep) <= 0 or c.identity < 0 or c.shared_ff < 0 or c.top > c.entries or c.entries % c.groups or \
                 c.keep > c.groups or c.keep * (c.entries // c.groups) < c.top:
             raise ValueError(f"mixture of experts: bad sizes {m}")
@@ -163,8 +174,12 @@ class MoeMlpConfig:
     def to_dict(self) -> dict:
         d = {"kind": "moe", "expert": {"ff": self.ff},
              "router": {"experts": self.experts, "top": self.top, "identity": self.identity, "scale": self.scale, "groups": {"count": self.groups, "keep": self.keep}}}
+        if self.limit:
+            d["expert"]["limit"] = self.limit
         if self.shared_ff:
             d["shared"] = {"ff": self.shared_ff}
+            if self.shared_limit:
+                d["shared"]["limit"] = self.shared_limit
         return d
 
 
@@ -324,9 +339,12 @@ class DecoderLayerConfig:
     weights_of: "int | None" = None      # the layer whose tensors this layer uses (its cache and state stay its own)
 
     @classmethod
-    def from_dict(cls, d: dict, mixers: "dict | None" = None) -> "DecoderLayerConfig":
-        """mixers: a design's own table of layer type -> reader of the 'mixer' entry, where its types mean other mixers than MIXERS'."""
+    def from_dict(cls, d: dict, mixers: "dict | None" = None, mlps: "dict | None" = None) -> "DecoderLayerConfig":
+        """mixers / mlps: a design's own table of layer type (feed-forward kind) -> reader of the 'mixer' ('mlp') entry, where its types mean
+        other mixers than MIXERS' (other feed-forwards than MLPS')."""
         MIXERS = mixers if mixers is not None else globals()["MIXERS"]
+        MLPS = mlps if mlps is not None else globals()["MLPS"]
+        read = lambda reader, entry: reader.from_dict(entry) if hasattr(reader, "from_dict") else reader(entry)
         kind = d.get("type")
         if kind not in MIXERS:
             raise ValueError(f"layer type '{kind}' is not built (known: {sorted(MIXERS)})")
@@ -334,8 +352,7 @@ class DecoderLayerConfig:
         share = d.get("weights_of")
         if mlp and mlp.get("kind", "dense") not in MLPS:
             raise ValueError(f"feed-forward kind '{mlp.get('kind')}' is not built (known: {sorted(MLPS)})")
-        reader = MIXERS[kind]
-        return cls(type=kind, mixer=reader.from_dict(d["mixer"]) if hasattr(reader, "from_dict") else reader(d["mixer"]), mlp=MLPS[mlp.get("kind", "dense")].from_dict(mlp) if mlp else None,
+        return cls(type=kind, mixer=read(MIXERS[kind], d["mixer"]), mlp=read(MLPS[mlp.get("kind", "dense")], mlp) if mlp else None,
                    weights_of=int(share) if share is not None else None)
 
 
@@ -585,13 +602,20 @@ class RotaryAttentionConfig:
     interleaved: bool = False
     rotate_values: bool = False
     head_gate: bool = False
+    window: int = 0                # a position sees itself and the window - 1 before it; 0: all earlier positions
+    keep_first: int = 0            # under a window: the first positions of the sequence that stay visible
+    sink: bool = False             # a learned score per head in the softmax's denominator, without key or value (tensor 'sink')
 
     @classmethod
     def from_dict(cls, m: dict, **design) -> "RotaryAttentionConfig":
+        mask = m.get("mask") or {}
         c = cls(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]),
-                softcap=float(m.get("softcap") or 0.0), rot=RotaryConfig.from_dict(m["rot"]) if m.get("rot") else None, **design)
+                softcap=float(m.get("softcap") or 0.0), rot=RotaryConfig.from_dict(m["rot"]) if m.get("rot") else None,
+                window=int(mask.get("size") or 0), keep_first=int(mask.get("keep_first") or 0), **design)
         if min(c.heads, c.kv_heads, c.dim, c.vdim) <= 0 or c.heads % c.kv_heads or c.softcap < 0 or (c.rot is not None and c.rot.dims > c.dim):
             raise ValueError(f"attention: bad sizes {m}")
+        if c.window < 0 or c.keep_first < 0:
+            raise ValueError(f"attention: bad mask {mask}")
         if c.rotate_values and c.rot is not None and c.vdim % 2:
             raise ValueError(f"attention: rotated values of an odd size {c.vdim}")
         return c
@@ -602,6 +626,8 @@ class RotaryAttentionConfig:
             d["softcap"] = self.softcap
         if self.rot is not None:
             d["rot"] = self.rot.to_dict()
+        if self.window:
+            d["mask"] = {"size": self.window, "keep_first": self.keep_first}
         return d
 
 
@@ -609,20 +635,25 @@ class RotaryAttentionConfig:
 class GatedDeltaConfig:
     """Gated delta rule: per head a (dim x vdim) matrix that decays by a scalar per head and token, is corrected towards the value along
     the (unit) key with a sigmoid strength, and is read by the (unit, scaled) query after the write; `kv_heads` query / key heads serve
-    `heads` value heads; a causal convolution of `conv` taps and silu in front of q, k and v; a gated RMS norm over vdim behind."""
+    `heads` value heads; a causal convolution of `conv` taps and silu in front of q, k and v; a gated RMS norm over vdim behind.
+    What a design fixes comes in as flags: decay 'head' (a scalar per head and token, projection 'a') or 'channel' (a factor per head and key
+    channel from a low-rank map 'a2' 'a1'); the output gate's function 'silu' (projection 'g') or 'sigmoid' (low-rank map 'g2' 'g1')."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv: int = 1
+    decay: str = "head"
+    gate: str = "silu"
 
     @property
     def conv_channels(self) -> int:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
     @classmethod
-    def from_dict(cls, m: dict) -> "GatedDeltaConfig":
-        c = cls(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), conv=int(m.get("conv", 1)))
+    def from_dict(cls, m: dict, **design) -> "GatedDeltaConfig":
+        c = cls(heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), conv=int(m.get("conv", 1)),
+                **design)
         if min(c.heads, c.kv_heads, c.dim, c.vdim, c.conv) <= 0 or c.heads % c.kv_heads:
             raise ValueError(f"gated delta rule: bad sizes {m}")
         return c
@@ -703,4 +734,80 @@ class FukatarConfig:
         d = {"architecture": "Fukatar", "vocab": self.vocab, "width": self.width, "embedding": emb, "norm": {"eps": self.norm_eps}, "layers": layers}
         if self.logit_softcap:
             d["logit_softcap"] = self.logit_softcap
+        return d
+
+
+# ---------------------------------------------------------------------------------------------------------------------------
+# Pukatar: a decoder whose layers run mixer and feed-forward side by side on one normed input, a stretch of layers repeated with the
+# same weights (each pass with a cache and state of its own), per layer one of two mixers - windowed rotated attention with kept first
+# positions and a learned sink, or a gated delta rule with a decay per key channel - and one of two feed-forwards, a gated one or a
+# mixture of clamped experts with a gated shared one.  Every size and constant comes from config.json.
+# ---------------------------------------------------------------------------------------------------------------------------
+PUKATAR_MIXERS = {"attention": lambda m: RotaryAttentionConfig.from_dict(m, sink=True),
+                  "channel_delta": lambda m: GatedDeltaConfig.from_dict(m, decay="channel", gate="sigmoid")}
+PUKATAR_MLPS = {"dense": DenseMlpConfig, "moe": lambda m: MoeMlpConfig.from_dict(m, router_bias=True, chosen_softmax=True, shared_gate=True)}
+
+
+@dataclass
+class LayerLoop:
+    """Layers start .. stop - 1 run `times` times in a row with the same weights."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
+class PukatarConfig:
+    vocab: int
+    width: int
+    layers: list
+    norm_eps: float = 1e-6
+    loop: "LayerLoop | None" = None
+    name: str = "Pukatar"
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def vocab_size(self) -> int:
+        return self.vocab
+
+    @property
+    def max_pos(self) -> int:
+        """Positions are computed, not tabulated: a sequence is bounded by the page pool only."""
+        return 1 << 30
+
+    def layer_runs(self) -> list:
+        """[(layer, number of the pass that begins in front of it or None)] in the order they run; run r has cache and state number r."""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return [(i, None) for i in range(n)]
+        runs = [(i, None) for i in range(lp.start)]
+        for t in range(lp.times):
+            runs += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
+        return runs + [(i, None) for i in range(lp.stop, n)]
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "PukatarConfig":
+        layers = [DecoderLayerConfig.from_dict(l, PUKATAR_MIXERS, PUKATAR_MLPS) for l in d["layers"]]
+        lp = d.get("loop")
+        c = cls(vocab=int(d["vocab"]), width=int(d["width"]), layers=layers, norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)),
+                loop=LayerLoop(int(lp["start"]), int(lp["stop"]), int(lp["times"])) if lp else None, name=str(d.get("architecture", "Pukatar")))
+        if min(c.vocab, c.width) <= 0 or not layers:
+            raise ValueError("bad sizes")
+        if c.loop is not None and (not 0 <= c.loop.start < c.loop.stop <= len(layers) or c.loop.times < 1):
+            raise ValueError(f"loop {lp} over {len(layers)} layers")
+        for i, l in enumerate(layers):
+            if l.weights_of is not None:
+                raise ValueError(f"layer {i}: this design has no layers that borrow tensors")
+            if l.mlp is not None and l.mlp.kind == "moe" and (l.mlp.limit <= 0 or (l.mlp.shared_ff and l.mlp.shared_limit <= 0)):
+                raise ValueError(f"layer {i}: the experts of this design are clamped, 'limit' is missing")
+        return c
+
+    def to_dict(self) -> dict:
+        d = {"architecture": "Pukatar", "vocab": self.vocab, "width": self.width, "norm": {"eps": self.norm_eps},
+             "layers": [{"type": l.type, "mixer": l.mixer.to_dict(), "mlp": l.mlp.to_dict() if l.mlp else None} for l in self.layers]}
+        if self.loop is not None:
+            d["loop"] = {"start": self.loop.start, "stop": self.loop.stop, "times": self.loop.times}
         return d

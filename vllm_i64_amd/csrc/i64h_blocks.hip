@@ -2,8 +2,9 @@
 //   gla_gates_kernel   : query activation and bounded forget gate, in place on the projection rows
 //   gla_scan_kernel    : linear attention with a decay per key channel, a head's matrix in registers (16 lanes per value column)
 //   gdn_gates_kernel / gdn_scan_kernel : gated delta rule - unit-vector queries and keys, write strength and decay; the recurrence with the
-//                        correction S^T k summed over the DPP row before the write, the read-out after it
-//   route_topk_kernel  : softmax scores, corrected choice, groups of neighbours, top-k and normalised weights, one wave per row
+//                        correction S^T k summed over the DPP row before the write, the read-out after it; a decay per head or per key channel
+//   route_topk_kernel  : softmax scores (over all entries or the chosen ones), corrected choice, groups of neighbours, top-k and normalised
+//                        weights, one wave per row
 //   moe_plan_kernel    : (token, choice) pairs grouped by expert: offsets, the token of every grouped row, the row of every pair
 //   moe_combine_kernel : weighted sum of the chosen experts' rows, pass-through entries and the shared expert's row
 // A row continues the row before it iff slot and position say so; state is taken as empty at position 0.  All arithmetic fp32.
@@ -167,7 +168,7 @@ __global__ __launch_bounds__(256) void gdn_gates_kernel(const i64h_gdn_args p) {
     for (int a = threadIdx.x; a < p.heads; a += 256) {
         const float* r = p.R + t * p.ldr;
         p.G[t * 2 * p.heads + a] = bl_sigmoid(r[p.b_off + a]);
-        p.G[t * 2 * p.heads + p.heads + a] = expf(-expf(p.A_log[a]) * bl_softplus(r[p.a_off + a] + p.dt_bias[a]));
+        if (p.a_off >= 0) p.G[t * 2 * p.heads + p.heads + a] = expf(-expf(p.A_log[a]) * bl_softplus(r[p.a_off + a] + p.dt_bias[a]));
     }
 }
 
@@ -175,7 +176,8 @@ __global__ __launch_bounds__(256) void gdn_gates_kernel(const i64h_gdn_args p) {
 // row share CPT value columns and hold KPT key channels of each in registers).  Per token the state decays, the row sums S^T k with DPP
 // moves (every lane of the row ends with the sum), the correction along k is written, and a second row sum reads the state out with
 // the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order; loads run GL_TG tokens ahead.
-template <int KPT, int CPT>
+// CHD: a decay per head and key channel (F) in the place of one per head.
+template <int KPT, int CPT, bool CHD>
 __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, const int ctiles, const int vec) {
     const int N = p.dim, P = p.vdim;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -210,9 +212,9 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
             }
         }
     }
-    const int qoff = p.q_off + kh * N + n0, koff = p.k_off + kh * N + n0;
+    const int qoff = p.q_off + kh * N + n0, koff = p.k_off + kh * N + n0, foff = a * N + n0;
     struct Tok {
-        float q[KPT], k[KPT], v[CPT], beta, g;
+        float q[KPT], k[KPT], f[CHD ? KPT : 1], v[CPT], beta;
     };
     auto fetch = [&](int64_t t, Tok& u) {
         if (t >= r1) return;
@@ -220,13 +222,15 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
         if (vec) {      // KPT % 4 == 0 and every slice starts at a multiple of four floats and lies inside the row
 #pragma unroll
             for (int k = 0; k < KPT; k += 4) {
-                float4 q = make_float4(0, 0, 0, 0), kk = q;
+                float4 q = make_float4(0, 0, 0, 0), kk = q, f = q;
                 if (n0 + k < N) {
                     q = *(const float4*)(row + qoff + k);
                     kk = *(const float4*)(row + koff + k);
+                    if (CHD) f = *(const float4*)(p.F + t * p.ldf + foff + k);
                 }
                 u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
                 u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
+                if (CHD) u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
             }
         } else {
 #pragma unroll
@@ -234,12 +238,13 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
                 const bool ok = n0 + k < N;
                 u.q[k] = ok ? row[qoff + k] : 0.0f;
                 u.k[k] = ok ? row[koff + k] : 0.0f;
+                if (CHD) u.f[k] = ok ? p.F[t * p.ldf + foff + k] : 0.0f;
             }
         }
 #pragma unroll
         for (int j = 0; j < CPT; ++j) u.v[j] = cbase + j < P ? row[p.v_off + a * P + cbase + j] : 0.0f;
         u.beta = p.G[t * 2 * p.heads + a];
-        u.g = p.G[t * 2 * p.heads + p.heads + a];
+        if (!CHD) u.f[0] = p.G[t * 2 * p.heads + p.heads + a];
     };
     auto step = [&](int64_t t, const Tok& u) {
         if (t >= r1) return;
@@ -248,7 +253,7 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
             float seen = 0.0f;
 #pragma unroll
             for (int k = 0; k < KPT; ++k) {
-                S[j][k] *= u.g;
+                S[j][k] *= u.f[CHD ? k : 0];
                 seen = fmaf(S[j][k], u.k[k], seen);
             }
             seen = group_sum(seen, 16);
@@ -316,14 +321,15 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
         const uint16_t* W = (const uint16_t*)p.W;
         const int K = p.K;
         const bool vec = (K & 3) == 0 && (p.ldh & 3) == 0 && ((uintptr_t)p.h & 15) == 0 && ((uintptr_t)p.W & 7) == 0;
-        for (int e0 = 0; e0 < E; e0 += 8) {
+        const int rows = p.gate_out ? E + 1 : E;
+        for (int e0 = 0; e0 < rows; e0 += 8) {
             float acc[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
             if (vec) {
                 for (int k = lane * 4; k < K; k += 256) {
                     const float4 x = *(const float4*)(h + k);
 #pragma unroll
                     for (int j = 0; j < 8; ++j) {
-                        if (e0 + j < E) {
+                        if (e0 + j < rows) {
                             const uint2 w = *(const uint2*)(W + (int64_t)(e0 + j) * K + k);
                             acc[j] = fmaf(x.x, __uint_as_float(w.x << 16), acc[j]);
                             acc[j] = fmaf(x.y, __uint_as_float(w.x & 0xffff0000u), acc[j]);
@@ -337,33 +343,42 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
                     const float x = h[k];
 #pragma unroll
                     for (int j = 0; j < 8; ++j)
-                        if (e0 + j < E) acc[j] = fmaf(x, __uint_as_float((uint32_t)W[(int64_t)(e0 + j) * K + k] << 16), acc[j]);
+                        if (e0 + j < rows) acc[j] = fmaf(x, __uint_as_float((uint32_t)W[(int64_t)(e0 + j) * K + k] << 16), acc[j]);
                 }
             }
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
                 const float v = wave_sum(acc[j]);
-                if (lane == 0 && e0 + j < E) ch[e0 + j] = v;
+                if (lane == 0 && e0 + j < E) ch[e0 + j] = p.bias ? v + p.bias[e0 + j] : v;
+                if (lane == 0 && e0 + j == E && p.gate_out) p.gate_out[t] = bl_sigmoid(v);
             }
         }
     } else {
         const float* z = p.logits + t * p.ld;
-        for (int e = lane; e < E; e += 64) ch[e] = z[e];
+        for (int e = lane; e < E; e += 64) ch[e] = p.bias ? z[e] + p.bias[e] : z[e];
     }
-    float mx = -INFINITY;
-    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, ch[e]);
-    mx = wave_max(mx);
-    float sum = 0.0f;
-    for (int e = lane; e < E; e += 64) {
-        const float v = expf(ch[e] - mx);
-        sc[e] = v;
-        sum += v;
-    }
-    sum = wave_sum(sum);
-    for (int e = lane; e < E; e += 64) {
-        const float s = sc[e] / sum;
-        sc[e] = s;
-        ch[e] = p.correction ? s + p.correction[e] : s;
+    if (p.chosen_softmax) {     // the choice falls on the logits themselves
+        for (int e = lane; e < E; e += 64) {
+            const float s = ch[e];
+            sc[e] = s;
+            if (p.correction) ch[e] = s + p.correction[e];
+        }
+    } else {
+        float mx = -INFINITY;
+        for (int e = lane; e < E; e += 64) mx = fmaxf(mx, ch[e]);
+        mx = wave_max(mx);
+        float sum = 0.0f;
+        for (int e = lane; e < E; e += 64) {
+            const float v = expf(ch[e] - mx);
+            sc[e] = v;
+            sum += v;
+        }
+        sum = wave_sum(sum);
+        for (int e = lane; e < E; e += 64) {
+            const float s = sc[e] / sum;
+            sc[e] = s;
+            ch[e] = p.correction ? s + p.correction[e] : s;
+        }
     }
     if (G > 1) {   // a group's score: its largest choice value; the `keep` best groups stay, the entries of the others cannot be chosen
         for (int g = lane; g < G; g += 64) {
@@ -403,6 +418,11 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
         wsum += s;
         if (lane == k) mine_w = s, mine_i = pick;
         if (lane == 0) ch[pick] = __builtin_nanf("");     // taken: out of every later comparison
+    }
+    if (p.chosen_softmax) {     // ... and the weights are the softmax over the chosen ones
+        const float top1 = wave_max(lane < p.top ? mine_w : -INFINITY);
+        mine_w = lane < p.top ? expf(mine_w - top1) : 0.0f;
+        wsum = wave_sum(mine_w);
     }
     if (lane < p.top) {
         p.idx[t * p.top + lane] = mine_i;
@@ -457,7 +477,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const i64h_moe_combine
             const float v = r >= 0 ? p.Y[(int64_t)r * W + c] : p.h[t * W + c];
             a += p.wgt[t * p.top + k] * v;
         }
-        if (p.shared) a += p.shared[t * W + c];
+        if (p.shared) a += p.shared_gate ? p.shared_gate[t] * p.shared[t * W + c] : p.shared[t * W + c];
         p.out[t * W + c] = a;
     }
 }
@@ -528,7 +548,7 @@ int i64h_gdn_gates(const i64h_gdn_args* dp, void* stream) {
     I64H_CHECK_ARG(dp != nullptr, "gdn_gates: no descriptor");
     const i64h_gdn_args& d = *dp;
     if (gdn_check(d, "gdn_gates")) return 1;
-    I64H_CHECK_ARG(d.R && d.A_log && d.dt_bias && d.b_off >= 0 && d.a_off >= 0, "gdn_gates: null operand or negative column");
+    I64H_CHECK_ARG(d.R && d.b_off >= 0 && (d.a_off < 0 || (d.A_log && d.dt_bias)), "gdn_gates: null operand or negative column");
     if (d.n == 0) return 0;
     hipLaunchKernelGGL(gdn_gates_kernel, dim3((unsigned)d.n), dim3(256), 0, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();
@@ -550,16 +570,21 @@ int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
     const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
     const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
     auto launch = [&](auto kern, int K) {
-        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldx % 4 == 0 && d.q_off % 4 == 0 && d.k_off % 4 == 0 && (uintptr_t)d.X % 16 == 0 && (uintptr_t)d.state % 16 == 0;
+        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldx % 4 == 0 && d.q_off % 4 == 0 && d.k_off % 4 == 0 && (uintptr_t)d.X % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
+                        (!d.F || (d.ldf % 4 == 0 && (uintptr_t)d.F % 16 == 0));
         hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
     };
-#define GDN_PICK(C)                                          \
-    if (kpt <= 1) launch(gdn_scan_kernel<1, C>, 1);          \
-    else if (kpt <= 2) launch(gdn_scan_kernel<2, C>, 2);     \
-    else if (kpt <= 4) launch(gdn_scan_kernel<4, C>, 4);     \
-    else if (kpt <= 8) launch(gdn_scan_kernel<8, C>, 8);     \
-    else launch(gdn_scan_kernel<16, C>, 16);
-    if (cpt == 2) { GDN_PICK(2) } else { GDN_PICK(1) }
+#define GDN_PICK(C, CHD)                                          \
+    if (kpt <= 1) launch(gdn_scan_kernel<1, C, CHD>, 1);          \
+    else if (kpt <= 2) launch(gdn_scan_kernel<2, C, CHD>, 2);     \
+    else if (kpt <= 4) launch(gdn_scan_kernel<4, C, CHD>, 4);     \
+    else if (kpt <= 8) launch(gdn_scan_kernel<8, C, CHD>, 8);     \
+    else launch(gdn_scan_kernel<16, C, CHD>, 16);
+    if (d.F) {
+        if (cpt == 2) { GDN_PICK(2, true) } else { GDN_PICK(1, true) }
+    } else {
+        if (cpt == 2) { GDN_PICK(2, false) } else { GDN_PICK(1, false) }
+    }
 #undef GDN_PICK
     I64H_CHECK_LAUNCH();
     return 0;
@@ -570,6 +595,7 @@ int i64h_route_topk(const i64h_route_args* dp, void* stream) {
     const i64h_route_args& d = *dp;
     I64H_CHECK_ARG(d.E > 0 && d.E <= 1024 && d.top > 0 && d.top <= RT_MAX_TOP && d.top <= d.E, "route_topk: %d entries (at most 1024), top %d (at most %d)", d.E, d.top, RT_MAX_TOP);
     I64H_CHECK_ARG(d.groups <= 1 || (d.E % d.groups == 0 && d.keep >= 1 && d.keep <= d.groups), "route_topk: %d entries in %d groups, %d kept", d.E, d.groups, d.keep);
+    I64H_CHECK_ARG(!d.gate_out || d.W, "route_topk: the gate's row lies behind the router's rows");
     I64H_CHECK_ARG(d.groups <= 1 || d.keep * (d.E / d.groups) >= d.top, "route_topk: %d kept groups of %d entries hold fewer than top %d", d.keep, d.E / (d.groups > 0 ? d.groups : 1), d.top);
     I64H_CHECK_ARG(d.idx && d.wgt && ((d.logits && d.ld >= d.E) || (d.W && d.h && d.K > 0 && d.ldh >= d.K)), "route_topk: null operand or row stride below the row");
     if (d.n == 0) return 0;

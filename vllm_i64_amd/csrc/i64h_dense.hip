@@ -31,15 +31,21 @@ __device__ __forceinline__ float dn_gelu_tanh(float z) {
 
 __device__ __forceinline__ float dn_gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
+__device__ __forceinline__ float dn_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+
 __device__ __forceinline__ float dn_xielu(float z, float a, float b) {
     return z > 0.0f ? a * z * z + 0.5f * z : b * (expm1f(z) - z) + 0.5f * z;
 }
-constexpr bool dn_dual(int epi) { return epi == I64H_EPI_GELU_MUL || epi == I64H_EPI_SILU_MUL; }  // two accumulators: gate rows and up rows
+constexpr bool dn_dual(int epi) { return epi == I64H_EPI_GELU_MUL || epi == I64H_EPI_SILU_MUL || epi == I64H_EPI_CLAMP_GLU; }  // two accumulators: gate rows and up rows
 
 template <int EPI>
 __device__ __forceinline__ float dn_epilogue(const i64h_linear& p, float acc, float acc2, int64_t b, int64_t r, int c) {
     if (EPI == I64H_EPI_GELU_MUL) return dn_gelu_tanh(acc) * acc2;
     if (EPI == I64H_EPI_SILU_MUL) return acc * dn_sigmoid(acc) * acc2;
+    if (EPI == I64H_EPI_CLAMP_GLU) {
+        const float u = fminf(acc, p.act_b), w = fminf(fmaxf(acc2, -p.act_b), p.act_b);
+        return u * dn_sigmoid(p.act_a * u) * (w + 1.0f);
+    }
     if (p.bias) acc += p.bias[b * p.bias_batch + c];
     if (EPI == I64H_EPI_XIELU) return dn_xielu(acc, p.act_a, p.act_b);
     if (EPI == I64H_EPI_RELU_SQ) return acc > 0.0f ? acc * acc : 0.0f;
@@ -47,6 +53,8 @@ __device__ __forceinline__ float dn_epilogue(const i64h_linear& p, float acc, fl
     if (EPI == I64H_EPI_SCALE) return acc * p.scale;
     if (EPI == I64H_EPI_MUL_SIGMOID) return acc * dn_sigmoid(p.E[b * p.e_batch + r * p.lde + c]);
     if (EPI == I64H_EPI_SOFTCAP) return p.softcap * tanhf(acc / p.softcap);
+    if (EPI == I64H_EPI_ADD) return acc + p.E[b * p.e_batch + r * p.lde + c];
+    if (EPI == I64H_EPI_DECAY) return expf(-p.E[b * p.e_batch + r * p.lde + c] * dn_softplus(acc));
     return acc;
 }
 
@@ -686,11 +694,14 @@ static void launch_tile(const i64h_linear& d, dim3 grid, hipStream_t s, int vecA
     switch (d.epilogue) {
         case I64H_EPI_GELU_MUL: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_GELU_MUL>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_SILU_MUL: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_SILU_MUL>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+        case I64H_EPI_CLAMP_GLU: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_CLAMP_GLU>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_MUL_SIGMOID: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_MUL_SIGMOID>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_SOFTCAP: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_SOFTCAP>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_GELU_ERF: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_GELU_ERF>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_XIELU: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_XIELU>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_RELU_SQ>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+        case I64H_EPI_ADD: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_ADD>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+        case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_DECAY>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_SCALE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         default: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_STORE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
     }
@@ -717,8 +728,9 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
     const i64h_linear& d = *dp;
     I64H_CHECK_ARG(d.M >= 0 && d.N > 0 && d.K > 0 && d.batch > 0, "linear: bad sizes M=%lld N=%d K=%d batch=%d", (long long)d.M, d.N, d.K, d.batch);
     I64H_CHECK_ARG(d.A && d.W && d.C, "linear: null operand");
-    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_RELU_SQ, "linear: epilogue %d", d.epilogue);
-    I64H_CHECK_ARG(d.epilogue != I64H_EPI_MUL_SIGMOID || d.E, "linear: the sigmoid epilogue needs E");
+    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_DECAY, "linear: epilogue %d", d.epilogue);
+    I64H_CHECK_ARG((d.epilogue != I64H_EPI_MUL_SIGMOID && d.epilogue != I64H_EPI_ADD && d.epilogue != I64H_EPI_DECAY) || d.E, "linear: epilogue %d needs E", d.epilogue);
+    I64H_CHECK_ARG(d.epilogue != I64H_EPI_CLAMP_GLU || d.act_b > 0.0f, "linear: bound %g of the clamped gate / up epilogue", (double)d.act_b);
     I64H_CHECK_ARG(d.epilogue != I64H_EPI_SOFTCAP || d.softcap > 0.0f, "linear: soft cap %g", (double)d.softcap);
     I64H_CHECK_ARG(!dn_dual(d.epilogue) || !d.bias, "linear: the gate / up epilogues take no bias");
     I64H_CHECK_ARG(d.lda >= d.K || d.M <= 1, "linear: lda %lld < K %d", (long long)d.lda, d.K);
@@ -735,11 +747,14 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
         switch (d.epilogue) {
             case I64H_EPI_GELU_MUL: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_GELU_MUL>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_SILU_MUL: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_SILU_MUL>), grid, dim3(256), lds, s, d, cpb); break;
+            case I64H_EPI_CLAMP_GLU: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_CLAMP_GLU>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_MUL_SIGMOID: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_MUL_SIGMOID>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_SOFTCAP: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_SOFTCAP>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_GELU_ERF: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_GELU_ERF>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_XIELU: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_XIELU>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_RELU_SQ>), grid, dim3(256), lds, s, d, cpb); break;
+            case I64H_EPI_ADD: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_ADD>), grid, dim3(256), lds, s, d, cpb); break;
+            case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_DECAY>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_SCALE>), grid, dim3(256), lds, s, d, cpb); break;
             default: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_STORE>), grid, dim3(256), lds, s, d, cpb); break;
         }
@@ -752,11 +767,14 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             // eight waves share the k steps where one accumulator is kept (the gate / up pair needs twice the LDS: four)
             case I64H_EPI_GELU_MUL: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_GELU_MUL, 4>), grid, dim3(256), 0, s, d); break;
             case I64H_EPI_SILU_MUL: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_SILU_MUL, 4>), grid, dim3(256), 0, s, d); break;
+            case I64H_EPI_CLAMP_GLU: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_CLAMP_GLU, 4>), grid, dim3(256), 0, s, d); break;
             case I64H_EPI_MUL_SIGMOID: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_MUL_SIGMOID, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_SOFTCAP: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_SOFTCAP, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_GELU_ERF: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_GELU_ERF, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_XIELU: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_XIELU, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_RELU_SQ, 8>), grid, dim3(512), 0, s, d); break;
+            case I64H_EPI_ADD: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_ADD, 8>), grid, dim3(512), 0, s, d); break;
+            case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_DECAY, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_SCALE, 8>), grid, dim3(512), 0, s, d); break;
             default: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_STORE, 8>), grid, dim3(512), 0, s, d); break;
         }
@@ -769,11 +787,14 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
         switch (d.epilogue) {
             case I64H_EPI_GELU_MUL: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_GELU_MUL>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_SILU_MUL: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_SILU_MUL>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+            case I64H_EPI_CLAMP_GLU: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_CLAMP_GLU>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_MUL_SIGMOID: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_MUL_SIGMOID>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_SOFTCAP: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_SOFTCAP>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_GELU_ERF: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_GELU_ERF>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_XIELU: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_XIELU>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_RELU_SQ>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+            case I64H_EPI_ADD: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_ADD>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+            case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_DECAY>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_SCALE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             default: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_STORE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         }

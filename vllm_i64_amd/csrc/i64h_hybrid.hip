@@ -11,7 +11,7 @@
 //   kattn_prep_kernel     : whole-row RMS norms of query and key, key-norm weights / scale / temperature folded into the query,
 //                           raw key row and its 1 / rms into the paged cache
 //   kattn_row_kernel      : attention over the cached keys (which are also the values, or with the values in front of them in the
-//                           same cached row) with distance bias, chunk mask and sink
+//                           same cached row) with distance bias, chunk mask or window with kept first positions, and sink
 //   kv_prep_kernel        : [q | k | v] projections -> the cached row [v | k] per key head and query rows with zeros in the value columns
 //   rot_prep_kernel       : the same with whole-row or per-head query / key norms, rotation of a part of every head in either pair layout
 //                           and values turned by their own position; rot_post_kernel turns a head's sum back and applies a gate per head
@@ -82,7 +82,7 @@ __global__ __launch_bounds__(256) void streams_kernel(const i64h_streams_args p)
     const int64_t plane = p.n * (int64_t)W;
     float* xs = p.streams + r * W;
     float ya = 1.0f, yb = 1.0f;
-    if (p.y && p.y2) {   // the two side-by-side results, each divided by its root mean square
+    if (p.y && p.y2 && p.yn_w) {   // the two side-by-side results, each divided by its root mean square
         float a = 0.0f, b = 0.0f;
         for (int c = tid; c < W; c += 256) {
             const float u = p.y[m * p.ldy + c], v = p.y2[m * p.ldy2 + c];
@@ -102,10 +102,12 @@ __global__ __launch_bounds__(256) void streams_kernel(const i64h_streams_args p)
         a = hy_block_sum(a, red);
         ya = sqrtf(a / (float)W + p.y_eps);     // divided by, as the norm in front is
     }
-    // the result as the residual receives it: both side-by-side parts normed and averaged, or the one result with its own norm, or as it is
+    // the result as the residual receives it: both side-by-side parts normed and averaged or simply summed, or the one result with its own
+    // norm, or as it is
     auto result = [&](int c) -> float {
         float v = p.y[m * p.ldy + c];
-        if (p.y2) v = 0.5f * (v * ya * p.yn_w[c] + p.y2[m * p.ldy2 + c] * yb * p.y2n_w[c]);
+        if (p.y2 && !p.yn_w) v += p.y2[m * p.ldy2 + c];
+        else if (p.y2) v = 0.5f * (v * ya * p.yn_w[c] + p.y2[m * p.ldy2 + c] * yb * p.y2n_w[c]);
         else if (p.yn_w) v = v / ya * p.yn_w[c];
         return v;
     };
@@ -173,7 +175,10 @@ __global__ __launch_bounds__(256) void streams_kernel(const i64h_streams_args p)
     }
     ss = hy_block_sum(ss, red);
     const float den = sqrtf(ss / (float)W + p.eps);
-    for (int c = tid; c < W; c += 256) p.h[m * W + c] = (sv[c] - mean) / den * p.norm_w[p.norm_w_len == 1 ? 0 : c];
+    for (int c = tid; c < W; c += 256) {
+        const float v = (sv[c] - mean) / den * p.norm_w[p.norm_w_len == 1 ? 0 : c];
+        p.h[m * W + c] = p.norm_b ? v + p.norm_b[c] : v;
+    }
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -378,7 +383,7 @@ __global__ __launch_bounds__(256) void gate_norm_kernel(const i64h_gate_norm_arg
     const int W = p.width;
     for (int c = tid; c < W; c += 256) {
         float v = p.y[m * p.ldy + c];
-        if (p.z && !p.gate_after) v *= hy_silu(p.z[m * p.ldz + c]);
+        if (p.z && !p.gate_after) v *= p.gate_act ? hy_sigmoid(p.z[m * p.ldz + c]) : hy_silu(p.z[m * p.ldz + c]);
         sv[c] = v;
     }
     __syncthreads();
@@ -395,7 +400,7 @@ __global__ __launch_bounds__(256) void gate_norm_kernel(const i64h_gate_norm_arg
     __syncthreads();
     for (int c = tid; c < W; c += 256) {
         float v = sv[c] / sv[W + c / gs] * p.w[p.w_len > 0 ? c % p.w_len : c];
-        if (p.z && p.gate_after) v *= hy_silu(p.z[m * p.ldz + c]);
+        if (p.z && p.gate_after) v *= p.gate_act ? hy_sigmoid(p.z[m * p.ldz + c]) : hy_silu(p.z[m * p.ldz + c]);
         p.out[m * p.ldo + c] = v;
     }
 }
@@ -512,16 +517,18 @@ __global__ __launch_bounds__(256) void kattn_row_kernel(const i64h_kattn_args p)
     const int dim = p.dim, vd = p.vdim > 0 ? p.vdim : dim, koff = p.vdim > 0 ? p.vdim : 0, gs = koff + dim;
     const int nk = p.kv_heads * gs;
     const int pos = p.positions[t], slot = p.slot_ids[t];
-    const int lo = p.chunk > 0 ? (pos / p.chunk) * p.chunk : 0;
+    const int lo = p.chunk > 0 ? (pos / p.chunk) * p.chunk : (p.window > 0 ? max(0, pos - p.window + 1) : 0);
+    // the visible keys in order: the kept first positions in front of the window, then lo .. pos
+    const int kept = p.chunk <= 0 && p.window > 0 ? min(p.keep_first, lo) : 0, total = kept + pos - lo + 1;
     const T* cache = (const T*)p.cache;
     for (int d = lane; d < dim; d += 64) sq[wid][d] = p.Q[(t * p.heads + h) * gs + koff + d];
-    float m = p.sink ? 0.0f : -INFINITY, l = p.sink ? 1.0f : 0.0f;
+    float m = p.sink ? (p.sink_w ? p.sink_w[h] : 0.0f) : -INFINITY, l = p.sink ? 1.0f : 0.0f;
     float acc[KA_MAX_DIM / 64] = {0.0f, 0.0f, 0.0f, 0.0f};
-    for (int j0 = lo; j0 <= pos; j0 += 64) {
-        const int j = j0 + lane;
+    for (int i0 = 0; i0 < total; i0 += 64) {
+        const int i = i0 + lane, j = i < kept ? i : lo + i - kept;
         float s = -INFINITY;
         int64_t row = 0;
-        if (j <= pos) {
+        if (i < total) {
             row = cache_row(p.block_table, p.max_blocks_per_seq, p.block_size, slot, j);
             const T* kr = cache + row * nk + g * gs + koff;
             float dot = 0.0f;
@@ -532,19 +539,19 @@ __global__ __launch_bounds__(256) void kattn_row_kernel(const i64h_kattn_args p)
         }
         srow[wid][lane] = row;
         const float mn = fmaxf(m, wave_max(s));
-        const float w = j <= pos ? expf(s - mn) : 0.0f;
+        const float w = i < total ? expf(s - mn) : 0.0f;
         const float f = expf(m - mn);      // m is finite or the first tile has a key (mn finite): no inf - inf
         l = l * f + wave_sum(w);
         m = mn;
         sp[wid][lane] = w;
-        const int cnt = min(64, pos - j0 + 1);
+        const int cnt = min(64, total - i0);
 #pragma unroll
-        for (int i = 0; i < KA_MAX_DIM / 64; ++i) {
-            const int d = lane + 64 * i;
+        for (int c = 0; c < KA_MAX_DIM / 64; ++c) {
+            const int d = lane + 64 * c;
             if (d < vd) {
-                float a = acc[i] * f;
+                float a = acc[c] * f;
                 for (int u = 0; u < cnt; ++u) a += sp[wid][u] * (float)cache[srow[wid][u] * nk + g * gs + d];
-                acc[i] = a;
+                acc[c] = a;
             }
         }
     }
@@ -757,7 +764,7 @@ int i64h_streams_step(const i64h_streams_args* dp, void* stream) {
     I64H_CHECK_ARG(d.S >= 1 && d.S <= HY_MAX_STREAMS && d.W > 0 && d.n >= 0, "streams: %d streams (at most %d), width %d", d.S, HY_MAX_STREAMS, d.W);
     I64H_CHECK_ARG(d.streams && (d.y || d.h), "streams: nothing to do");
     I64H_CHECK_ARG(!d.y || d.out_w, "streams: the write needs out_w");
-    I64H_CHECK_ARG(!d.y2 || (d.y && d.yn_w && d.y2n_w), "streams: two results need both norm weights");
+    I64H_CHECK_ARG(!d.y2 || (d.y && !d.yn_w == !d.y2n_w), "streams: two results take both norm weights or none");
     I64H_CHECK_ARG(!d.h || (d.norm_w && (d.norm_w_len == 1 || d.norm_w_len == d.W)), "streams: the read needs a norm weight of 1 or W values");
     I64H_CHECK_ARG(!d.rows || !d.y, "streams: gathered rows are read only");
     const int64_t rows = d.rows ? d.m_rows : d.n;
@@ -884,6 +891,7 @@ int i64h_kattn(const i64h_kattn_args* dp, void* stream) {
     I64H_CHECK_ARG(d.Q && d.cache && (d.kscale || d.vdim > 0) && d.block_table && d.slot_ids && d.positions && d.out, "kattn: null operand");
     I64H_CHECK_ARG(d.cache_dtype == 0 || d.cache_dtype == 2, "kattn: cache type %d", d.cache_dtype);
     I64H_CHECK_ARG(!d.bias || d.bias_rows > 0, "kattn: an empty bias table");
+    I64H_CHECK_ARG(d.keep_first >= 0 && (!d.sink_w || d.sink), "kattn: %d kept positions, or sink scores without the sink", d.keep_first);
     I64H_CHECK_ARG(d.block_size > 0 && d.max_blocks_per_seq > 0, "kattn: bad paging");
     if (d.n == 0) return 0;
     // the matrix-core kernel of the latent attention scores against a whole cached row part and sums its first columns: the keys as values
@@ -892,10 +900,10 @@ int i64h_kattn(const i64h_kattn_args* dp, void* stream) {
     if (d.mode != 1 && d.cache_dtype == 2 && vals % 16 == 0 && vals <= 256 && gs % 8 == 0 && gs <= 320 && (uintptr_t)d.Q % 16 == 0 && (uintptr_t)d.cache % 16 == 0) {
         i64h_latent_attn_args a = {};
         a.Q = d.Q, a.cache = d.cache, a.cache_dtype = d.cache_dtype, a.block_table = d.block_table, a.max_blocks_per_seq = d.max_blocks_per_seq;
-        a.block_size = d.block_size, a.slot_ids = d.slot_ids, a.positions = d.positions, a.window = 0, a.scale = 1.0f, a.out = d.out, a.n = d.n;
+        a.block_size = d.block_size, a.slot_ids = d.slot_ids, a.positions = d.positions, a.window = d.window, a.keep_first = d.keep_first, a.scale = 1.0f, a.out = d.out, a.n = d.n;
         a.heads = d.heads, a.kv_rank = vals, a.rot_dim = gs - vals, a.mode = d.mode == 3 ? 3 : 2, a.splits = d.splits, a.workspace = d.workspace;
         a.row_stride = d.kv_heads * gs, a.kv_groups = d.kv_heads, a.chunk = d.chunk, a.kscale = d.kscale, a.bias = d.bias, a.bias_rows = d.bias_rows;
-        a.sink = d.sink, a.softcap = d.softcap;
+        a.sink = d.sink, a.sink_w = d.sink_w, a.softcap = d.softcap;
         a.key_off = d.vdim > 0 ? d.vdim : 0;
         return i64h_latent_attn(&a, stream);
     }

@@ -78,15 +78,17 @@ __global__ __launch_bounds__(256) void latent_attn_row_kernel(const i64h_latent_
     for (int d = lane; d < D; d += 64) sq[d] = q[d] * p.scale;
     __syncthreads();
     const int j0 = p.window > 0 ? max(0, pos - p.window + 1) : 0;
+    // the visible keys in order: the kept first positions in front of the window, then j0 .. pos
+    const int kept = p.window > 0 ? min(p.keep_first, j0) : 0, total = kept + pos - j0 + 1;
     const int32_t* bt = p.block_table + (int64_t)slot * p.max_blocks_per_seq;
     // the sink: one more score (a learned one per head, or zero) that counts in the denominator and carries no value
     float m = p.sink ? (p.sink_w ? p.sink_w[h] : 0.0f) : -INFINITY, l = p.sink ? 1.0f : 0.0f, acc[LT_MAXC];
 #pragma unroll
     for (int i = 0; i < LT_MAXC; ++i) acc[i] = 0.0f;
-    for (int jb = j0; jb <= pos; jb += 64) {
-        const int j = jb + lane;
-        const bool valid = j <= pos;
-        const int jj = valid ? j : pos;
+    for (int ib = 0; ib < total; ib += 64) {
+        const int i = ib + lane;
+        const bool valid = i < total;
+        const int jj = valid ? (i < kept ? i : j0 + i - kept) : pos;
         const int64_t rj = (int64_t)bt[jj / p.block_size] * p.block_size + jj % p.block_size;
         float s = 0.0f;
         if (p.cache_dtype == 0) {
@@ -126,7 +128,7 @@ __global__ __launch_bounds__(256) void latent_attn_row_kernel(const i64h_latent_
         sp[lane] = pj;
         srow[lane] = (int)rj;
         __syncthreads();
-        const int cnt = min(64, pos - jb + 1);
+        const int cnt = min(64, total - ib);
 #pragma unroll
         for (int i = 0; i < LT_MAXC; ++i) acc[i] *= alpha;
         for (int k = 0; k < cnt; ++k) {
@@ -180,6 +182,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(2, KD > 4 ? 
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int lane = threadIdx.x, n = lane & 15, kg = lane >> 4;
     const int r = p.kv_rank, D = r + p.rot_dim, H = p.heads, bs = p.block_size, win = p.window;
+    const int keep = p.chunk <= 0 && win > 0 ? p.keep_first : 0;
     uint16_t* Vt = (uint16_t*)smem;           // [r][LT_VLD]
     uint16_t* Ph = Vt + r * LT_VLD;           // [16][LT_VLD]
     uint16_t* Pl = Ph + 16 * LT_VLD;
@@ -265,7 +268,10 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(2, KD > 4 ? 
             lo = min(lo, p.chunk > 0 ? (pp / p.chunk) * p.chunk : (win > 0 ? max(0, pp - win + 1) : 0));
         }
         const int32_t* bt = p.block_table + (int64_t)sl * p.max_blocks_per_seq;
-        for (int kb = (lo & ~31) + 32 * split; kb <= hi; kb += 32 * splits) {
+        // tiles of 32 keys: those of the kept first positions that lie in front of the window's first tile, then the window's
+        const int t0 = lo >> 5, kt = min((keep + 31) >> 5, t0), tiles = kt + (hi >> 5) - t0 + 1;
+        for (int tile = split; tile < tiles; tile += splits) {
+            const int kb = (tile < kt ? tile : t0 + tile - kt) * 32;
             if (lane < 32) {
                 const int jc = min(kb + lane, hi);
                 rowoff[lane] = bt[jc / bs] * bs + jc % bs;
@@ -308,7 +314,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(2, KD > 4 ? 
 #pragma unroll
                 for (int b = 0; b < 2; ++b) {
                     const int j = kb + 16 * b + n;
-                    const bool vis = in_run && j <= pr && j >= lor[g];
+                    const bool vis = in_run && j <= pr && (j >= lor[g] || j < keep);
                     float sc = S[b][g] * ksc[b];
                     if (capl > 0.0f) sc = capl * tanhf(sc / capl);
                     if (p.bias) sc += 1.4426950408889634f * p.bias[(int64_t)min(max(pr - j, 0), p.bias_rows - 1) * H + hrow[g]];
@@ -384,6 +390,7 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int lane = threadIdx.x, n = lane & 15, kg = lane >> 4;
     const int r = p.kv_rank, D = r + p.rot_dim, H = p.heads, bs = p.block_size, win = p.window;
+    const int keep = p.chunk <= 0 && win > 0 ? p.keep_first : 0;
     uint16_t* Vt = (uint16_t*)smem;
     uint16_t* Ph = Vt + r * LT_VLD;
     uint16_t* Pl = Ph + 16 * LT_VLD;
@@ -402,8 +409,9 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
     const int lo = p.chunk > 0 ? (pos / p.chunk) * p.chunk : (win > 0 ? max(0, pos - win + 1) : 0), hi = pos;
     const int32_t* bt = p.block_table + (int64_t)slot * p.max_blocks_per_seq;
     const uint16_t* cache = (const uint16_t*)p.cache;
-    const int step = 32 * splits;
-    const int kb0 = (lo & ~31) + 32 * split;
+    // tiles of 32 keys, dealt to the splits in turn: those of the kept first positions in front of the window's first tile, then the window's
+    const int t0 = lo >> 5, kt = min((keep + 31) >> 5, t0), tiles = kt + (hi >> 5) - t0 + 1;
+    auto first_key = [&](int tile) { return (tile < kt ? tile : t0 + tile - kt) * 32; };
     auto lookup = [&](int kb, int buf) {
         if (lane < 32) {
             const int jc = min(kb + lane, hi);
@@ -422,9 +430,9 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
             }
         }
     };
-    if (kb0 <= hi) {
-        lookup(kb0, 0);
-        if (kb0 + step <= hi) lookup(kb0 + step, 1);
+    if (split < tiles) {
+        lookup(first_key(split), 0);
+        if (split + splits < tiles) lookup(first_key(split + splits), 1);
         __builtin_amdgcn_wave_barrier();
         request(0);
     }
@@ -465,8 +473,8 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
         lrow[g] = sink ? 1.0f : 0.0f;
     }
     int it = 0;
-    for (int kb = kb0; kb <= hi; kb += step, ++it) {
-        const int cur = it & 1;
+    for (int tile = split; tile < tiles; tile += splits, ++it) {
+        const int cur = it & 1, kb = first_key(tile);
         lt_v4f S[2];
         float ksc[2] = {1.0f, 1.0f};
         if (p.kscale) {
@@ -494,7 +502,7 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
             }
         }
         __builtin_amdgcn_wave_barrier();
-        if (kb + step <= hi) request(cur ^ 1);          // the next tile travels under this tile's softmax and second product
+        if (tile + splits < tiles) request(cur ^ 1);          // the next tile travels under this tile's softmax and second product
         float al[4];
 #pragma unroll
         for (int g = 0; g < 4; ++g) {
@@ -506,7 +514,7 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
                 float sc = S[b][g] * ksc[b];
                 if (capl > 0.0f) sc = capl * tanhf(sc / capl);
                 if (p.bias) sc += 1.4426950408889634f * p.bias[(int64_t)min(max(pos - j, 0), p.bias_rows - 1) * H + hrow[g]];
-                sv[b] = (j <= pos && j >= lo) ? sc : -INFINITY;
+                sv[b] = (j <= pos && (j >= lo || j < keep)) ? sc : -INFINITY;
             }
             const float mx = row16_max(fmaxf(sv[0], sv[1]));
             const float mn = fmaxf(mrow[g], mx);
@@ -536,7 +544,7 @@ __global__ __launch_bounds__(64) void latent_attn_mfma_decode_kernel(const i64h_
             }
         }
         __builtin_amdgcn_wave_barrier();
-        if (kb + 2 * step <= hi) lookup(kb + 2 * step, cur);   // rows of the tile after next, into the buffer this tile is done with
+        if (tile + 2 * splits < tiles) lookup(first_key(tile + 2 * splits), cur);   // rows of the tile after next, into the buffer this tile is done with
     }
     if (splits > 1) {
         float* w = p.workspace + ((int64_t)task * splits + split) * 16 * (r + 2);
@@ -641,6 +649,7 @@ int i64h_latent_attn(const i64h_latent_attn_args* dp, void* stream) {
     I64H_CHECK_ARG(mfma_ok || (d.kv_groups <= 1 && d.row_stride <= 0 && d.chunk <= 0 && !d.kscale && !d.bias),
                    "latent_attn: key heads, chunks, key scales and bias are built for the matrix-core form only");
     I64H_CHECK_ARG(!d.sink_w || d.sink, "latent_attn: sink scores without the sink");
+    I64H_CHECK_ARG(d.keep_first >= 0, "latent_attn: %d kept positions", d.keep_first);
     if (d.mode != 1 && mfma_ok) {
         const int row_tiles = d.mode == 3;
         const int G = d.kv_groups > 1 ? d.kv_groups : 1;

@@ -21,17 +21,15 @@ everything in 32 bits.  torch holds memory and streams; every arithmetic step is
 I64MoEModel's, so the same engine, scheduler and decoders drive it."""
 from __future__ import annotations
 
-import os
 from typing import Dict, List, Optional
 
 import torch
 
 from . import ops_dense as D
 from .config import FukatarConfig
+from .hybrid_runner import HybridRunner
 from .model import attention_segments
 from .paged_cache import HybridCache
-
-UNIT_EPS = 1e-6     # inside the root of the delta rule's unit vectors: a constant of the design, not of a checkpoint
 
 
 class _StepBuffers:
@@ -53,29 +51,13 @@ class _StepBuffers:
         self.attn_ws: Dict[tuple, torch.Tensor] = {}
 
 
-class FukatarModel:
-    MAX_BUFFER_SETS = int(os.environ.get("I64H_MAX_BUFFER_SETS", "8"))
-    ATTN_MAX_SEGMENTS = 4
-    ATTN_WAVES = {64: 3072, 128: 2048, 256: 1024}     # waves a decode-sized attention launch aims at, by the width of a key head's cached part
+class FukatarModel(HybridRunner):
+    BUFFERS = _StepBuffers
 
     def __init__(self, cfg: FukatarConfig, weights: Dict[str, torch.Tensor], device="cuda:0", dtype: str = "bfloat16", max_seqs: int = 4,
                  num_kv_blocks: int = 256, kv_block: int = 16, cache_dtype: Optional[torch.dtype] = None):
-        if dtype not in ("bfloat16", "float32"):
-            raise ValueError(f"dtype {dtype}: bfloat16 or float32")
-        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
-        self.exact = dtype == "float32"
-        dev = self.device
-        bf = lambda t: t.to(device=dev, dtype=torch.bfloat16).contiguous()
-        f = lambda t: t.to(device=dev, dtype=torch.float32).contiguous()
-        W = cfg.width
-
-        def need(name, shape):
-            if name not in weights:
-                raise KeyError(f"tensor '{name}' is missing")
-            if tuple(weights[name].shape) != tuple(shape):
-                raise ValueError(f"'{name}': shape {tuple(weights[name].shape)}, config says {tuple(shape)}")
-            return weights[name]
-
+        self._init_runner(cfg, device, dtype)
+        dev, bf, f, need, W = self.device, self._bf, self._f, self._reader(weights), cfg.width
         self.embed, self.head = bf(need("embed", (cfg.vocab, W))), bf(need("head", (cfg.vocab, W)))
         self.bigram = bf(need("bigram", (cfg.bigram.buckets + 1, W))) if cfg.bigram is not None else None
         self.final_norm = f(need("final.norm", (W,)))
@@ -104,20 +86,8 @@ class FukatarModel:
             cache_dtype = torch.float32 if self.exact else torch.bfloat16
         self.kv = HybridCache(specs, num_kv_blocks, max_seqs, dev, dtype=cache_dtype, block=kv_block,
                               seq_state={"prev_token": ((), torch.int64)} if cfg.bigram is not None else None)
-        self._bufs: Dict[tuple, _StepBuffers] = {}
-        self._pinned: set = set()
-        self._arange: Dict[int, torch.Tensor] = {}
 
     # ---- load-time layout work: one weight for everything that reads the mixer's input; small vectors and tables in fp32 ----
-    def _rotary(self, a, d: dict, f) -> None:
-        """Frequency tables of a rotated attention: evaluated in 64 bits on the host, rounded once to fp32."""
-        d["inv_freq"], d["rot_mult"], d["v_freq"] = None, 1.0, None
-        if a.rot is not None and a.rot.dims:
-            fr, d["rot_mult"] = a.rot.frequencies()
-            d["inv_freq"] = f(torch.tensor(fr, dtype=torch.float64))
-        if a.rot is not None and a.rotate_values:
-            d["v_freq"] = f(torch.tensor([a.rot.base ** (-2.0 * i / a.vdim) for i in range(a.vdim // 2)], dtype=torch.float64))
-
     def _load_layer(self, i: int, L, need, bf, f) -> dict:
         W, p = self.cfg.width, f"l{i}."
         d = dict(type=L.type, m=L.mixer, mlp=L.mlp)
@@ -148,7 +118,7 @@ class FukatarModel:
                 d["g_off"], n_in = n_in, n_in + a.heads
             d["q_norm"] = f(need(ap + "q.norm", (nq,))) if a.qk_norm == "row" else None
             d["k_norm"] = f(need(ap + "k.norm", (nk,))) if a.qk_norm == "row" else None
-            self._rotary(a, d, f)
+            self._rotary_tables(a, d)
             d["o"] = bf(need(ap + "o", (W, a.heads * a.vdim)))
             d["n_a"], d["n_b"] = a.heads * (a.vdim + a.dim), a.heads * a.vdim
             if L.type == "parallel":
@@ -171,96 +141,7 @@ class FukatarModel:
             d["up"], d["down"] = bf(need(p + "mlp.up", (L.mlp.ff, W))), bf(need(p + "mlp.down", (W, L.mlp.ff)))
         return d
 
-    # ---- step buffers (same policy as the other runners: the most recent row counts are kept, pinned sets stay for captured graphs) ----
-    def buffers(self, n: int, m: int) -> _StepBuffers:
-        key = (n, m)
-        B = self._bufs.pop(key, None)
-        if B is None:
-            B = _StepBuffers(self, n, m)
-        self._bufs[key] = B
-        loose = [k for k in self._bufs if k not in self._pinned and k != key]
-        for k in loose[:max(0, len(loose) + 1 - self.MAX_BUFFER_SETS)]:
-            del self._bufs[k]
-        return B
-
-    def pin_buffers(self, n: int, m: int) -> None:
-        self.buffers(n, m)
-        self._pinned.add((n, m))
-
-    def check_sync(self, force: bool = True):
-        """No launch of this runner waits on a grid barrier: nothing to read back."""
-
-    def snapshot_state(self):
-        """The per-sequence state, for a caller that runs a step which must not count (a warm-up before a graph capture)."""
-        return self.kv.snapshot()
-
-    def restore_state(self, held) -> None:
-        self.kv.restore(held)
-
-    def _runs(self, n: int, slot_ids: torch.Tensor, tokens_per_seq, rows_are_slots: bool):
-        """First rows of the runs of consecutive rows of one sequence, int32 [runs + 1] on the device, and their number."""
-        if rows_are_slots:
-            t = self._arange.get(n)
-            if t is None:
-                t = self._arange[n] = torch.arange(n + 1, dtype=torch.int32, device=self.device)
-            return t, n
-        if tokens_per_seq is None:      # (a caller that does not say how its rows are grouped: read it off the slot ids)
-            s = slot_ids.tolist()
-            tokens_per_seq, k = [], 0
-            for j in range(1, n + 1):
-                if j == n or s[j] != s[j - 1]:
-                    tokens_per_seq.append(j - k)
-                    k = j
-        starts = [0]
-        for t in tokens_per_seq:
-            if int(t) > 0:
-                starts.append(starts[-1] + int(t))
-        if starts[-1] != n:
-            raise ValueError(f"tokens_per_seq adds up to {starts[-1]} rows, the step has {n}")
-        return torch.tensor(starts, dtype=torch.int32).to(self.device), len(starts) - 1
-
-    def _splits(self, B, rows: int, heads: int, kv_heads: int, vals: int, width: int, ctx_hint: int, floats):
-        """How many waves share a decode row's keys (about ATTN_WAVES waves in the launch, a wave keeping at least two tiles of 32 keys),
-        and the workspace their partial results meet in."""
-        tasks = rows * kv_heads * ((heads // kv_heads + 15) // 16)
-        waves = self.ATTN_WAVES[64 if width <= 64 else (128 if width <= 128 else 256)]
-        splits = max(1, min(waves // max(1, tasks), ctx_hint // 64, 64))
-        if splits <= 1:
-            return 1, None
-        key = (rows, heads, kv_heads, vals, splits)
-        ws = B.attn_ws.get(key)
-        if ws is None:
-            ws = B.attn_ws[key] = torch.empty(max(1, floats(splits)), dtype=torch.float32, device=self.device)
-        return splits, ws
-
     # ---- mixers: the input is B.h; the result lands in B.y (and B.y2 for the second of two side-by-side mixers) ----
-    def _rotary_attention(self, B, d, a, P, l, n, positions, slot_ids, kvc, runs, ctx_hint, out) -> None:
-        """Rotated attention on the projection rows P (already computed): prep -> paged [values | keys] rows and query rows, attention,
-        the turn back and the head gate, out-projection into `out`."""
-        ex = self.exact
-        gs = a.vdim + a.dim
-        Q = B.a[: n * a.heads * gs].view(n, a.heads * gs)
-        rows = kvc.rows[l]
-        D.rot_prep(P, q_off=d["q_off"], k_off=d["k_off"], v_off=d["v_off"], heads=a.heads, kv_heads=a.kv_heads, dim=a.dim, vdim=a.vdim, q_norm_w=d["q_norm"],
-                   k_norm_w=d["k_norm"], eps=self.cfg.norm_eps, rot_dims=a.rot.dims if a.rot is not None else 0, interleaved=a.interleaved,
-                   inv_freq=d["inv_freq"], rot_mult=d["rot_mult"], head_norm=a.qk_norm == "head", v_freq=d["v_freq"], scale=a.scale, positions=positions,
-                   slot_ids=slot_ids, block_table=kvc.block_table, cache=rows, q=Q, n=n)
-        O = B.b[: n * a.heads * a.vdim].view(n, a.heads * a.vdim)
-        # runs of rows that are one per sequence (a wave takes a token's query heads of one key head, the keys dealt to several waves) and
-        # runs of prompt portions (a wave takes 16 consecutive rows of one head), each one launch
-        for r0, r1, one_per_seq in runs:
-            splits, ws = 1, None
-            if one_per_seq and not ex:
-                splits, ws = self._splits(B, r1 - r0, a.heads, a.kv_heads, a.vdim, gs, ctx_hint,
-                                          lambda s: D.kattn_workspace_floats(r1 - r0, a.heads, a.kv_heads, a.vdim, s))
-            D.kattn(Q[r0:r1], rows, None, kvc.block_table, slot_ids[r0:r1], positions[r0:r1], chunk=0, bias=None, sink=False, heads=a.heads,
-                    kv_heads=a.kv_heads, dim=a.dim, vdim=a.vdim, out=O[r0:r1], n=r1 - r0, mode=2 if one_per_seq else 3, splits=splits, workspace=ws,
-                    softcap=a.softcap)
-        if d["v_freq"] is not None or a.head_gate:
-            D.rot_post(O, heads=a.heads, vdim=a.vdim, interleaved=a.interleaved, v_freq=d["v_freq"], positions=positions,
-                       gate=P if a.head_gate else None, gate_off=d.get("g_off", 0), ldg=d["n_in"], n=n)
-        D.linear(O, d["o"], out, exact=ex)
-
     def _attention(self, B, d, l, n, positions, slot_ids, kvc, runs, ctx_hint) -> None:
         P = B.p[: n * d["n_in"]].view(n, d["n_in"])
         D.linear(B.h, d["w_in"], P, exact=self.exact)
@@ -290,24 +171,11 @@ class FukatarModel:
         D.linear(og, d["o"], B.y, m=n, k=H * m.vdim, lda=H * m.vdim, exact=ex)
 
     def _parallel(self, B, d, l, n, positions, slot_ids, kvc, seg, nseg, runs, ctx_hint, single) -> None:
-        a, r, ex = d["m"].left, d["m"].right, self.exact
-        N1 = d["n_in"]
-        P = B.p[: n * N1].view(n, N1)
-        D.linear(B.h, d["w_in"], P, exact=ex)
+        a, r = d["m"].left, d["m"].right
+        P = B.p[: n * d["n_in"]].view(n, d["n_in"])
+        D.linear(B.h, d["w_in"], P, exact=self.exact)
         self._rotary_attention(B, d, a, P, l, n, positions, slot_ids, kvc, runs, ctx_hint, B.y)
-        st = kvc.state[l]
-        C, rk, rv = r.conv_channels, r.kv_heads * r.dim, r.heads * r.vdim
-        X = B.a[: n * C].view(n, C)
-        D.causal_conv(P, off=d["r_off"], channels=C, w=d["conv_w"], bias=None, positions=positions, slot_ids=slot_ids, state=st.get("conv"), out=X, n=n,
-                      single_rows=single)
-        G = B.g[: n * 2 * r.heads].view(n, 2 * r.heads)
-        cols = dict(q_off=0, k_off=rk, v_off=2 * rk, heads=r.heads, kv_heads=r.kv_heads, dim=r.dim, vdim=r.vdim, n=n)
-        D.gdn_gates(X, G, P, b_off=d["rb_off"], a_off=d["ra_off"], a_log=d["A_log"], dt_bias=d["dt_bias"], unit_eps=UNIT_EPS, q_scale=r.dim ** -0.5, **cols)
-        R = B.b[: n * rv].view(n, rv)
-        D.gdn_scan(X, G, seg_start=seg, nseg=nseg, positions=positions, slot_ids=slot_ids, state=st["gdn"], out=R, **cols)
-        Rn = B.c[: n * rv].view(n, rv)
-        D.gate_norm(R, d["r_norm"], Rn, groups=r.heads, eps=self.cfg.norm_eps, z=P, z_off=d["rg_off"], ldz=N1, n=n, gate_after=True, width=rv)
-        D.linear(Rn, d["o_right"], B.y2, exact=ex)
+        self._gated_delta(B, d, r, P, l, n, positions, slot_ids, kvc, seg, nseg, single, B.y2)
 
     @torch.no_grad()
     def forward(self, token_ids: torch.Tensor, positions: torch.Tensor, slot_ids: torch.Tensor, ctx_len: Optional[torch.Tensor] = None,

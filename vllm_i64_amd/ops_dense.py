@@ -12,7 +12,8 @@ from ._lib import call_dense, ptr
 from .ops import _chk, _stream
 
 EPI_STORE, EPI_GELU_MUL, EPI_MUL_SIGMOID, EPI_SOFTCAP, EPI_GELU_ERF, EPI_SCALE, EPI_SILU_MUL, EPI_XIELU, EPI_RELU_SQ = 0, 1, 2, 3, 4, 5, 6, 7, 8
-_DUAL = (EPI_GELU_MUL, EPI_SILU_MUL)
+EPI_CLAMP_GLU, EPI_ADD, EPI_DECAY = 9, 10, 11
+_DUAL = (EPI_GELU_MUL, EPI_SILU_MUL, EPI_CLAMP_GLU)
 CACHE_DTYPE_CODE = {torch.float32: 0, torch.bfloat16: 2}
 
 
@@ -27,7 +28,7 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
            bias: Optional[torch.Tensor] = None, bias_batch: int = 0, scale: float = 1.0, act_a: float = 0.0, act_b: float = 0.0,
            group_off: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out[b][:, c_off + b * c_batch : + n] = epilogue(a[b][rows, a_off + b * a_batch : + k] @ w[b]^T): see i64h_linear.  a, out and e are
-    fp32 matrices addressed by (column offset, row stride); w is bf16 [n, k] (EPI_GELU_MUL / EPI_SILU_MUL: [2n, k], gate rows first), or a
+    fp32 matrices addressed by (column offset, row stride; e with lde = 0 is one row for all); w is bf16 [n, k] (the gate / up epilogues: [2n, k], gate rows first), or a
     stack [batch, n, k] with w_batch = n * k.  bias fp32 [n] (per batch: bias_batch apart) is added before the epilogue.  group_off int32
     [batch + 1] on the device: batch b takes the rows [group_off[b], group_off[b + 1]) of a_rows (or a) and out; m is then the most rows a
     batch may have, and a_rows / a / out must hold group_off[batch] rows (the caller's business: the counts stay on the device)."""
@@ -194,13 +195,14 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
                  y2n_w: Optional[torch.Tensor] = None, y_eps: float = 0.0, mix: Optional[torch.Tensor] = None, out_w: Optional[torch.Tensor] = None,
                  in_w: Optional[torch.Tensor] = None, norm_w: Optional[torch.Tensor] = None, eps: float = 0.0, h: Optional[torch.Tensor] = None,
                  rows: Optional[torch.Tensor] = None, post_w: Optional[torch.Tensor] = None, post_center: bool = False,
-                 h_center: bool = False) -> Optional[torch.Tensor]:
+                 h_center: bool = False, norm_b: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """See i64h_streams_step.  streams fp32 [S, n, W], updated in place when y is given; h fp32 [n, W] (or [rows, W]).  post_w fp32 [W]: a
-    norm over the result as a whole (centred with post_center) before it is added; h_center: the read's norm is centred."""
+    norm over the result as a whole (centred with post_center) before it is added; h_center: the read's norm is centred; norm_b: added behind
+    the read's norm weight.  y2 without norm weights is simply added to y."""
     _chk(streams, torch.float32, "streams")
     S, n, W = streams.shape
     for t, name in ((y, "y"), (y2, "y2"), (yn_w, "yn_w"), (y2n_w, "y2n_w"), (mix, "mix"), (out_w, "out_w"), (in_w, "in_w"), (norm_w, "norm_w"), (h, "h"),
-                    (post_w, "post_w")):
+                    (post_w, "post_w"), (norm_b, "norm_b")):
         if t is not None:
             _chk(t, torch.float32, name)
     for t, name in ((y, "y"), (y2, "y2")):
@@ -210,6 +212,8 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
         raise _lib.I64HError("streams_step: stream weights do not fit the number of streams")
     if (yn_w is not None and yn_w.numel() != W) or (y2n_w is not None and y2n_w.numel() != W) or (post_w is not None and post_w.numel() != W):
         raise _lib.I64HError("streams_step: result norm weights are not [W]")
+    if norm_b is not None and norm_b.numel() != W:
+        raise _lib.I64HError("streams_step: the norm's offsets are not [W]")
     m_rows = n
     if rows is not None:
         _chk(rows, torch.int32, "rows")
@@ -218,7 +222,8 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
         raise _lib.I64HError("streams_step: h smaller than the rows it receives")
     d = _lib.Streams(streams=ptr(streams), S=S, n=n, W=W, y=ptr(y), ldy=W, y2=ptr(y2), ldy2=W, yn_w=ptr(yn_w), y2n_w=ptr(y2n_w), y_eps=float(y_eps),
                      mix=ptr(mix), out_w=ptr(out_w), in_w=ptr(in_w), norm_w=ptr(norm_w), norm_w_len=norm_w.numel() if norm_w is not None else 0,
-                     eps=float(eps), h=ptr(h), rows=ptr(rows), m_rows=m_rows, post_w=ptr(post_w), post_center=int(bool(post_center)), h_center=int(bool(h_center)))
+                     eps=float(eps), h=ptr(h), rows=ptr(rows), m_rows=m_rows, post_w=ptr(post_w), post_center=int(bool(post_center)), h_center=int(bool(h_center)),
+                     norm_b=ptr(norm_b))
     call_dense("i64h_streams_step", _ref(d), _stream())
     return h
 
@@ -271,9 +276,9 @@ def ssm_scan(xbc: torch.Tensor, dt: torch.Tensor, *, dt_off: int, lddt: int, dt_
 
 
 def gate_norm(y: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, groups: int, eps: float, z: Optional[torch.Tensor] = None, z_off: int = 0,
-              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None) -> torch.Tensor:
+              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None, sigmoid: bool = False) -> torch.Tensor:
     """out = rms_groups(y * silu(z)) * w: see i64h_gate_norm.  y, out fp32 [n, width]; z the columns [z_off, + width) of a matrix of row stride ldz.
-    gate_after: out = rms_groups(y) * w * silu(z).  width (default: w's length): the row's width, w then repeats over it."""
+    gate_after: out = rms_groups(y) * w * silu(z).  sigmoid: the gate is sigmoid(z).  width (default: w's length): the row's width, w then repeats over it."""
     _chk(y, torch.float32, "y"), _chk(w, torch.float32, "w"), _chk(out, torch.float32, "out")
     w_len = w.numel()
     width = int(width if width is not None else w_len)
@@ -287,7 +292,7 @@ def gate_norm(y: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, groups: in
         if z.numel() < (rows - 1) * ldz + z_off + width:
             raise _lib.I64HError("gate_norm: gate smaller than the launch reads")
     d = _lib.GateNorm(y=ptr(y), ldy=width, z=(ptr(z) + 4 * z_off) if z is not None else 0, ldz=ldz, w=ptr(w), width=width, groups=groups, eps=float(eps),
-                      out=ptr(out), ldo=width, n=rows, gate_after=int(bool(gate_after)), w_len=w_len if w_len != width else 0)
+                      out=ptr(out), ldo=width, n=rows, gate_after=int(bool(gate_after)), w_len=w_len if w_len != width else 0, gate_act=int(bool(sigmoid)))
     call_dense("i64h_gate_norm", _ref(d), _stream())
     return out
 
@@ -331,9 +336,11 @@ def kattn_prep(p: torch.Tensor, *, q_off: int, k_off: int, heads: int, kv_heads:
 
 def kattn(q: torch.Tensor, cache: torch.Tensor, kscale: torch.Tensor, block_table: torch.Tensor, slot_ids: torch.Tensor, positions: torch.Tensor, *,
           chunk: int, bias: Optional[torch.Tensor], sink: bool, heads: int, kv_heads: int, dim: int, out: torch.Tensor, n: Optional[int] = None,
-          mode: int = 0, splits: int = 1, workspace: Optional[torch.Tensor] = None, vdim: int = 0, softcap: float = 0.0) -> torch.Tensor:
+          mode: int = 0, splits: int = 1, workspace: Optional[torch.Tensor] = None, vdim: int = 0, softcap: float = 0.0,
+          window: int = 0, keep_first: int = 0, sink_w: Optional[torch.Tensor] = None) -> torch.Tensor:
     """See i64h_kattn.  q, out fp32 [n, heads * dim]; bias fp32 [distances, heads].  vdim > 0: separate values - the cache rows are
-    [kv_heads, vdim + dim], q fp32 [n, heads, vdim + dim], out fp32 [n, heads * vdim], kscale may be None."""
+    [kv_heads, vdim + dim], q fp32 [n, heads, vdim + dim], out fp32 [n, heads * vdim], kscale may be None.  window > 0: the last `window`
+    positions and the first keep_first ones are seen.  sink_w fp32 [heads]: the sink's score per head."""
     _chk(q, torch.float32, "q"), _chk(out, torch.float32, "out"), _chk(cache, None, "cache")
     if kscale is not None or vdim <= 0:
         _chk(kscale, torch.float32, "kscale")
@@ -344,6 +351,10 @@ def kattn(q: torch.Tensor, cache: torch.Tensor, kscale: torch.Tensor, block_tabl
         _chk(bias, torch.float32, "bias")
         if bias.dim() != 2 or bias.shape[1] != heads:
             raise _lib.I64HError("kattn: bias is not [distances, heads]")
+    if sink_w is not None:
+        _chk(sink_w, torch.float32, "sink_w")
+        if sink_w.numel() != heads:
+            raise _lib.I64HError("kattn: the sink scores are not [heads]")
     gs, vals = (vdim + dim, vdim) if vdim > 0 else (dim, dim)
     if cache.shape[-1] != kv_heads * gs or (kscale is not None and kscale.numel() != cache.shape[0] * cache.shape[1]) or q.numel() < rows * heads * gs or \
             out.numel() < rows * heads * vals:
@@ -359,7 +370,7 @@ def kattn(q: torch.Tensor, cache: torch.Tensor, kscale: torch.Tensor, block_tabl
                    max_blocks_per_seq=block_table.shape[1], block_size=cache.shape[-2], slot_ids=ptr(slot_ids), positions=ptr(positions), chunk=int(chunk),
                    bias=ptr(bias), bias_rows=bias.shape[0] if bias is not None else 0, sink=int(bool(sink)), out=ptr(out), n=rows, heads=heads,
                    kv_heads=kv_heads, dim=dim, mode=int(mode), splits=int(splits) if splits > 1 else 1, workspace=ptr(workspace) if splits > 1 else 0,
-                   vdim=int(vdim), softcap=float(softcap))
+                   vdim=int(vdim), softcap=float(softcap), window=int(window), keep_first=int(keep_first), sink_w=ptr(sink_w))
     call_dense("i64h_kattn", _ref(d), _stream())
     return out
 
@@ -452,27 +463,35 @@ def _gdn_args(x: torch.Tensor, g: torch.Tensor, *, q_off: int, k_off: int, v_off
 
 
 def gdn_gates(x: torch.Tensor, g: torch.Tensor, raw: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int, kv_heads: int, dim: int, vdim: int,
-              b_off: int, a_off: int, a_log: torch.Tensor, dt_bias: torch.Tensor, unit_eps: float, q_scale: float, n: int) -> None:
+              b_off: int, a_off: int, a_log: Optional[torch.Tensor], dt_bias: Optional[torch.Tensor], unit_eps: float, q_scale: float, n: int) -> None:
     """See i64h_gdn_gates: unit-vector queries and keys in place on x fp32 [n, ldx]; g fp32 [n, 2 * heads] receives write strength and decay from
-    the columns b_off / a_off of raw fp32 [n, ldr]."""
-    _chk(raw, torch.float32, "raw"), _chk(a_log, torch.float32, "a_log"), _chk(dt_bias, torch.float32, "dt_bias")
-    if max(b_off, a_off) + heads > raw.shape[-1] or raw.numel() < n * raw.shape[-1] or min(a_log.numel(), dt_bias.numel()) < heads:
+    the columns b_off / a_off of raw fp32 [n, ldr] (a_off < 0: the write strength alone)."""
+    _chk(raw, torch.float32, "raw")
+    if a_off >= 0:
+        _chk(a_log, torch.float32, "a_log"), _chk(dt_bias, torch.float32, "dt_bias")
+    if max(b_off, a_off) + heads > raw.shape[-1] or raw.numel() < n * raw.shape[-1] or (a_off >= 0 and min(a_log.numel(), dt_bias.numel()) < heads):
         raise _lib.I64HError("gdn_gates: shapes do not fit the sizes")
     d = _gdn_args(x, g, q_off=q_off, k_off=k_off, v_off=v_off, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, n=n, R=ptr(raw), ldr=raw.shape[-1],
-                  b_off=b_off, a_off=a_off, A_log=ptr(a_log), dt_bias=ptr(dt_bias), unit_eps=float(unit_eps), q_scale=float(q_scale))
+                  b_off=b_off, a_off=a_off, A_log=ptr(a_log) if a_off >= 0 else 0, dt_bias=ptr(dt_bias) if a_off >= 0 else 0, unit_eps=float(unit_eps), q_scale=float(q_scale))
     call_dense("i64h_gdn_gates", _ref(d), _stream())
 
 
 def gdn_scan(x: torch.Tensor, g: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int, kv_heads: int, dim: int, vdim: int, seg_start: torch.Tensor,
-             nseg: int, positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n: int) -> torch.Tensor:
-    """See i64h_gdn_scan.  state fp32 [slots, heads, vdim, dim]; out fp32 [n, heads * vdim]."""
+             nseg: int, positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n: int,
+             f: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """See i64h_gdn_scan.  state fp32 [slots, heads, vdim, dim]; out fp32 [n, heads * vdim]; f fp32 [n, heads * dim]: a decay per key channel."""
+    if f is not None:
+        _chk(f, torch.float32, "f")
+        if f.shape[-1] < heads * dim or f.numel() < n * f.shape[-1]:
+            raise _lib.I64HError("gdn_scan: the decays are not [n, heads * dim]")
     _chk(state, torch.float32, "state"), _chk(out, torch.float32, "out")
     _chk(seg_start, torch.int32, "seg_start"), _chk(positions, torch.int32, "positions"), _chk(slot_ids, torch.int32, "slot_ids")
     _rows_ok("gdn_scan", n, positions, slot_ids)
     if tuple(state.shape[1:]) != (heads, vdim, dim) or out.numel() < n * heads * vdim or seg_start.numel() < nseg + 1:
         raise _lib.I64HError("gdn_scan: shapes do not fit the sizes")
     d = _gdn_args(x, g, q_off=q_off, k_off=k_off, v_off=v_off, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, n=n, seg_start=ptr(seg_start), nseg=nseg,
-                  positions=ptr(positions), slot_ids=ptr(slot_ids), state=ptr(state), out=ptr(out), ldo=heads * vdim)
+                  positions=ptr(positions), slot_ids=ptr(slot_ids), state=ptr(state), out=ptr(out), ldo=heads * vdim, F=ptr(f),
+                  ldf=f.shape[-1] if f is not None else 0)
     call_dense("i64h_gdn_scan", _ref(d), _stream())
     return out
 
@@ -513,16 +532,18 @@ def gla_scan(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int,
 
 
 def route_topk(logits: Optional[torch.Tensor], *, entries: int, correction: Optional[torch.Tensor], groups: int, keep: int, top: int, scale: float, idx: torch.Tensor,
-               wgt: torch.Tensor, n: Optional[int] = None, h: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None) -> None:
+               wgt: torch.Tensor, n: Optional[int] = None, h: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None,
+               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, gate_out: Optional[torch.Tensor] = None) -> None:
     """See i64h_route_topk.  logits fp32 [n, ld >= entries], or None with h fp32 [n, K] and w bf16 [entries, K]: the launch computes the
-    logits itself in 32 bits; idx int32 [n, top]; wgt fp32 [n, top]."""
+    logits itself in 32 bits; idx int32 [n, top]; wgt fp32 [n, top].  bias fp32 [entries]; gate_out fp32 [n]: w has one more row, whose
+    product's sigmoid it receives."""
     _chk(idx, torch.int32, "idx"), _chk(wgt, torch.float32, "wgt")
     if logits is None:
         if h is None or w is None:
             raise _lib.I64HError("route_topk: logits, or the router's input and weight")
         _chk(h, torch.float32, "h"), _chk(w, torch.bfloat16, "w")
         rows = int(n if n is not None else h.shape[0])
-        if w.dim() != 2 or w.shape[0] != entries or h.shape[-1] != w.shape[1] or h.numel() < rows * h.shape[-1]:
+        if w.dim() != 2 or w.shape[0] != entries + (1 if gate_out is not None else 0) or h.shape[-1] != w.shape[1] or h.numel() < rows * h.shape[-1]:
             raise _lib.I64HError("route_topk: the router's input and weight do not fit the sizes")
     else:
         _chk(logits, torch.float32, "logits")
@@ -533,11 +554,20 @@ def route_topk(logits: Optional[torch.Tensor], *, entries: int, correction: Opti
         _chk(correction, torch.float32, "correction")
         if correction.numel() != entries:
             raise _lib.I64HError("route_topk: the correction is not [entries]")
+    if bias is not None:
+        _chk(bias, torch.float32, "bias")
+        if bias.numel() != entries:
+            raise _lib.I64HError("route_topk: the bias is not [entries]")
+    if gate_out is not None:
+        _chk(gate_out, torch.float32, "gate_out")
+        if logits is not None or gate_out.numel() < rows:
+            raise _lib.I64HError("route_topk: the gate needs the router's weight and a value per row")
     if idx.numel() < rows * top or wgt.numel() < rows * top:
         raise _lib.I64HError("route_topk: shapes do not fit the sizes")
     d = _lib.Route(logits=ptr(logits), ld=logits.shape[-1] if logits is not None else 0, E=entries, correction=ptr(correction), groups=int(groups), keep=int(keep),
                    top=int(top), scale=float(scale), idx=ptr(idx), wgt=ptr(wgt), n=rows, h=ptr(h) if logits is None else 0,
-                   ldh=h.shape[-1] if logits is None else 0, W=ptr(w) if logits is None else 0, K=w.shape[1] if logits is None else 0)
+                   ldh=h.shape[-1] if logits is None else 0, W=ptr(w) if logits is None else 0, K=w.shape[1] if logits is None else 0,
+                   bias=ptr(bias), chosen_softmax=int(bool(chosen_softmax)), gate_out=ptr(gate_out))
     call_dense("i64h_route_topk", _ref(d), _stream())
 
 
@@ -552,15 +582,19 @@ def moe_plan(idx: torch.Tensor, *, n: int, top: int, experts: int, group_off: to
 
 
 def moe_combine(y: torch.Tensor, pair_row: torch.Tensor, wgt: torch.Tensor, h: torch.Tensor, shared: Optional[torch.Tensor], out: torch.Tensor, *,
-                n: int, top: int, width: int) -> torch.Tensor:
-    """See i64h_moe_combine.  y fp32 [pairs, width]; h, shared, out fp32 [n, width]."""
+                n: int, top: int, width: int, shared_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """See i64h_moe_combine.  y fp32 [pairs, width]; h, shared, out fp32 [n, width]; shared_gate fp32 [n]."""
+    if shared_gate is not None:
+        _chk(shared_gate, torch.float32, "shared_gate")
+        _rows_ok("moe_combine", n, shared_gate)
     _chk(y, torch.float32, "y"), _chk(pair_row, torch.int32, "pair_row"), _chk(wgt, torch.float32, "wgt"), _chk(h, torch.float32, "h"), _chk(out, torch.float32, "out")
     if shared is not None:
         _chk(shared, torch.float32, "shared")
     if min(h.numel(), out.numel(), shared.numel() if shared is not None else out.numel()) < n * width or min(pair_row.numel(), wgt.numel()) < n * top or \
             y.numel() < n * top * width:
         raise _lib.I64HError("moe_combine: shapes do not fit the sizes")
-    d = _lib.MoeCombine(Y=ptr(y), pair_row=ptr(pair_row), wgt=ptr(wgt), h=ptr(h), shared=ptr(shared), out=ptr(out), n=n, top=top, W=width)
+    d = _lib.MoeCombine(Y=ptr(y), pair_row=ptr(pair_row), wgt=ptr(wgt), h=ptr(h), shared=ptr(shared), out=ptr(out), n=n, top=top, W=width,
+                        shared_gate=ptr(shared_gate))
     call_dense("i64h_moe_combine", _ref(d), _stream())
     return out
 

@@ -78,6 +78,25 @@ def _load_fukatar(config: dict, tensors, *, device, dtype, max_seqs, max_tokens,
     return FukatarModel(cfg, tensors, device=device, dtype=dtype, max_seqs=max_seqs, num_kv_blocks=blocks, kv_block=kv_block)
 
 
+def _load_pukatar(config: dict, tensors, *, device, dtype, max_seqs, max_tokens, kv_block=16, **_):
+    from .config import PukatarConfig
+    from .pukatar import PukatarModel
+    config = dict(config)
+    for key, axis in (("vocab", 0), ("width", 1)):      # sizes that the file may leave to the tensors' shapes
+        if key not in config and "embed" in tensors:
+            config[key] = int(tensors["embed"].shape[axis])
+    layers = []
+    for i, l in enumerate(config.get("layers") or []):     # (the convolution's taps likewise)
+        name = f"l{i}.mix.q.conv"
+        if l.get("type") == "channel_delta" and "conv" not in (l.get("mixer") or {"conv": 0}) and name in tensors:
+            l = dict(l, mixer=dict(l["mixer"], conv=int(tensors[name].shape[1])))
+        layers.append(l)
+    config["layers"] = layers
+    cfg = PukatarConfig.from_dict(config)
+    blocks = max(1, (int(max_tokens) + kv_block - 1) // kv_block)
+    return PukatarModel(cfg, tensors, device=device, dtype=dtype, max_seqs=max_seqs, num_kv_blocks=blocks, kv_block=kv_block)
+
+
 def _load_complexity_deep(config: dict, tensors, *, device, dtype, max_seqs, max_tokens, quant="int8", **_):
     import torch
     from .checkpoint import config_from_dict, native_to_weights
@@ -92,6 +111,7 @@ register("Morilorn", _load_morilorn)
 register("Dogalorn", _load_dogalorn)
 register("Zabutar", _load_zabutar)
 register("Fukatar", _load_fukatar)
+register("Pukatar", _load_pukatar)
 register("complexity-deep", _load_complexity_deep)
 register("ComplexityDeepModel", _load_complexity_deep)
 

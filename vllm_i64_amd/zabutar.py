@@ -21,7 +21,6 @@ interface is I64MoEModel's, so the same engine, scheduler and decoders drive it.
 from __future__ import annotations
 
 import math
-import os
 from typing import Dict, List, Optional
 
 import torch
@@ -29,6 +28,7 @@ import torch
 from . import ops_dense as D
 from .config import ZabutarConfig
 from .dogalorn import distance_bias_table
+from .hybrid_runner import HybridRunner
 from .model import attention_segments
 from .paged_cache import HybridCache
 
@@ -40,7 +40,6 @@ def _softplus(x: float) -> float:
 class _StepBuffers:
     def __init__(self, model: "ZabutarModel", n: int, m: int):
         f32 = dict(dtype=torch.float32, device=model.device)
-        i32 = dict(dtype=torch.int32, device=model.device)
         W = model.cfg.width
         self.streams = torch.empty(1, n, W, **f32)              # the residual (one stream of the multi-stream kernel)
         self.h = torch.empty(n, W, **f32)                       # the normed input of the current sublayer
@@ -51,42 +50,19 @@ class _StepBuffers:
         self.a = torch.empty(n * model.max_a, **f32)            # queries / recurrence output
         self.b = torch.empty(n * model.max_a, **f32)            # attention output / normed recurrence output
         self.act = torch.empty(n * max(model.max_act, 1), **f32)
-        self.sact = torch.empty(n * max(model.max_shared, 1), **f32)
-        t = model.max_top
-        self.ey = torch.empty(n * t, W, **f32) if t else None   # the chosen experts' outputs, grouped by expert
-        self.idx = torch.empty(n * max(t, 1), **i32)
-        self.wgt = torch.empty(n * max(t, 1), **f32)
-        self.pair_token = torch.empty(n * max(t, 1), **i32)
-        self.pair_row = torch.empty(n * max(t, 1), **i32)
-        self.group_off = torch.empty(model.max_experts + 1, **i32)
+        HybridRunner.moe_buffers(self, model, n)
         self.xf = torch.empty(m, W, **f32)
         self.logits = torch.empty(m, model.cfg.vocab, **f32)
         self.attn_ws: Dict[tuple, torch.Tensor] = {}
 
 
-class ZabutarModel:
-    MAX_BUFFER_SETS = int(os.environ.get("I64H_MAX_BUFFER_SETS", "8"))
-    ATTN_MAX_SEGMENTS = 4
-    ATTN_WAVES = {64: 3072, 128: 2048, 256: 1024}     # waves a decode-sized attention launch aims at, by the width of a key head's cached part
+class ZabutarModel(HybridRunner):
+    BUFFERS = _StepBuffers
 
     def __init__(self, cfg: ZabutarConfig, weights: Dict[str, torch.Tensor], device="cuda:0", dtype: str = "bfloat16", max_seqs: int = 4,
                  num_kv_blocks: int = 256, kv_block: int = 16, cache_dtype: Optional[torch.dtype] = None):
-        if dtype not in ("bfloat16", "float32"):
-            raise ValueError(f"dtype {dtype}: bfloat16 or float32")
-        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
-        self.exact = dtype == "float32"
-        dev = self.device
-        bf = lambda t: t.to(device=dev, dtype=torch.bfloat16).contiguous()
-        f = lambda t: t.to(device=dev, dtype=torch.float32).contiguous()
-        W = cfg.width
-
-        def need(name, shape):
-            if name not in weights:
-                raise KeyError(f"tensor '{name}' is missing")
-            if tuple(weights[name].shape) != tuple(shape):
-                raise ValueError(f"'{name}': shape {tuple(weights[name].shape)}, config says {tuple(shape)}")
-            return weights[name]
-
+        self._init_runner(cfg, device, dtype)
+        dev, bf, f, need, W = self.device, self._bf, self._f, self._reader(weights), cfg.width
         self._one_plus = lambda t: f(1.0 + t.to(torch.float32))      # norm weights are stored as distances from one
         self.embed, self.head = bf(need("embed", (cfg.vocab, W))), bf(need("head", (cfg.vocab, W)))
         self.pos = bf(need("pos", (cfg.max_positions, W)))
@@ -109,18 +85,10 @@ class ZabutarModel:
                 specs.append({"rows": m.kv_heads * (m.vdim + m.dim), "kscale": False, "state": state})
         self.max_proj = max(d["n_in"] for d in self.layers)
         self.max_a = max(d["n_a"] for d in self.layers)
-        moes = [l.mlp for l in cfg.layers if l.mlp is not None and l.mlp.kind == "moe"]
-        self.max_top = max([m.top for m in moes] or [0])
-        self.max_experts = max([m.experts for m in moes] or [0])
-        self.max_shared = max([m.shared_ff for m in moes] or [0])
-        self.max_act = max([l.mlp.ff for l in cfg.layers if l.mlp is not None and l.mlp.kind == "dense"] + [m.ff * m.top for m in moes] +
-                           [0])
+        self._moe_sizes([l.mlp for l in cfg.layers])
         if cache_dtype is None:
             cache_dtype = torch.float32 if self.exact else torch.bfloat16
         self.kv = HybridCache(specs, num_kv_blocks, max_seqs, dev, dtype=cache_dtype, block=kv_block, position_limit=cfg.max_positions)
-        self._bufs: Dict[tuple, _StepBuffers] = {}
-        self._pinned: set = set()
-        self._arange: Dict[int, torch.Tensor] = {}
 
     # ---- load-time layout work: one weight for everything that reads the sublayer input; small vectors in fp32 ----
     def _load_layer(self, i: int, L, weights, need, bf, f) -> dict:
@@ -161,64 +129,9 @@ class ZabutarModel:
             a, b = (float(v) for v in need(p + "mlp.act", (2,)).float())
             d["act_a"], d["act_b"] = _softplus(a), 0.5 + _softplus(b)
         elif ff is not None:
-            d["router"] = bf(need(p + "mlp.router", (ff.entries, W)))
+            self._load_moe(p + "mlp.", ff, need, d)
             d["correction"] = f(need(p + "mlp.correction", (ff.entries,)))
-            # per expert [gate rows; up rows], all experts stacked: one grouped launch for the pair, one for the way down
-            d["gate_up"] = bf(torch.stack([torch.cat([need(f"{p}mlp.e{e}.gate", (ff.ff, W)), need(f"{p}mlp.e{e}.up", (ff.ff, W))], 0) for e in range(ff.experts)]))
-            d["e_down"] = bf(torch.stack([need(f"{p}mlp.e{e}.down", (W, ff.ff)) for e in range(ff.experts)]))
-            if ff.shared_ff:
-                s = ff.shared_ff
-                d["s_gate_up"] = bf(torch.cat([need(p + "mlp.shared.gate", (s, W)), need(p + "mlp.shared.up", (s, W))], 0))
-                d["s_down"] = bf(need(p + "mlp.shared.down", (W, s)))
         return d
-
-    # ---- step buffers (same policy as the other runners: the most recent row counts are kept, pinned sets stay for captured graphs) ----
-    def buffers(self, n: int, m: int) -> _StepBuffers:
-        key = (n, m)
-        B = self._bufs.pop(key, None)
-        if B is None:
-            B = _StepBuffers(self, n, m)
-        self._bufs[key] = B
-        loose = [k for k in self._bufs if k not in self._pinned and k != key]
-        for k in loose[:max(0, len(loose) + 1 - self.MAX_BUFFER_SETS)]:
-            del self._bufs[k]
-        return B
-
-    def pin_buffers(self, n: int, m: int) -> None:
-        self.buffers(n, m)
-        self._pinned.add((n, m))
-
-    def check_sync(self, force: bool = True):
-        """No launch of this runner waits on a grid barrier: nothing to read back."""
-
-    def snapshot_state(self):
-        """The per-sequence recurrent state, for a caller that runs a step which must not count (a warm-up before a graph capture)."""
-        return self.kv.snapshot()
-
-    def restore_state(self, held) -> None:
-        self.kv.restore(held)
-
-    def _runs(self, n: int, slot_ids: torch.Tensor, tokens_per_seq, rows_are_slots: bool):
-        """First rows of the runs of consecutive rows of one sequence, int32 [runs + 1] on the device, and their number."""
-        if rows_are_slots:
-            t = self._arange.get(n)
-            if t is None:
-                t = self._arange[n] = torch.arange(n + 1, dtype=torch.int32, device=self.device)
-            return t, n
-        if tokens_per_seq is None:      # (a caller that does not say how its rows are grouped: read it off the slot ids)
-            s = slot_ids.tolist()
-            tokens_per_seq, k = [], 0
-            for j in range(1, n + 1):
-                if j == n or s[j] != s[j - 1]:
-                    tokens_per_seq.append(j - k)
-                    k = j
-        starts = [0]
-        for t in tokens_per_seq:
-            if int(t) > 0:
-                starts.append(starts[-1] + int(t))
-        if starts[-1] != n:
-            raise ValueError(f"tokens_per_seq adds up to {starts[-1]} rows, the step has {n}")
-        return torch.tensor(starts, dtype=torch.int32).to(self.device), len(starts) - 1
 
     # ---- mixers and feed-forwards: the sublayer input is B.hc; the result lands in B.y ----
     def _hgrn2(self, B, d, l, n, positions, slot_ids, kvc, seg, nseg) -> None:
@@ -244,22 +157,7 @@ class ZabutarModel:
         D.kv_prep(P, q_off=0, k_off=nq, v_off=nq + nk, heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, scale=m.scale, positions=positions,
                   slot_ids=slot_ids, block_table=kvc.block_table, cache=rows if m.kv_from is None else None, q=Q, n=n, block_size=kvc.block)
         O = B.b[: n * m.heads * m.vdim].view(n, m.heads * m.vdim)
-        # runs of rows that are one per sequence (a wave takes a token's query heads of one key head, the keys dealt to several waves) and
-        # runs of prompt portions (a wave takes 16 consecutive rows of one head), each one launch
-        for r0, r1, one_per_seq in runs:
-            splits, ws = 1, None
-            if one_per_seq and not ex:
-                tasks = (r1 - r0) * m.kv_heads * ((m.heads // m.kv_heads + 15) // 16)
-                waves = self.ATTN_WAVES[64 if gs <= 64 else (128 if gs <= 128 else 256)]
-                splits = max(1, min(waves // max(1, tasks), ctx_hint // 64, 64))
-                if splits > 1:
-                    key = (r1 - r0, m.heads, m.kv_heads, m.vdim, splits)
-                    ws = B.attn_ws.get(key)
-                    if ws is None:
-                        ws = B.attn_ws[key] = torch.empty(max(1, D.kattn_workspace_floats(r1 - r0, m.heads, m.kv_heads, m.vdim, splits)), dtype=torch.float32,
-                                                          device=self.device)
-            D.kattn(Q[r0:r1], rows, None, kvc.block_table, slot_ids[r0:r1], positions[r0:r1], chunk=0, bias=d["bias"], sink=False, heads=m.heads,
-                    kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, out=O[r0:r1], n=r1 - r0, mode=2 if one_per_seq else 3, splits=splits, workspace=ws)
+        self._kattn(B, m, Q, O, rows, kvc, slot_ids, positions, runs, ctx_hint, bias=d["bias"])
         D.linear(O, d["o"], B.y, exact=ex)
 
     def _dense_ff(self, B, d, n) -> None:
@@ -267,26 +165,6 @@ class ZabutarModel:
         act = B.act[: n * ff].view(n, ff)
         D.linear(B.hc, d["up"], act, exact=self.exact, bias=d["up_b"], epilogue=D.EPI_XIELU, act_a=d["act_a"], act_b=d["act_b"])
         D.linear(act, d["down"], B.y, exact=self.exact, bias=d["down_b"])
-
-    def _moe_ff(self, B, d, n, record=None, l=0) -> None:
-        f, ex, W = d["mlp"], self.exact, self.cfg.width
-        E, top = f.experts, f.top
-        # the router's products in 32 bits in both modes (a choice between experts is not rounding's to make), inside the choice's launch
-        D.route_topk(None, h=B.hc, w=d["router"], entries=f.entries, correction=d["correction"], groups=f.groups, keep=f.keep, top=top, scale=f.scale,
-                     idx=B.idx, wgt=B.wgt, n=n)
-        if record is not None:
-            record[f"l{l}.route"] = B.idx[: n * top].view(n, top).clone()
-        D.moe_plan(B.idx, n=n, top=top, experts=E, group_off=B.group_off, pair_token=B.pair_token, pair_row=B.pair_row)
-        # the (token, expert) pairs lie grouped by expert: one launch runs every expert over its own rows, the counts stay on the device
-        act = B.act[: n * top * f.ff].view(n * top, f.ff)
-        D.linear(B.hc, d["gate_up"], act, m=n, a_rows=B.pair_token, batch=E, w_batch=2 * f.ff * W, exact=ex, epilogue=D.EPI_SILU_MUL, group_off=B.group_off)
-        D.linear(act, d["e_down"], B.ey, m=n, batch=E, w_batch=W * f.ff, exact=ex, group_off=B.group_off)
-        shared = None
-        if f.shared_ff:
-            sact = B.sact[: n * f.shared_ff].view(n, f.shared_ff)
-            D.linear(B.hc, d["s_gate_up"], sact, exact=ex, epilogue=D.EPI_SILU_MUL)
-            shared = D.linear(sact, d["s_down"], B.y2, exact=ex)
-        D.moe_combine(B.ey, B.pair_row, B.wgt, B.hc, shared, B.y, n=n, top=top, width=W)
 
     @torch.no_grad()
     def forward(self, token_ids: torch.Tensor, positions: torch.Tensor, slot_ids: torch.Tensor, ctx_len: Optional[torch.Tensor] = None,
@@ -324,7 +202,7 @@ class ZabutarModel:
             if q == 2 and d["mlp"].kind == "dense":
                 self._dense_ff(B, d, n)
             elif q == 2:
-                self._moe_ff(B, d, n, record, l)
+                self._moe_ff(B, d, n, B.hc, B.y, B.y2, record, f"l{l}")
             elif d["type"] == "hgrn2":
                 self._hgrn2(B, d, l, n, positions, slot_ids, kvc, seg, nseg)
             else:
