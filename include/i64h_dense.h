@@ -538,6 +538,8 @@ typedef struct {
 } i64h_gdn_args;
 int i64h_gdn_gates(const i64h_gdn_args* d, void* stream);
 int i64h_gdn_scan(const i64h_gdn_args* d, void* stream);
+int i64h_set_gdn_scan_form(int32_t form); /* tuning / test knob: 0 (default) = by the runs' length; 1 = loads straight into registers; 2, 3, 4 = staged
+                                             through LDS with 1, 2, 4 value columns per lane (where 16-byte rows allow); same results bit for bit */
 
 /* ---- router: softmax scores, corrected choice, groups of neighbours, top-k ---------------------------------------------------------------------
  * Per row t of logits (fp32, row stride ld, E entries):  s = softmax(logits[t]);  choice = s + correction (correction may be NULL);

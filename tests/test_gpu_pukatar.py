@@ -293,6 +293,41 @@ def test_channel_delta_rule_in_a_launch_of_many_runs(dev, cut_sizes):
         assert close(got[s], delta_oracle(m, w, h[s], 1e-6), 5e-5), s
 
 
+@pytest.mark.parametrize("channel", [True, False])
+@pytest.mark.parametrize("H,G,d,dv", [(4, 2, 64, 32), (3, 3, 40, 24), (2, 1, 128, 128), (2, 2, 200, 40), (1, 1, 12, 5), (8, 8, 256, 256)])
+def test_delta_scan_forms_agree_bit_for_bit(dev, channel, H, G, d, dv):
+    """Loads straight into registers, or tokens staged through LDS with one, two or four value columns per lane: runs of unequal length (also
+    one row, a tile of rows, one more), continued from slots' states or fresh, in scattered slots."""
+    from vllm_i64_amd import _lib, ops_dense as D
+    g = torch.Generator().manual_seed(d + dv)
+    r = Rows(dev, [(4, 0, 33), (1, 7, 1), (0, 3, 16), (3, 0, 17), (2, 50, 70)])
+    C = 2 * G * d + H * dv
+    X, Gt, F = torch.randn(r.n, C, generator=g) * 0.2, torch.rand(r.n, 2 * H, generator=g), torch.rand(r.n, H * d, generator=g)
+    S0 = torch.randn(5, H, dv, d, generator=g)
+    X, Gt, F = X.to(dev), Gt.to(dev), F.to(dev)
+    got = []
+    try:
+        for form in (1, 2, 3, 4, 0):
+            _lib.call_dense("i64h_set_gdn_scan_form", form)
+            S, O = S0.to(dev).clone(), torch.full((r.n, H * dv), 7.0, device=dev)
+            D.gdn_scan(X, Gt, f=F if channel else None, q_off=0, k_off=G * d, v_off=2 * G * d, heads=H, kv_heads=G, dim=d, vdim=dv, seg_start=r.seg, nseg=r.nseg,
+                       positions=r.pos, slot_ids=r.slots, state=S, out=O, n=r.n)
+            got.append((O.cpu(), S.cpu()))
+    finally:
+        _lib.call_dense("i64h_set_gdn_scan_form", 0)
+    for O, S in got[1:]:
+        assert torch.equal(O, got[0][0]) and torch.equal(S, got[0][1])
+    own = torch.arange(H) // (H // G)
+    at = 0
+    for slot, p, c in [(4, 0, 33), (1, 7, 1), (0, 3, 16), (3, 0, 17), (2, 50, 70)]:      # (the fresh runs against the oracle's recurrence)
+        x, gt, f = (t[at:at + c].cpu().double() for t in (X, Gt, F))
+        if p == 0:
+            q, k, v = x[:, :G * d].reshape(c, G, d)[:, own], x[:, G * d:2 * G * d].reshape(c, G, d)[:, own], x[:, 2 * G * d:].reshape(c, H, dv)
+            dec = f.reshape(c, H, d) if channel else gt[:, H:].unsqueeze(-1).expand(c, H, d)
+            assert close(got[0][0][at:at + c], R.channel_delta_rule(q, k, v, gt[:, :H], dec).reshape(c, H * dv), 2e-5)
+        at += c
+
+
 @pytest.mark.parametrize("cut_sizes", [[500], [1], [64, 3]])
 def test_channel_delta_rule_keeps_one_channel_and_forgets_another(dev, cut_sizes):
     """What the first token wrote along a channel whose decay is next to one is still there 500 tokens later; along a channel that decays

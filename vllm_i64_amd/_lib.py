@@ -228,6 +228,7 @@ DENSE_SIGNATURES: Dict[str, str] = {
     "i64h_rot_post": "pp",
     "i64h_gdn_gates": "pp",
     "i64h_gdn_scan": "pp",
+    "i64h_set_gdn_scan_form": "i",
     "i64h_gla_gates": "pp",
     "i64h_gla_scan": "pp",
     "i64h_route_topk": "pp",

@@ -1,8 +1,9 @@
-"""`bench.py --design morilorn | dogalorn | zabutar | fukatar`: prefill and decode throughput of a registered design at layer sizes of real models
+"""`bench.py --design morilorn | dogalorn | zabutar | fukatar | pukatar`: prefill and decode throughput of a registered design at layer sizes of real models
 (random weights), beside the package's closest existing model at equal width, depth, feed-forward size and batch (Morilorn: the dense
 int8 decoder; Dogalorn: Morilorn, which shares its library, bf16 Linears and 32-bit residual; Zabutar: Dogalorn, the other design of
 recurrent layers beside attention with a distance bias; Fukatar: Zabutar, the other design with a norm behind every sublayer, a matrix-valued
-recurrence and attention over separate keys and values), and the design's kernels one by one against their rooflines beside the like
+recurrence and attention over separate keys and values; Pukatar: Fukatar, the other design of rotated attention and a gated delta rule),
+and the design's kernels one by one against their rooflines beside the like
 kernel of that model.  Prints one JSON line."""
 from __future__ import annotations
 
@@ -706,6 +707,207 @@ def run_fukatar(args) -> dict:
     return result
 
 
+PUKATAR_SIZES = {
+    "w1024": dict(width=1024, blocks=3, loop_blocks=1, heads=16, kv_heads=4, dim=64, vdim=64, rot_dims=64, window=1024, keep_first=4, rec_heads=8, rec_kv_heads=8, rec_dim=128,
+                  rec_vdim=128, taps=4, ff=2752, experts=8, top=2, expert_ff=896, shared_ff=896),
+    "w2048": dict(width=2048, blocks=1, loop_blocks=1, heads=32, kv_heads=8, dim=64, vdim=64, rot_dims=64, window=1024, keep_first=4, rec_heads=16, rec_kv_heads=16, rec_dim=128,
+                  rec_vdim=128, taps=4, ff=5504, experts=8, top=2, expert_ff=1792, shared_ff=1792),
+}
+PUKATAR_RANK = 128      # of the low-rank decay and gate maps
+
+
+def _pukatar_kernels(sz, rows, batch, ctx, dev):
+    """Single launches at the step's shapes with the share of their roofline (matrix products: bf16 matrix peak; recurrences: the larger of
+    bytes / HBM rate and flop / fp32 vector rate; everything else: bytes / HBM rate), each beside the like kernel of Fukatar (of Zabutar for
+    the mixture of experts)."""
+    from . import ops_dense as D
+    W, ff, H, G, dm, dv = sz["width"], sz["ff"], sz["heads"], sz["kv_heads"], sz["dim"], sz["vdim"]
+    Hr, Gr, dk, dr, taps = sz["rec_heads"], sz["rec_kv_heads"], sz["rec_dim"], sz["rec_vdim"], sz["taps"]
+    E, top, eff, win, keep, R = sz["experts"], sz["top"], sz["expert_ff"], sz["window"], sz["keep_first"], PUKATAR_RANK
+    out = {}
+    g = torch.Generator(device=dev).manual_seed(1)
+    rn = lambda *s: torch.randn(*s, device=dev, generator=g)
+
+    def row(name, t, flops=0.0, bytes_=0.0, peak=BF16_TFLOPS):
+        share = max(flops / t / (peak * 1e12), bytes_ / t / (HBM_GBS * 1e9))
+        out[name] = {"us": round(t * 1e6, 1), "roofline_share": round(share, 3)}
+
+    seq = 512
+    warm_a, warm_w, warm_c = rn(rows, W), (rn(W, W) * 0.02).to(torch.bfloat16), torch.empty(rows, W, device=dev)
+    _time(lambda: D.linear(warm_a, warm_w, warm_c), 20)      # clocks and caches settle before the first timed launch
+    for n, tag in ((rows, "prefill"), (batch, "decode")):
+        nseq = n // seq if tag == "prefill" else n
+        per = seq if tag == "prefill" else 1
+        pos0 = 0 if tag == "prefill" else ctx - 1
+        pos = (torch.arange(per, dtype=torch.int32) + pos0).repeat(nseq).to(dev)
+        slots = torch.arange(nseq, dtype=torch.int32).repeat_interleave(per).to(dev)
+        seg = (torch.arange(nseq + 1, dtype=torch.int32) * per).to(dev)
+        single = tag == "decode"
+        reps = 5 if tag == "prefill" else 20
+        a = rn(n, W)
+        # dense feed-forward's gate / up pair; beside Fukatar's up-projection with the squared relu
+        w_gu = (rn(2 * ff, W) * 0.02).to(torch.bfloat16)
+        act = torch.empty(n, ff, device=dev)
+        t = _time(lambda: D.linear(a, w_gu, act, epilogue=D.EPI_SILU_MUL), reps)
+        row(f"linear_gate_up_{tag}", t, flops=4.0 * n * ff * W, bytes_=4.0 * ff * W + 4.0 * n * (W + ff))
+        act2 = torch.empty(n, 2 * ff, device=dev)
+        t = _time(lambda: D.linear(a, w_gu, act2, epilogue=D.EPI_RELU_SQ), reps)
+        row(f"fukatar_linear_up_relu_sq_{tag}", t, flops=4.0 * n * ff * W, bytes_=4.0 * ff * W + 4.0 * n * (W + 2 * ff))
+        # what a pass over the repeated layers starts from; beside the plain Linear of the same size
+        lw, lx0, lb, lo = (rn(W, W) * 0.02).to(torch.bfloat16), rn(n, W), rn(W), torch.empty(n, W, device=dev)
+        lbytes = 2.0 * W * W + 4.0 * n * W * 2
+        t = _time(lambda: D.linear(a, lw, lo, bias=lb, epilogue=D.EPI_ADD, e=lx0, lde=W), reps)
+        row(f"loop_entry_{tag}", t, flops=2.0 * n * W * W, bytes_=lbytes + 4.0 * n * W)
+        t = _time(lambda: D.linear(a, lw, lo), reps)
+        row(f"fukatar_linear_square_{tag}", t, flops=2.0 * n * W * W, bytes_=lbytes)
+        # mixture of experts; beside Zabutar's (other activation, softmax over all entries, no gate)
+        w_r = (rn(E + 1, W) * 0.1).to(torch.bfloat16)
+        idx, wgt, rb, sg = torch.empty(n, top, dtype=torch.int32, device=dev), torch.empty(n, top, device=dev), torch.zeros(E, device=dev), torch.empty(n, device=dev)
+        rbytes = 4.0 * n * (W + 2 * top) + 2.0 * E * W
+        w_e = w_r[:E].contiguous()
+        t = _time(lambda: D.route_topk(None, h=a, w=w_e, entries=E, correction=rb, groups=1, keep=1, top=top, scale=1.0, idx=idx, wgt=wgt, n=n), reps)
+        row(f"zabutar_route_topk_{tag}", t, bytes_=rbytes)
+        t = _time(lambda: D.route_topk(None, h=a, w=w_r, entries=E, correction=None, groups=1, keep=1, top=top, scale=1.0, idx=idx, wgt=wgt, n=n, bias=rb, chosen_softmax=True,
+                                       gate_out=sg), reps)
+        row(f"route_chosen_softmax_gate_{tag}", t, bytes_=rbytes)
+        goff, ptok, prow = torch.empty(E + 1, dtype=torch.int32, device=dev), torch.empty(n * top, dtype=torch.int32, device=dev), torch.empty(n * top, dtype=torch.int32, device=dev)
+        t = _time(lambda: D.moe_plan(idx, n=n, top=top, experts=E, group_off=goff, pair_token=ptok, pair_row=prow), reps)
+        row(f"moe_plan_{tag}", t, bytes_=4.0 * n * top * 3)
+        pairs = int(goff[-1])
+        w_egu = (rn(E, 2 * eff, W) * 0.02).to(torch.bfloat16)
+        eact, ey = torch.empty(n * top, eff, device=dev), torch.empty(n * top, W, device=dev)
+        eflops, ebytes = 4.0 * pairs * eff * W, 4.0 * E * eff * W + 4.0 * pairs * (W + eff)
+        ek = dict(m=n, a_rows=ptok, batch=E, w_batch=2 * eff * W, group_off=goff)
+        t = _time(lambda: D.linear(a, w_egu, eact, epilogue=D.EPI_CLAMP_GLU, act_a=1.702, act_b=7.0, **ek), reps)
+        row(f"experts_clamped_gate_up_{tag}", t, flops=eflops, bytes_=ebytes)
+        t = _time(lambda: D.linear(a, w_egu, eact, epilogue=D.EPI_SILU_MUL, **ek), reps)
+        row(f"zabutar_experts_gate_up_{tag}", t, flops=eflops, bytes_=ebytes)
+        w_dn = (rn(E, W, eff) * 0.02).to(torch.bfloat16)
+        t = _time(lambda: D.linear(eact, w_dn, ey, m=n, batch=E, w_batch=W * eff, group_off=goff), reps)
+        row(f"experts_down_{tag}", t, flops=2.0 * pairs * eff * W, bytes_=2.0 * E * eff * W + 4.0 * pairs * (W + eff))
+        sh, yo = rn(n, W), torch.empty(n, W, device=dev)
+        t = _time(lambda: D.moe_combine(ey, prow, wgt, a, sh, yo, n=n, top=top, width=W, shared_gate=sg), reps)
+        row(f"moe_combine_gated_{tag}", t, bytes_=4.0 * n * W * (top + 2))
+        t = _time(lambda: D.moe_combine(ey, prow, wgt, a, sh, yo, n=n, top=top, width=W), reps)
+        row(f"zabutar_moe_combine_{tag}", t, bytes_=4.0 * n * W * (top + 2))
+        # residual: both results added, the next layer's centred norm with offset; beside Fukatar's centred norm of one result
+        st, y, y2, h = rn(1, n, W), rn(n, W), rn(n, W), torch.empty(n, W, device=dev)
+        wn, bn, one = torch.ones(W, device=dev), torch.zeros(W, device=dev), torch.ones(1, device=dev)
+        t = _time(lambda: D.streams_step(st, y=y, y2=y2, out_w=one, norm_w=wn, norm_b=bn, eps=1e-6, h=h, h_center=True), reps)
+        row(f"residual_two_results_norm_{tag}", t, bytes_=4.0 * n * W * 5)
+        t = _time(lambda: D.streams_step(st, y=y, y_eps=1e-6, out_w=one, post_w=wn, post_center=True), reps)
+        row(f"fukatar_residual_centred_norm_{tag}", t, bytes_=4.0 * n * W * 3)
+        # attention: prep (rotation, cache write), window with kept first positions and sink; beside Fukatar's (norms, rotated values; caps, all keys)
+        plen = seq if tag == "prefill" else ctx
+        nb = (plen + 15) // 16
+        bt = torch.arange(nseq * nb, dtype=torch.int32, device=dev).view(nseq, nb).contiguous()
+        gs = dv + dm
+        kc = (rn(nseq * nb, 16, G * gs) * 0.5).to(torch.bfloat16)
+        nq, nk, nv = H * dm, G * dm, G * dv
+        P = rn(n, nq + nk + nv) * 0.3
+        q, oa = torch.empty(n, H * gs, device=dev), torch.empty(n, H * dv, device=dev)
+        inv, vfr = torch.rand(dm // 2, device=dev, generator=g), torch.rand(dv // 2, device=dev, generator=g)
+        qw, kw = torch.ones(nq, device=dev), torch.ones(nk, device=dev)
+        pk = dict(q_off=0, k_off=nq, v_off=nq + nk, heads=H, kv_heads=G, dim=dm, vdim=dv, eps=1e-6, rot_dims=dm, interleaved=False, inv_freq=inv, head_norm=False, scale=0.125,
+                  positions=pos, slot_ids=slots, block_table=bt, cache=kc, q=q, n=n)
+        pbytes = 4.0 * n * (nq + nk + nv + H * gs) + 2.0 * n * G * gs
+        t = _time(lambda: D.rot_prep(P, q_norm_w=None, k_norm_w=None, rot_mult=1.0, v_freq=None, **pk), reps)
+        row(f"rot_prep_{tag}", t, bytes_=pbytes)
+        t = _time(lambda: D.rot_prep(P, q_norm_w=qw, k_norm_w=kw, rot_mult=1.1, v_freq=vfr, **pk), reps)
+        row(f"fukatar_rot_prep_{tag}", t, bytes_=pbytes)
+        waves = 3072 if gs <= 64 else (2048 if gs <= 128 else 1024)
+        tasks = max(1, n * G * ((H // G + 15) // 16))
+        sink = torch.zeros(H, device=dev)
+        keys = seq * (seq + 1) / 2 * nseq if tag == "prefill" else float(ctx) * n
+        wkeys = sum(min(p + 1, win + keep) for p in range(seq)) * nseq if tag == "prefill" else float(min(ctx, win + keep)) * n
+        mode = 3 if tag == "prefill" else 2
+        kk = dict(chunk=0, bias=None, heads=H, kv_heads=G, dim=dm, vdim=dv, out=oa, n=n, mode=mode)
+        for name, seen, opts in (("window_sink_attention", wkeys, dict(sink=True, sink_w=sink, window=win, keep_first=keep)), ("fukatar_capped_attention", keys, dict(sink=False, softcap=50.0))):
+            sp = 1 if tag == "prefill" else max(1, min(waves // tasks, int(seen / n) // 64, 64))
+            ws = torch.empty(max(1, D.kattn_workspace_floats(n, H, G, dv, sp)), device=dev) if sp > 1 else None
+            t = _time(lambda: D.kattn(q, kc, None, bt, slots, pos, splits=sp, workspace=ws, **kk, **opts), reps)
+            row(f"{name}_{tag}", t, flops=2.0 * seen * H * (dm + dv), bytes_=(2.0 * seen * G * gs if tag == "decode" else 0.0) + 4.0 * n * H * (gs + dv))
+        # delta rule: convolution + silu, unit vectors and write strength, low-rank decay, scan, gated head norm; beside Fukatar's
+        rk, rv, nd = Gr * dk, Hr * dr, Hr * dk
+        C = 2 * rk + rv
+        Pr = rn(n, C + 2 * Hr + rv + 2 * R) * 0.5
+        cw2, cst2, X = rn(C, taps) * 0.3, torch.zeros(nseq, taps - 1, C, device=dev), torch.empty(n, C, device=dev)
+        t = _time(lambda: D.causal_conv(Pr, off=0, channels=C, w=cw2, bias=None, positions=pos, slot_ids=slots, state=cst2, out=X, n=n, single_rows=single), reps)
+        row(f"delta_conv_silu_{tag}", t, bytes_=4.0 * n * C * 2)
+        Gt = torch.empty(n, 2 * Hr, device=dev)
+        cols = dict(q_off=0, k_off=rk, v_off=2 * rk, heads=Hr, kv_heads=Gr, dim=dk, vdim=dr, n=n)
+        al, db = torch.linspace(-4.0, 0.0, Hr, device=dev), torch.zeros(Hr, device=dev)
+        t = _time(lambda: D.gdn_gates(X, Gt, Pr, b_off=C, a_off=-1, a_log=None, dt_bias=None, unit_eps=1e-6, q_scale=dk ** -0.5, **cols), reps)
+        row(f"delta_unit_vectors_{tag}", t, bytes_=4.0 * n * rk * 4)
+        t = _time(lambda: D.gdn_gates(X, Gt, Pr, b_off=C, a_off=C + Hr, a_log=al, dt_bias=db, unit_eps=1e-6, q_scale=dk ** -0.5, **cols), reps)
+        row(f"fukatar_delta_gates_{tag}", t, bytes_=4.0 * n * rk * 4)
+        a2, F, rate, dtb = (rn(nd, R) * 0.02).to(torch.bfloat16), torch.empty(n, nd, device=dev), torch.rand(nd, device=dev, generator=g), torch.zeros(nd, device=dev)
+        dbytes = 2.0 * nd * R + 4.0 * n * (R + nd)
+        t = _time(lambda: D.linear(Pr, a2, F, m=n, a_off=C + 2 * Hr, bias=dtb, epilogue=D.EPI_DECAY, e=rate), reps)
+        row(f"channel_decay_linear_{tag}", t, flops=2.0 * n * nd * R, bytes_=dbytes)
+        F2 = torch.empty(n, nd, device=dev)
+        t = _time(lambda: D.linear(Pr, a2, F2, m=n, a_off=C + 2 * Hr), reps)
+        row(f"fukatar_linear_low_rank_{tag}", t, flops=2.0 * n * nd * R, bytes_=dbytes)
+        dstate, ro, rg = torch.zeros(nseq, Hr, dr, dk, device=dev), torch.empty(n, rv, device=dev), torch.empty(n, rv, device=dev)
+        sc = dict(seg_start=seg, nseg=nseq, positions=pos, slot_ids=slots, state=dstate, out=ro, **cols)
+        sbytes = 4.0 * n * (2 * rk + 2 * rv) + 8.0 * nseq * Hr * dk * dr
+        t = _time(lambda: D.gdn_scan(X, Gt, f=F, **sc), reps)
+        row(f"channel_delta_scan_{tag}", t, flops=7.0 * n * Hr * dk * dr, bytes_=sbytes + 4.0 * n * nd, peak=F32_TFLOPS)
+        t = _time(lambda: D.gdn_scan(X, Gt, **sc), reps)
+        row(f"fukatar_delta_scan_{tag}", t, flops=7.0 * n * Hr * dk * dr, bytes_=sbytes, peak=F32_TFLOPS)
+        nwv, Z = torch.ones(dr, device=dev), rn(n, rv)
+        t = _time(lambda: D.gate_norm(ro, nwv, rg, groups=Hr, eps=1e-6, z=Z, ldz=rv, n=n, gate_after=True, width=rv, sigmoid=True), reps)
+        row(f"gated_head_norm_{tag}", t, bytes_=4.0 * n * rv * 3)
+        t = _time(lambda: D.gate_norm(ro, nwv, rg, groups=Hr, eps=1e-6, z=Z, ldz=rv, n=n, gate_after=True, width=rv), reps)
+        row(f"fukatar_gated_head_norm_{tag}", t, bytes_=4.0 * n * rv * 3)
+    return out
+
+
+def run_pukatar(args) -> dict:
+    from . import _lib, synth
+    from .fukatar import FukatarModel
+    from .model import GreedyDecoder
+    from .pukatar import PukatarModel
+    _lib.load(), _lib.load_dense()
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    batch, ctx, rows = args.batch, args.prompt_len, 4096
+    result = {"metric": "prefill / decode tokens/s of the Pukatar design beside Fukatar at equal sizes", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+              "warmup": args.warmup, "dtype": "bf16 matrix products, fp32 residual / norms / recurrences / attention math (both designs)", "data": "synthetic",
+              "config": {"batch": batch, "context": ctx, "prefill_step": f"{rows} rows = {rows // 512} prompts of 512 tokens"}, "sizes": {}}
+    for name in (args.design_sizes.split(",") if args.design_sizes else sorted(PUKATAR_SIZES)):
+        sz = PUKATAR_SIZES[name]
+        need_tokens = batch * (ctx + args.steps + args.warmup + 64)
+
+        def fill(m):
+            g = torch.Generator(device=dev).manual_seed(5)
+            for t in {id(t): t for t in m.kv.rows if t is not None}.values():
+                t.copy_((0.5 * torch.randn(t.shape, device=dev, generator=g)).to(t.dtype))
+            for d in m.kv.state:
+                for t in d.values():
+                    t.copy_(0.1 * torch.randn(t.shape, device=dev, generator=g))
+
+        cfg = synth.pukatar_config(**sz)
+        model = PukatarModel(cfg, synth.make_pukatar_weights(cfg, rank=PUKATAR_RANK), device=dev, dtype="bfloat16", max_seqs=batch, num_kv_blocks=need_tokens // 16)
+        p, d, ms = _steps(model, GreedyDecoder, batch, ctx, rows, 512, args.steps, args.warmup, fill, cfg.vocab, dev)
+        entry = {"pukatar": {"prefill_tokens_per_s": round(p, 1), "decode_tokens_per_s": round(d, 1), "decode_ms_per_step": round(ms, 3), "layers": cfg.num_layers,
+                             "layer_runs": len(cfg.layer_runs()), "shape": sz}}
+        del model
+        torch.cuda.empty_cache()
+        fcfg = synth.fukatar_config(**FUKATAR_SIZES[name])
+        fm = FukatarModel(fcfg, synth.make_fukatar_weights(fcfg), device=dev, dtype="bfloat16", max_seqs=batch, num_kv_blocks=need_tokens // 16)
+        p, d, ms = _steps(fm, GreedyDecoder, batch, ctx, rows, 512, args.steps, args.warmup, fill, fcfg.vocab, dev)
+        entry["fukatar"] = {"prefill_tokens_per_s": round(p, 1), "decode_tokens_per_s": round(d, 1), "decode_ms_per_step": round(ms, 3), "layers": fcfg.num_layers}
+        del fm
+        torch.cuda.empty_cache()
+        entry["kernels"] = _pukatar_kernels(sz, rows, batch, ctx, dev)
+        result["sizes"][name] = entry
+    first = result["sizes"][sorted(result["sizes"])[0]]["pukatar"]
+    result["value"], result["ms_per_step"] = first["decode_tokens_per_s"], first["decode_ms_per_step"]
+    result["higher_is_better"], result["scaling"], result["vs_baseline"] = True, "weak", None
+    return result
+
+
 def main(args) -> int:
-    print(json.dumps({"dogalorn": run_dogalorn, "zabutar": run_zabutar, "fukatar": run_fukatar}.get(args.design, run)(args)), flush=True)
+    print(json.dumps({"dogalorn": run_dogalorn, "zabutar": run_zabutar, "fukatar": run_fukatar, "pukatar": run_pukatar}.get(args.design, run)(args)), flush=True)
     return 0

@@ -3,6 +3,7 @@
 //   gla_scan_kernel    : linear attention with a decay per key channel, a head's matrix in registers (16 lanes per value column)
 //   gdn_gates_kernel / gdn_scan_kernel : gated delta rule - unit-vector queries and keys, write strength and decay; the recurrence with the
 //                        correction S^T k summed over the DPP row before the write, the read-out after it; a decay per head or per key channel
+//   gdn_tile_kernel    : the same recurrence for long runs, tokens staged through LDS
 //   route_topk_kernel  : softmax scores (over all entries or the chosen ones), corrected choice, groups of neighbours, top-k and normalised
 //                        weights, one wave per row
 //   moe_plan_kernel    : (token, choice) pairs grouped by expert: offsets, the token of every grouped row, the row of every pair
@@ -175,9 +176,15 @@ __global__ __launch_bounds__(256) void gdn_gates_kernel(const i64h_gdn_args p) {
 // gdn_scan_kernel: the layout of gla_scan_kernel (one workgroup per (head, 16 * CPT value columns, run of rows); the 16 lanes of a DPP
 // row share CPT value columns and hold KPT key channels of each in registers).  Per token the state decays, the row sums S^T k with DPP
 // moves (every lane of the row ends with the sum), the correction along k is written, and a second row sum reads the state out with
-// the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order; loads run GL_TG tokens ahead.
+// the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order; loads run TG tokens ahead.
 // CHD: a decay per head and key channel (F) in the place of one per head.
-template <int KPT, int CPT, bool CHD>
+// TG is chosen so that two waves fit a SIMD's registers (the loads in flight are most of them); one where every run is a single row.
+// A lane's KPT channels: four neighbours in every stripe of 64 (so that 16 lanes read 256 consecutive bytes at a time).
+template <int KPT>
+__device__ __forceinline__ int gd_channel(int nlane, int k) {
+    return KPT >= 4 ? 4 * (nlane + 16 * (k >> 2)) + (k & 3) : nlane * KPT + k;
+}
+template <int KPT, int CPT, bool CHD, int TG>
 __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, const int ctiles, const int vec) {
     const int N = p.dim, P = p.vdim;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -187,9 +194,8 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
     const int cbase = (blockIdx.x % ctiles) * 16 * CPT + (w * 4 + cl) * CPT;
     const int64_t r0 = p.seg_start[seg], r1 = p.seg_start[seg + 1];
     if (r1 <= r0) return;
-    const int n0 = nlane * KPT;
     float S[CPT][KPT];
-    float* gS = p.state + ((int64_t)p.slot_ids[r0] * p.heads + a) * P * N + n0;      // + column * N
+    float* gS = p.state + ((int64_t)p.slot_ids[r0] * p.heads + a) * P * N;      // + column * N
     const bool fresh = p.positions[r0] == 0;
 #pragma unroll
     for (int j = 0; j < CPT; ++j) {
@@ -201,18 +207,18 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
             if (vec) {
 #pragma unroll
                 for (int k = 0; k < KPT; k += 4)
-                    if (n0 + k < N) {
-                        const float4 v = *(const float4*)(src + k);
+                    if (gd_channel<KPT>(nlane, k) < N) {
+                        const float4 v = *(const float4*)(src + gd_channel<KPT>(nlane, k));
                         S[j][k] = v.x, S[j][k + 1] = v.y, S[j][k + 2] = v.z, S[j][k + 3] = v.w;
                     }
             } else {
 #pragma unroll
                 for (int k = 0; k < KPT; ++k)
-                    if (n0 + k < N) S[j][k] = src[k];
+                    if (gd_channel<KPT>(nlane, k) < N) S[j][k] = src[gd_channel<KPT>(nlane, k)];
             }
         }
     }
-    const int qoff = p.q_off + kh * N + n0, koff = p.k_off + kh * N + n0, foff = a * N + n0;
+    const int qoff = p.q_off + kh * N, koff = p.k_off + kh * N, foff = a * N;
     struct Tok {
         float q[KPT], k[KPT], f[CHD ? KPT : 1], v[CPT], beta;
     };
@@ -223,10 +229,10 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
 #pragma unroll
             for (int k = 0; k < KPT; k += 4) {
                 float4 q = make_float4(0, 0, 0, 0), kk = q, f = q;
-                if (n0 + k < N) {
-                    q = *(const float4*)(row + qoff + k);
-                    kk = *(const float4*)(row + koff + k);
-                    if (CHD) f = *(const float4*)(p.F + t * p.ldf + foff + k);
+                if (gd_channel<KPT>(nlane, k) < N) {
+                    q = *(const float4*)(row + qoff + gd_channel<KPT>(nlane, k));
+                    kk = *(const float4*)(row + koff + gd_channel<KPT>(nlane, k));
+                    if (CHD) f = *(const float4*)(p.F + t * p.ldf + foff + gd_channel<KPT>(nlane, k));
                 }
                 u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
                 u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
@@ -235,10 +241,11 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
         } else {
 #pragma unroll
             for (int k = 0; k < KPT; ++k) {
-                const bool ok = n0 + k < N;
-                u.q[k] = ok ? row[qoff + k] : 0.0f;
-                u.k[k] = ok ? row[koff + k] : 0.0f;
-                if (CHD) u.f[k] = ok ? p.F[t * p.ldf + foff + k] : 0.0f;
+                const int c = gd_channel<KPT>(nlane, k);
+                const bool ok = c < N;
+                u.q[k] = ok ? row[qoff + c] : 0.0f;
+                u.k[k] = ok ? row[koff + c] : 0.0f;
+                if (CHD) u.f[k] = ok ? p.F[t * p.ldf + foff + c] : 0.0f;
             }
         }
 #pragma unroll
@@ -268,18 +275,18 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
             if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = part;
         }
     };
-    Tok A[GL_TG], B[GL_TG];
+    Tok A[TG], B[TG];
 #pragma unroll
-    for (int i = 0; i < GL_TG; ++i) fetch(r0 + i, A[i]);
-    for (int64_t t = r0; t < r1; t += 2 * GL_TG) {
+    for (int i = 0; i < TG; ++i) fetch(r0 + i, A[i]);
+    for (int64_t t = r0; t < r1; t += 2 * TG) {
 #pragma unroll
-        for (int i = 0; i < GL_TG; ++i) fetch(t + GL_TG + i, B[i]);
+        for (int i = 0; i < TG; ++i) fetch(t + TG + i, B[i]);
 #pragma unroll
-        for (int i = 0; i < GL_TG; ++i) step(t + i, A[i]);
+        for (int i = 0; i < TG; ++i) step(t + i, A[i]);
 #pragma unroll
-        for (int i = 0; i < GL_TG; ++i) fetch(t + 2 * GL_TG + i, A[i]);
+        for (int i = 0; i < TG; ++i) fetch(t + 2 * TG + i, A[i]);
 #pragma unroll
-        for (int i = 0; i < GL_TG; ++i) step(t + GL_TG + i, B[i]);
+        for (int i = 0; i < TG; ++i) step(t + TG + i, B[i]);
     }
 #pragma unroll
     for (int j = 0; j < CPT; ++j) {
@@ -288,11 +295,163 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
         if (vec) {
 #pragma unroll
             for (int k = 0; k < KPT; k += 4)
-                if (n0 + k < N) *(float4*)(dst + k) = make_float4(S[j][k], S[j][k + 1], S[j][k + 2], S[j][k + 3]);
+                if (gd_channel<KPT>(nlane, k) < N) *(float4*)(dst + gd_channel<KPT>(nlane, k)) = make_float4(S[j][k], S[j][k + 1], S[j][k + 2], S[j][k + 3]);
         } else {
 #pragma unroll
             for (int k = 0; k < KPT; ++k)
-                if (n0 + k < N) dst[k] = S[j][k];
+                if (gd_channel<KPT>(nlane, k) < N) dst[gd_channel<KPT>(nlane, k)] = S[j][k];
+        }
+    }
+}
+
+// gdn_tile_kernel: the same recurrence, bit for bit, for runs of many rows.  What every wave of a workgroup reads of a token (query, key,
+// decays) is loaded once per workgroup, TT tokens at a time, into one of two LDS tiles while the other one is computed: the loads of a
+// tile have the arithmetic of a whole tile to arrive, and the waves read 16 bytes per lane from LDS one token ahead.  Needs 16-byte rows.
+template <int KPT, int CPT, bool CHD>
+__global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, const int ctiles) {
+    static_assert(KPT % 4 == 0, "whole 16-byte slices per lane");
+    constexpr int TT = KPT > 8 ? 8 : 16;      // tokens per tile
+    constexpr int NP = 16 * KPT, PARTS = CHD ? 3 : 2, LPP = TT * NP / 4 / 256, WC = 16 * CPT;     // LPP: 16-byte loads per thread and part
+    constexpr int VPT = (TT * WC + 255) / 256;
+    __shared__ __attribute__((aligned(16))) float sX[2][PARTS][TT][NP];
+    __shared__ float sV[2][TT][WC];
+    __shared__ float sG[2][TT][2];      // write strength, decay per head
+    const int N = p.dim, P = p.vdim;
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+    const int nlane = lane & 15, cl = lane >> 4;
+    const int a = blockIdx.x / ctiles, seg = blockIdx.y;
+    const int kh = a / (p.heads / p.kv_heads);
+    const int wg0 = (blockIdx.x % ctiles) * WC, cw = (w * 4 + cl) * CPT, cbase = wg0 + cw;
+    const int64_t r0 = p.seg_start[seg], r1 = p.seg_start[seg + 1];
+    if (r1 <= r0) return;      // (the whole workgroup)
+    float S[CPT][KPT];
+    float* gS = p.state + ((int64_t)p.slot_ids[r0] * p.heads + a) * P * N;
+    const bool fresh = p.positions[r0] == 0;
+#pragma unroll
+    for (int j = 0; j < CPT; ++j) {
+        const bool cok = cbase + j < P;
+        const float* src = gS + (int64_t)(cok ? cbase + j : 0) * N;
+#pragma unroll
+        for (int k = 0; k < KPT; k += 4) {
+            const int c = gd_channel<KPT>(nlane, k);
+            float4 v = make_float4(0, 0, 0, 0);
+            if (!fresh && cok && c < N) v = *(const float4*)(src + c);
+            S[j][k] = v.x, S[j][k + 1] = v.y, S[j][k + 2] = v.z, S[j][k + 3] = v.w;
+        }
+    }
+    float4 st[PARTS][LPP];
+    float sv[VPT], sg = 0.0f;
+    auto gload = [&](int64_t t0) {
+#pragma unroll
+        for (int u = 0; u < LPP; ++u) {
+            const int e = tid + 256 * u, c = (e % (NP / 4)) * 4;
+            const int64_t t = t0 + e / (NP / 4);
+            const bool ok = t < r1 && c < N;
+            const float* row = p.X + t * p.ldx;
+            st[0][u] = ok ? *(const float4*)(row + p.q_off + kh * N + c) : make_float4(0, 0, 0, 0);
+            st[1][u] = ok ? *(const float4*)(row + p.k_off + kh * N + c) : make_float4(0, 0, 0, 0);
+            if (CHD) st[PARTS - 1][u] = ok ? *(const float4*)(p.F + t * p.ldf + a * N + c) : make_float4(0, 0, 0, 0);
+        }
+#pragma unroll
+        for (int u = 0; u < VPT; ++u) {
+            const int e = tid + 256 * u, c = wg0 + e % WC;
+            const int64_t t = t0 + e / WC;
+            sv[u] = (t < r1 && c < P) ? p.X[t * p.ldx + p.v_off + a * P + c] : 0.0f;
+        }
+        if (tid < 2 * TT) {
+            const int64_t t = t0 + (tid >> 1);
+            sg = (t < r1 && !(CHD && (tid & 1))) ? p.G[t * 2 * p.heads + (tid & 1) * p.heads + a] : 0.0f;
+        }
+    };
+    auto lstore = [&](int b) {
+#pragma unroll
+        for (int u = 0; u < LPP; ++u) {
+            const int e = tid + 256 * u;
+#pragma unroll
+            for (int x = 0; x < PARTS; ++x) *(float4*)&sX[b][x][e / (NP / 4)][(e % (NP / 4)) * 4] = st[x][u];
+        }
+#pragma unroll
+        for (int u = 0; u < VPT; ++u)
+            if (tid + 256 * u < TT * WC) sV[b][(tid + 256 * u) / WC][(tid + 256 * u) % WC] = sv[u];
+        if (tid < 2 * TT) sG[b][tid >> 1][tid & 1] = sg;
+    };
+    struct Tok {
+        float q[KPT], k[KPT], f[CHD ? KPT : 1], v[CPT], beta;
+    };
+    auto fetch = [&](int b, int i, Tok& u) {
+#pragma unroll
+        for (int k = 0; k < KPT; k += 4) {
+            const int c = gd_channel<KPT>(nlane, k);
+            const float4 q = *(const float4*)&sX[b][0][i][c], kk = *(const float4*)&sX[b][1][i][c];
+            u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
+            u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
+            if (CHD) {
+                const float4 f = *(const float4*)&sX[b][PARTS - 1][i][c];
+                u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < CPT; ++j) u.v[j] = sV[b][i][cw + j];
+        u.beta = sG[b][i][0];
+        if (!CHD) u.f[0] = sG[b][i][1];
+    };
+    auto step = [&](int64_t t, const Tok& u) {
+        float seen[CPT], part[CPT], d[CPT];
+#pragma unroll
+        for (int j = 0; j < CPT; ++j) {
+            seen[j] = 0.0f;
+#pragma unroll
+            for (int k = 0; k < KPT; ++k) {
+                S[j][k] *= u.f[CHD ? k : 0];
+                seen[j] = fmaf(S[j][k], u.k[k], seen[j]);
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < CPT; ++j) d[j] = u.beta * (u.v[j] - group_sum(seen[j], 16));
+#pragma unroll
+        for (int j = 0; j < CPT; ++j) {
+            part[j] = 0.0f;
+#pragma unroll
+            for (int k = 0; k < KPT; ++k) {
+                S[j][k] = fmaf(u.k[k], d[j], S[j][k]);
+                part[j] = fmaf(S[j][k], u.q[k], part[j]);
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < CPT; ++j) {
+            const float o = group_sum(part[j], 16);
+            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = o;
+        }
+    };
+    gload(r0);
+    lstore(0);
+    __syncthreads();
+    int b = 0;
+    for (int64_t t0 = r0; t0 < r1; t0 += TT, b ^= 1) {
+        const int cnt = (int)min((int64_t)TT, r1 - t0);
+        const bool more = t0 + TT < r1;
+        if (more) gload(t0 + TT);
+        Tok A, B;
+        fetch(b, 0, A);
+        for (int i = 0; i < cnt; i += 2) {
+            fetch(b, i + 1, B);            // (a tile has TT rows, an even number: zeros past the run's end)
+            step(t0 + i, A);
+            if (i + 1 < cnt) {
+                if (i + 2 < cnt) fetch(b, i + 2, A);
+                step(t0 + i + 1, B);
+            }
+        }
+        if (more) lstore(b ^ 1);
+        __syncthreads();
+    }
+#pragma unroll
+    for (int j = 0; j < CPT; ++j) {
+        if (cbase + j >= P) continue;
+        float* dst = gS + (int64_t)(cbase + j) * N;
+#pragma unroll
+        for (int k = 0; k < KPT; k += 4) {
+            const int c = gd_channel<KPT>(nlane, k);
+            if (c < N) *(float4*)(dst + c) = make_float4(S[j][k], S[j][k + 1], S[j][k + 2], S[j][k + 3]);
         }
     }
 }
@@ -555,6 +714,13 @@ int i64h_gdn_gates(const i64h_gdn_args* dp, void* stream) {
     return 0;
 }
 
+static int g_gdn_form = 0;
+int i64h_set_gdn_scan_form(int32_t form) {
+    I64H_CHECK_ARG(form >= 0 && form <= 4, "gdn_scan: form %d", form);
+    g_gdn_form = form;
+    return 0;
+}
+
 int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
     I64H_CHECK_ARG(dp != nullptr, "gdn_scan: no descriptor");
     const i64h_gdn_args& d = *dp;
@@ -564,27 +730,53 @@ int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
     I64H_CHECK_ARG(d.nseg <= 65535, "gdn_scan: %d runs in one launch", d.nseg);
     if (d.nseg <= 0 || d.n == 0) return 0;
     const int kpt = (d.dim + 15) / 16;
+    auto vec_ok = [&](int K) {
+        return K % 4 == 0 && d.dim % 4 == 0 && d.ldx % 4 == 0 && d.q_off % 4 == 0 && d.k_off % 4 == 0 && (uintptr_t)d.X % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
+               (!d.F || (d.ldf % 4 == 0 && (uintptr_t)d.F % 16 == 0));
+    };
+    const int kround = kpt <= 4 ? 4 : (kpt <= 8 ? 8 : 16);
+    if (g_gdn_form != 1 && vec_ok(kround) && (g_gdn_form > 1 || d.n >= 8 * (int64_t)d.nseg)) {
+        // one value column per lane while that is at most two workgroups per CU, two (fewer reads of the tile) beyond
+        const int cpt = g_gdn_form > 1 ? (g_gdn_form == 4 ? 4 : g_gdn_form - 1) : ((int64_t)d.heads * ((d.vdim + 15) / 16) * d.nseg <= 512 ? 1 : 2);
+        const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
+        const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
+        auto launch = [&](auto kern) { hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles); };
+#define GDN_TILE(C, CHD)                                      \
+    if (kround == 4) launch(gdn_tile_kernel<4, C, CHD>);      \
+    else if (kround == 8) launch(gdn_tile_kernel<8, C, CHD>); \
+    else launch(gdn_tile_kernel<16, C, CHD>);
+        if (d.F) {
+            if (cpt == 1) { GDN_TILE(1, true) } else if (cpt == 2) { GDN_TILE(2, true) } else { GDN_TILE(4, true) }
+        } else {
+            if (cpt == 1) { GDN_TILE(1, false) } else if (cpt == 2) { GDN_TILE(2, false) } else { GDN_TILE(4, false) }
+        }
+#undef GDN_TILE
+        I64H_CHECK_LAUNCH();
+        return 0;
+    }
     // columns per lane: query and key are loaded once for both - unless the launch would then leave most of the chip idle
     // (two columns also give the two row sums of a token independent work to overlap: measured faster from 256 workgroups on)
     const int cpt = (d.vdim > 16 && (int64_t)d.heads * ((d.vdim + 31) / 32) * d.nseg >= 256) ? 2 : 1;
     const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
     const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
     auto launch = [&](auto kern, int K) {
-        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldx % 4 == 0 && d.q_off % 4 == 0 && d.k_off % 4 == 0 && (uintptr_t)d.X % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
-                        (!d.F || (d.ldf % 4 == 0 && (uintptr_t)d.F % 16 == 0));
+        const int vec = vec_ok(K);
         hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
     };
-#define GDN_PICK(C, CHD)                                          \
-    if (kpt <= 1) launch(gdn_scan_kernel<1, C, CHD>, 1);          \
-    else if (kpt <= 2) launch(gdn_scan_kernel<2, C, CHD>, 2);     \
-    else if (kpt <= 4) launch(gdn_scan_kernel<4, C, CHD>, 4);     \
-    else if (kpt <= 8) launch(gdn_scan_kernel<8, C, CHD>, 8);     \
-    else launch(gdn_scan_kernel<16, C, CHD>, 16);
+#define GDN_PICK(C, CHD, ONE)                                                              \
+    if (kpt <= 1) launch(gdn_scan_kernel<1, C, CHD, ONE ? 1 : 4>, 1);                       \
+    else if (kpt <= 2) launch(gdn_scan_kernel<2, C, CHD, ONE ? 1 : 4>, 2);                  \
+    else if (kpt <= 4) launch(gdn_scan_kernel<4, C, CHD, ONE ? 1 : 4>, 4);                  \
+    else if (kpt <= 8) launch(gdn_scan_kernel<8, C, CHD, ONE ? 1 : (CHD ? 2 : 4)>, 8);      \
+    else launch(gdn_scan_kernel<16, C, CHD, ONE ? 1 : (CHD ? 1 : 2)>, 16);
+#define GDN_PICK2(C, CHD) \
+    if (d.nseg == d.n) { GDN_PICK(C, CHD, true) } else { GDN_PICK(C, CHD, false) }
     if (d.F) {
-        if (cpt == 2) { GDN_PICK(2, true) } else { GDN_PICK(1, true) }
+        if (cpt == 2) { GDN_PICK2(2, true) } else { GDN_PICK2(1, true) }
     } else {
-        if (cpt == 2) { GDN_PICK(2, false) } else { GDN_PICK(1, false) }
+        if (cpt == 2) { GDN_PICK2(2, false) } else { GDN_PICK2(1, false) }
     }
+#undef GDN_PICK2
 #undef GDN_PICK
     I64H_CHECK_LAUNCH();
     return 0;

@@ -31,7 +31,13 @@ __device__ __forceinline__ float dn_gelu_tanh(float z) {
 
 __device__ __forceinline__ float dn_gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
-__device__ __forceinline__ float dn_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// log(1 + e^z) with one logarithm: with u = 1 + x rounded, log(u) x / (u - 1) is log(1 + x) to a few units in the last place (Kahan's
+// correction of the rounding of u)
+__device__ __forceinline__ float dn_softplus(float z) {
+    const float x = expf(z), u = 1.0f + x, d = u - 1.0f;
+    const float l = d > 0.0f ? logf(u) * (x * __builtin_amdgcn_rcpf(d)) : x;
+    return z > 20.0f ? z : l;
+}
 
 __device__ __forceinline__ float dn_xielu(float z, float a, float b) {
     return z > 0.0f ? a * z * z + 0.5f * z : b * (expm1f(z) - z) + 0.5f * z;

@@ -276,3 +276,66 @@ def make_fukatar_weights(cfg, seed: int = 0, std: float = 0.02) -> Dict[str, tor
                       rp + "A_log": torch.linspace(-4.0, 0.0, r.heads).to(torch.bfloat16), rp + "dt_bias": torch.zeros(r.heads, dtype=torch.bfloat16),
                       rp + "norm": one(r.vdim), rp + "g": rn(rv, W), rp + "o": rn(W, rv), p + "mix.left.out": one(W), p + "mix.right.out": one(W)})
     return w
+
+
+def pukatar_config(width: int = 1024, blocks: int = 3, loop_blocks: int = 1, heads: int = 16, kv_heads: int = 4, dim: int = 64, vdim: int = 64, rot_dims: int = 64, window: int = 1024,
+                   keep_first: int = 4, rec_heads: int = 8, rec_kv_heads: int = 8, rec_dim: int = 128, rec_vdim: int = 128, taps: int = 4, ff: int = 2752, experts: int = 8,
+                   top: int = 2, expert_ff: int = 896, shared_ff: int = 896, vocab: int = 32000):
+    """A Pukatar configuration with layers of a real model's proportions: `blocks` times (delta rule with a dense feed-forward, delta rule
+    with a mixture of experts, windowed attention with a dense feed-forward, delta rule with a mixture), the first loop_blocks of them run
+    twice; random weights: make_pukatar_weights."""
+    from .config import PukatarConfig
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "shared": {"ff": shared_ff, "limit": 7.0}, "router": {"experts": experts, "top": top}}
+    rec = {"type": "channel_delta", "mixer": {"heads": rec_heads, "kv_heads": rec_kv_heads, "dim": rec_dim, "vdim": rec_vdim, "conv": taps}}
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "rot": {"base": 10000.0, "dims": rot_dims},
+                                          "mask": {"size": window, "keep_first": keep_first}}}
+    layers = []
+    for _ in range(blocks):
+        layers += [dict(rec, mlp=dense), dict(rec, mlp=moe), dict(att, mlp=dense), dict(rec, mlp=moe)]
+    d = {"architecture": "Pukatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers}
+    if loop_blocks:
+        d["loop"] = {"start": 0, "stop": 4 * loop_blocks, "times": 2}
+    return PukatarConfig.from_dict(d)
+
+
+def make_pukatar_weights(cfg, seed: int = 0, std: float = 0.02, rank: int = 128) -> Dict[str, torch.Tensor]:
+    """bf16 N(0, std) matrices, norm weights one and offsets zero, convolution taps small, sinks zero, decays spread over the heads, low-rank
+    maps of `rank`, a router wide enough that the experts' loads differ from token to token."""
+    g = torch.Generator().manual_seed(seed)
+    W = cfg.width
+
+    def rn(*shape, s=std):
+        return torch.empty(*shape, dtype=torch.float32).normal_(0.0, s, generator=g).to(torch.bfloat16)
+
+    one, zero = (lambda *n: torch.ones(*n, dtype=torch.bfloat16)), (lambda *n: torch.zeros(*n, dtype=torch.bfloat16))
+    w = {"embed": rn(cfg.vocab, W), "head": rn(cfg.vocab, W)}
+    for name in ("embed.norm", "final.norm", *(f"l{i}.norm1" for i in range(len(cfg.layers)))):
+        w.update({name: one(W), name + ".b": zero(W)})
+    if cfg.loop is not None:
+        w.update({"loop.in": rn(W, 2 * W), "loop.step": zero(cfg.loop.times, W)})
+
+    def glu(p, ff):
+        w.update({p + "gate": rn(ff, W), p + "up": rn(ff, W), p + "down": rn(W, ff)})
+
+    for i, L in enumerate(cfg.layers):
+        p, m, f = f"l{i}.", L.mixer, L.mlp
+        mp = p + "mix."
+        rk, rv, nd = m.kv_heads * m.dim, m.heads * m.vdim, m.heads * m.dim
+        w.update({mp + "k": rn(rk, W), mp + "o": rn(W, rv)})
+        if L.type == "attention":
+            w.update({mp + "q": rn(nd, W), mp + "v": rn(m.kv_heads * m.vdim, W), mp + "sink": zero(m.heads)})
+        else:
+            w.update({mp + "q": rn(rk, W), mp + "v": rn(rv, W), mp + "q.conv": rn(rk, m.conv, s=0.3), mp + "k.conv": rn(rk, m.conv, s=0.3), mp + "v.conv": rn(rv, m.conv, s=0.3),
+                      mp + "b": rn(m.heads, W), mp + "A_log": torch.linspace(-4.0, 0.0, m.heads).to(torch.bfloat16), mp + "dt_bias": zero(nd), mp + "norm": one(m.vdim),
+                      mp + "a1": rn(rank, W), mp + "a2": rn(nd, rank), mp + "g1": rn(rank, W), mp + "g2": rn(rv, rank)})
+        if f is not None and f.kind == "dense":
+            glu(p + "mlp.", f.ff)
+        elif f is not None:
+            w.update({p + "mlp.router": rn(f.experts, W, s=0.1), p + "mlp.router.b": zero(f.experts)})
+            for e in range(f.experts):
+                glu(f"{p}mlp.e{e}.", f.ff)
+            if f.shared_ff:
+                glu(p + "mlp.shared.", f.shared_ff)
+                w[p + "mlp.shared.sg"] = rn(1, W)
+    return w
