@@ -4,6 +4,7 @@ A design's own file holds its weight layout, its residual and the order in which
 from __future__ import annotations
 
 import os
+from contextlib import contextmanager
 from typing import Callable, Dict, List, Optional
 
 import torch
@@ -22,6 +23,7 @@ class HybridRunner:
     ATTN_MAX_SEGMENTS = 4
     ATTN_WAVES = {64: 3072, 128: 2048, 256: 1024}     # waves a decode-sized attention launch aims at, by the width of a key head's cached part
     BUFFERS: Optional[Callable] = None                # (runner, rows, logit rows) -> the step's buffers
+    SIDE_STREAM = False                               # a second stream for a sublayer that runs beside another one
 
     def _init_runner(self, cfg, device, dtype: str) -> None:
         if dtype not in ("bfloat16", "float32"):
@@ -31,6 +33,24 @@ class HybridRunner:
         self._bufs: Dict[tuple, object] = {}
         self._pinned: set = set()
         self._arange: Dict[int, torch.Tensor] = {}
+        self.side = torch.cuda.Stream(device=self.device) if self.SIDE_STREAM and self.device.type == "cuda" else None
+
+    # ---- two sublayers side by side ----
+    @contextmanager
+    def _beside(self):
+        """The launches of the body run on the side stream (of default priority), behind what the current stream holds so far and beside what
+        it gets next, until _meet(); a captured graph keeps the two branches.  Without a side stream they simply run here.  One level only:
+        the body forks no further."""
+        if self.side is None:
+            yield
+            return
+        self.side.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(self.side):
+            yield
+
+    def _meet(self) -> None:
+        if self.side is not None:
+            torch.cuda.current_stream().wait_stream(self.side)
 
     # ---- tensors by name and shape, in the two forms the kernels read ----
     def _bf(self, t: torch.Tensor) -> torch.Tensor:

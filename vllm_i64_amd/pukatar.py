@@ -59,6 +59,7 @@ class _StepBuffers:
 
 class PukatarModel(HybridRunner):
     BUFFERS = _StepBuffers
+    SIDE_STREAM = True
 
     def __init__(self, cfg: PukatarConfig, weights: Dict[str, torch.Tensor], device="cuda:0", dtype: str = "bfloat16", max_seqs: int = 4,
                  num_kv_blocks: int = 256, kv_block: int = 16, cache_dtype: Optional[torch.dtype] = None):
@@ -152,6 +153,12 @@ class PukatarModel(HybridRunner):
             self._load_moe(p + "mlp.", ff, need, d)
         return d
 
+    def _feed_forward(self, B, d, n, record, r) -> None:
+        if d["mlp"].kind == "dense":
+            self._dense_ff(B, d, n)
+        else:
+            self._moe_ff(B, d, n, B.h, B.y2, B.y3, record, f"r{r}")
+
     def _dense_ff(self, B, d, n) -> None:
         ff = d["mlp"].ff
         act = B.act[: n * ff].view(n, ff)
@@ -196,6 +203,10 @@ class PukatarModel(HybridRunner):
                 cur = 1 - cur
             if r == 0 or t is not None:      # (elsewhere the launch that wrote the residual has normed it)
                 D.streams_step(B.x[cur], **read(d["norm1"], B.h))
+            # mixer and feed-forward read the same input and meet at the residual: they run side by side
+            if d["mlp"] is not None:
+                with self._beside():
+                    self._feed_forward(B, d, n, record, r)
             P = B.p[: n * d["ld"]].view(n, d["ld"])
             D.linear(B.h, d["w_in"], P, exact=ex)
             if d["type"] == "attention":
@@ -205,10 +216,7 @@ class PukatarModel(HybridRunner):
             write = dict(y=B.y, out_w=self.ones1)
             if d["mlp"] is not None:
                 write["y2"] = B.y2
-                if d["mlp"].kind == "dense":
-                    self._dense_ff(B, d, n)
-                else:
-                    self._moe_ff(B, d, n, B.h, B.y2, B.y3, record, f"r{r}")
+                self._meet()
             if r + 1 < len(self.layer_runs) and self.layer_runs[r + 1][1] is None:
                 write.update(read(self.layers[self.layer_runs[r + 1][0]]["norm1"], B.h))
             D.streams_step(B.x[cur], **write)
