@@ -276,6 +276,8 @@ typedef struct {
     int32_t mode;
     int32_t single_rows; /* 1: every row is the only row of its sequence in this launch: the launch that computes a row also stores its
                             sequence's new carried inputs (no second launch) */
+    const int32_t* seg_start; /* int32 [nseg + 1] (may be NULL): the runs' first rows, so that the second launch visits a run's last row only */
+    int32_t nseg;
 } i64h_causal_conv_args;
 int i64h_causal_conv(const i64h_causal_conv_args* d, void* stream);
 

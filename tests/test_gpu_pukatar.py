@@ -245,7 +245,7 @@ def delta_run(dev, m, w, h, lens, cut_sizes, eps):
         P = torch.cat([h[s][p:p + c] for s, p, c in runs]).float().to(dev).contiguous()
         X, Gt, F, O, On = (torch.empty(r.n, k, device=dev) for k in (C, 2 * H, nd, rv, rv))
         D.causal_conv(P, off=0, channels=C, w=conv_w, bias=None, positions=r.pos, slot_ids=r.slots, state=conv_state, out=X, n=r.n,
-                      single_rows=all(c == 1 for _, _, c in runs))
+                      single_rows=all(c == 1 for _, _, c in runs), seg_start=r.seg, nseg=r.nseg)
         cols = dict(q_off=0, k_off=rk, v_off=2 * rk, heads=H, kv_heads=G, dim=d, vdim=dv, n=r.n)
         D.gdn_gates(X, Gt, P, b_off=C, a_off=-1, a_log=None, dt_bias=None, unit_eps=1e-6, q_scale=d ** -0.5, **cols)
         D.linear(P, eye, F, m=r.n, a_off=C + H, exact=True, bias=w["dt_bias"].float().to(dev), epilogue=D.EPI_DECAY, e=rate)

@@ -282,7 +282,7 @@ class Streams(ctypes.Structure):
 class CausalConv(ctypes.Structure):
     """Mirror of i64h_causal_conv_args (include/i64h_dense.h)."""
     _fields_ = [("P", _P), ("ldp", _L), ("off", _I), ("channels", _I), ("taps", _I), ("w", _P), ("bias", _P), ("positions", _P), ("slot_ids", _P),
-                ("state", _P), ("out", _P), ("ldo", _L), ("n", _L), ("mode", _I), ("single_rows", _I)]
+                ("state", _P), ("out", _P), ("ldo", _L), ("n", _L), ("mode", _I), ("single_rows", _I), ("seg_start", _P), ("nseg", _I)]
 
 
 class SsmScan(ctypes.Structure):

@@ -244,9 +244,9 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(const i64h_causal
 }
 
 __global__ __launch_bounds__(256) void conv_carry_kernel(const i64h_causal_conv_args p) {
-    const int64_t t = blockIdx.y;
+    const int64_t t = p.seg_start ? (int64_t)p.seg_start[blockIdx.y + 1] - 1 : (int64_t)blockIdx.y;
     const int c = blockIdx.x * 256 + threadIdx.x;
-    if (t + 1 < p.n && hy_continues(p.slot_ids, p.positions, t + 1, 1)) return;   // only the last row of a run
+    if (t < 0 || (t + 1 < p.n && hy_continues(p.slot_ids, p.positions, t + 1, 1))) return;   // only the last row of a run
     if (c >= p.channels) return;
     const int before = conv_rows_before(p, t);
     float v[HY_MAX_TAPS];   // the inputs 0 .. taps - 2 positions back, read before any is overwritten
@@ -783,6 +783,7 @@ int i64h_causal_conv(const i64h_causal_conv_args* dp, void* stream) {
     I64H_CHECK_ARG(d.P && d.w && d.out && d.positions && d.slot_ids && (d.state || d.taps == 1), "causal_conv: null operand");
     I64H_CHECK_ARG(d.n <= 65535, "causal_conv: %lld rows in one launch (at most 65535)", (long long)d.n);
     I64H_CHECK_ARG(d.mode == 0 || d.mode == 1, "causal_conv: mode %d", d.mode);
+    I64H_CHECK_ARG(!d.seg_start || (d.nseg > 0 && d.nseg <= d.n) || d.n == 0, "causal_conv: %d runs in %lld rows", d.nseg, (long long)d.n);
     if (d.n == 0) return 0;
     const dim3 grid((unsigned)((d.channels + 255) / 256), (unsigned)d.n);
     const dim3 walk((unsigned)((d.channels + 255) / 256), (unsigned)((d.n + CV_ROWS - 1) / CV_ROWS));
@@ -799,7 +800,8 @@ int i64h_causal_conv(const i64h_causal_conv_args* dp, void* stream) {
     }
     I64H_CHECK_LAUNCH();
     if (d.taps > 1 && !d.single_rows) {
-        hipLaunchKernelGGL(conv_carry_kernel, grid, dim3(256), 0, (hipStream_t)stream, d);
+        const dim3 carry(grid.x, d.seg_start ? (unsigned)d.nseg : grid.y);
+        hipLaunchKernelGGL(conv_carry_kernel, carry, dim3(256), 0, (hipStream_t)stream, d);
         I64H_CHECK_LAUNCH();
     }
     return 0;

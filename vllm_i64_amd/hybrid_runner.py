@@ -183,7 +183,7 @@ class HybridRunner:
         C, rk, rv = r.conv_channels, r.kv_heads * r.dim, r.heads * r.vdim
         X = B.a[: n * C].view(n, C)
         D.causal_conv(P, off=d["r_off"], channels=C, w=d["conv_w"], bias=None, positions=positions, slot_ids=slot_ids, state=st.get("conv"), out=X, n=n,
-                      single_rows=single)
+                      single_rows=single, seg_start=seg, nseg=nseg)
         G = B.g[: n * 2 * r.heads].view(n, 2 * r.heads)
         cols = dict(q_off=0, k_off=rk, v_off=2 * rk, heads=r.heads, kv_heads=r.kv_heads, dim=r.dim, vdim=r.vdim, n=n)
         channel = r.decay == "channel"

@@ -230,10 +230,15 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
 
 def causal_conv(p: torch.Tensor, *, off: int, channels: int, w: torch.Tensor, bias: Optional[torch.Tensor], positions: torch.Tensor,
                 slot_ids: torch.Tensor, state: Optional[torch.Tensor], out: torch.Tensor, n: Optional[int] = None, added: bool = False,
-                single_rows: bool = False) -> torch.Tensor:
+                single_rows: bool = False, seg_start: Optional[torch.Tensor] = None, nseg: int = 0) -> torch.Tensor:
     """See i64h_causal_conv.  p fp32 [n, ldp]; w fp32 [channels, taps]; state fp32 [slots, taps - 1, channels]; out fp32 [n, channels].
     added: the convolution is added to its own input and no activation follows (mode 1).  single_rows: the caller vouches that every row
-    is the only row of its sequence in this launch; the carried inputs are then stored by the same launch."""
+    is the only row of its sequence in this launch; the carried inputs are then stored by the same launch.  seg_start int32 [nseg + 1]: the
+    first rows of the runs of one sequence."""
+    if seg_start is not None:
+        _chk(seg_start, torch.int32, "seg_start")
+        if seg_start.numel() < nseg + 1:
+            raise _lib.I64HError("causal_conv: seg_start needs nseg + 1 entries")
     _chk(p, torch.float32, "p"), _chk(w, torch.float32, "w"), _chk(out, torch.float32, "out")
     _chk(positions, torch.int32, "positions"), _chk(slot_ids, torch.int32, "slot_ids")
     rows = int(n if n is not None else positions.numel())
@@ -250,7 +255,8 @@ def causal_conv(p: torch.Tensor, *, off: int, channels: int, w: torch.Tensor, bi
             (bias is not None and bias.numel() != channels) or (taps > 1 and (state.shape[-1] != channels or state.shape[-2] != taps - 1)):
         raise _lib.I64HError("causal_conv: shapes do not fit the sizes")
     d = _lib.CausalConv(P=ptr(p), ldp=p.shape[-1], off=off, channels=channels, taps=taps, w=ptr(w), bias=ptr(bias), positions=ptr(positions),
-                        slot_ids=ptr(slot_ids), state=ptr(state), out=ptr(out), ldo=channels, n=rows, mode=1 if added else 0, single_rows=int(bool(single_rows)))
+                        slot_ids=ptr(slot_ids), state=ptr(state), out=ptr(out), ldo=channels, n=rows, mode=1 if added else 0, single_rows=int(bool(single_rows)),
+                        seg_start=ptr(seg_start), nseg=int(nseg) if seg_start is not None else 0)
     call_dense("i64h_causal_conv", _ref(d), _stream())
     return out
 
