@@ -833,7 +833,7 @@ def _pukatar_kernels(sz, rows, batch, ctx, dev):
         Pr = rn(n, C + 2 * Hr + rv + 2 * R) * 0.5
         cw2, cst2, X = rn(C, taps) * 0.3, torch.zeros(nseq, taps - 1, C, device=dev), torch.empty(n, C, device=dev)
         t = _time(lambda: D.causal_conv(Pr, off=0, channels=C, w=cw2, bias=None, positions=pos, slot_ids=slots, state=cst2, out=X, n=n, single_rows=single,
-                                        seg_start=seg, nseg=nseg), reps)
+                                        seg_start=seg, nseg=nseq), reps)
         row(f"delta_conv_silu_{tag}", t, bytes_=4.0 * n * C * 2)
         Gt = torch.empty(n, 2 * Hr, device=dev)
         cols = dict(q_off=0, k_off=rk, v_off=2 * rk, heads=Hr, kv_heads=Gr, dim=dk, vdim=dr, n=n)
