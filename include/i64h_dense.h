@@ -36,7 +36,10 @@ int i64h_device_check(void);
  *   I64H_EPI_XIELU: v > 0 ? act_a v^2 + v / 2 : act_b (exp(v) - 1 - v) + v / 2  (the caller passes act_a = softplus(p), act_b = 1/2 + softplus(q)).
  *   I64H_EPI_RELU_SQ: max(v, 0)^2.
  *   I64H_EPI_CLAMP_GLU: u = min(A W^T, act_b), w = clamp(A W2^T, -act_b, act_b), u * sigmoid(act_a * u) * (w + 1), laid out as I64H_EPI_GELU_MUL;
- *   I64H_EPI_ADD: v + E[b][m, n];  I64H_EPI_DECAY: exp(-E[b][m, n] * softplus(v))  (with lde = 0 E is one row for all m).
+ *   I64H_EPI_ADD: v + E[b][m, n];  I64H_EPI_DECAY: exp(-E[b][m, n] * softplus(v))  (with lde = 0 E is one row for all m);
+ *   I64H_EPI_ROW_SIGMOID: v * sigmoid(E[b][m]), one gate for all columns of a row (a head's gate where the batch is the heads).
+ *   row_scale (may be NULL; fp32, one per row of C, the gate / up epilogues only): both sums are multiplied by row_scale[m] first - the
+ *   input row times that factor.
  *   bias (may be NULL; fp32 [N], batch stride bias_batch) is added to the sum before any epilogue but the three gate / up ones.
  * group_off (may be NULL; device int32 [batch + 1], ascending): batch b takes the rows [group_off[b], group_off[b + 1]) of a_rows
  *   (of A itself without a_rows) and of C instead of all M rows; M is then the most rows any batch may have (it sizes the launch,
@@ -56,6 +59,7 @@ int i64h_device_check(void);
 #define I64H_EPI_CLAMP_GLU 9
 #define I64H_EPI_ADD 10
 #define I64H_EPI_DECAY 11
+#define I64H_EPI_ROW_SIGMOID 12
 #define I64H_SKINNY_ROWS 8
 typedef struct {
     const float* A;
@@ -78,6 +82,7 @@ typedef struct {
     float scale;
     float act_a, act_b;
     const int32_t* group_off;
+    const float* row_scale;
 } i64h_linear;
 int i64h_linear_run(const i64h_linear* d, void* stream);
 
@@ -122,7 +127,7 @@ int i64h_gated_postnorm(const i64h_postnorm* d, void* stream);
  *   key    = rotate(P[t, dkv_off + kv_rank : +rot_dim], position)               -> cache row, columns [kv_rank, +rot_dim)
  *   Q[t, h, kv_rank : +rot_dim] = rotate(P[t, q_off + h * (dim + rot_dim) + dim : +rot_dim], position)   for every head h
  * rotate: the first rot_dims values in interleaved pairs (2i, 2i+1) by the angle position * inv_freq[i] (fp32 product,
- * full-range sine / cosine), the rest unchanged.  Q fp32 [n, heads, kv_rank + rot_dim]; its first kv_rank columns per head
+ * full-range sine / cosine, both times rot_mult), the rest unchanged.  Q fp32 [n, heads, kv_rank + rot_dim]; its first kv_rank columns per head
  * (the query carried into latent space) are written by the caller's Linear. */
 typedef struct {
     const float* P;
@@ -140,6 +145,9 @@ typedef struct {
     int32_t cache_dtype;
     float* Q;
     int64_t n;
+    const float* Qsrc;   /* NULL: the queries are columns of P; else fp32, row stride ldqs, q_off counts in its rows */
+    int64_t ldqs;
+    float rot_mult;      /* multiplies sine and cosine */
 } i64h_latent_prep_args;
 int i64h_latent_prep(const i64h_latent_prep_args* d, void* stream);
 
@@ -222,6 +230,7 @@ int i64h_embed_bigram(const i64h_embed_bigram_args* d, void* stream);
  *                       (rms over the W columns with y_eps; weights [W]; a single normed result is the post-norm of a sandwich layer)
  *                       post_w != NULL: v <- norm(v) * post_w, over the W columns with y_eps - the root mean square, or with post_center the
  *                       centred norm (v - mean) / sqrt(mean((v - mean)^2) + y_eps): a norm on a sublayer's result, whatever it is made of
+ *                       y_scale (may be NULL, [W]): v <- v * y_scale, a learned factor per column
  *                       new_t = sum_s mix[s * S + t] * old_s + out_w[t] * v          (mix == NULL: new_t = old_t + out_w[t] * v)
  *   read  (h != NULL):  u = sum_s in_w[s] * x_s  (in_w == NULL: the plain sum);  h = u / sqrt(mean(u^2) + eps) * norm_w[c % norm_w_len],
  *                       or with h_center the centred norm (u - mean) / sqrt(mean((u - mean)^2) + eps) * norm_w;  norm_b (may be NULL, [W])
@@ -252,6 +261,7 @@ typedef struct {
     int32_t post_center;
     int32_t h_center;
     const float* norm_b;
+    const float* y_scale;
 } i64h_streams_args;
 int i64h_streams_step(const i64h_streams_args* d, void* stream);
 
@@ -440,7 +450,8 @@ int i64h_kv_prep(const i64h_kv_prep_args* d, void* stream);
  * q_t = P[t, q_off + a * dim : + dim], f_t likewise at f_off, v_t = P[t, v_off + a * vdim : + vdim];  k_t = P[...k_off...] or, with k_off < 0,
  * k_t = 1 - f_t (the forget gate also decides what is written).  state fp32 [slots, heads, vdim, dim] (S transposed; dim <= 256).
  * i64h_gla_gates prepares q and f in place:  q <- q_act ? silu(q) : q;   f <- lower + (1 - lower) * sigmoid(f)   (lower fp32 [heads * dim] or NULL = 0).
- * All arithmetic fp32, the tokens of a sequence strictly in their order. */
+ * The scan multiplies its read-out by q_scale.  F: decays that are no columns of P (see I64H_EPI_DECAY).
+ * All arithmetic fp32, the tokens of a sequence strictly in their order.  Runs of many rows with separate keys are staged through LDS. */
 typedef struct {
     float* P;
     int64_t ldp;
@@ -456,6 +467,9 @@ typedef struct {
     float* out;          /* fp32 [n, heads * vdim], row stride ldo */
     int64_t ldo;
     int64_t n;
+    const float* F;      /* the decays in a matrix of their own (fp32, row stride ldf, columns [f_off, + heads * dim)); NULL: columns of P */
+    int64_t ldf;
+    float q_scale;       /* multiplies the read-out S^T q (scan only) */
 } i64h_gla_args;
 int i64h_gla_gates(const i64h_gla_args* d, void* stream);
 int i64h_gla_scan(const i64h_gla_args* d, void* stream);
@@ -464,6 +478,7 @@ int i64h_gla_scan(const i64h_gla_args* d, void* stream);
  * i64h_rot_prep, per row t of the projections P (position pos):  q = P[t, q_off : + heads * dim], k = P[t, k_off : + kv_heads * dim],
  * v = P[t, v_off : + kv_heads * vdim];
  *   1. q_norm_w / k_norm_w (may be NULL, together): q <- q / sqrt(mean(q^2) + eps) * q_norm_w over the WHOLE row of heads * dim values, k likewise;
+ *      with norm_heads the mean is over each head's dim values and the weights are [dim], shared by the heads;
  *   2. the first rot_dims values of every head turn by pos * inv_freq[i] (fp32 product, full-range sine / cosine, both multiplied by rot_mult):
  *      pairs (i, i + rot_dims / 2) or, with interleaved, (2i, 2i + 1); (u, v) -> (u cos - v sin, v cos + u sin); the rest pass unchanged;
  *   3. head_norm: q and k are divided by sqrt(mean over the head's dim values of the square + eps), no weight;
@@ -493,6 +508,7 @@ typedef struct {
     int32_t cache_dtype;
     float* Q;
     int64_t n;
+    int32_t norm_heads;
 } i64h_rot_prep_args;
 int i64h_rot_prep(const i64h_rot_prep_args* d, void* stream);
 typedef struct {
@@ -550,7 +566,8 @@ int i64h_set_gdn_scan_form(int32_t form); /* tuning / test knob: 0 (default) = b
  * wgt[t, k] = s[idx[t, k]] / (sum_k s[idx[t, k]] + 1e-20) * scale.   E <= 1024, top <= 32.
  * W (bf16 [E, K], with h fp32 of row stride ldh; logits == NULL): the launch computes the logits itself in 32 bits.  bias (fp32 [E], may be
  * NULL) is added to the logits.  chosen_softmax: the choice falls on the logits (plus correction) as they are and the weights are the softmax
- * over the chosen logits alone, times scale.  gate_out (fp32 [n], may be NULL; with W): W has one more row, gate_out[t] = sigmoid(h[t] . W[E]). */
+ * over the chosen logits alone, times scale.  sigmoid_scores: s = sigmoid(logits) entry by entry (choice: the logits, or s + correction).
+ * raw_weights: wgt[t, k] = s[idx[t, k]] * scale, not renormalised.  gate_out (fp32 [n], may be NULL; with W): W has one more row, gate_out[t] = sigmoid(h[t] . W[E]). */
 typedef struct {
     const float* logits;
     int64_t ld;
@@ -568,6 +585,7 @@ typedef struct {
     const float* bias;
     int32_t chosen_softmax;
     float* gate_out;
+    int32_t sigmoid_scores, raw_weights;
 } i64h_route_args;
 int i64h_route_topk(const i64h_route_args* d, void* stream);
 
@@ -575,9 +593,10 @@ int i64h_route_topk(const i64h_route_args* d, void* stream);
  * i64h_moe_plan: from idx int32 [n, top] (entries >= experts are not experts and get no row) the (token, choice) pairs grouped by expert:
  *   group_off int32 [experts + 1] (ascending offsets), pair_token int32 [n * top] (the token of every grouped row, the a_rows of a grouped
  *   Linear), pair_row int32 [n, top] (where the pair's row lies, -1 for a non-expert).  The order of rows inside a group is not fixed;
- *   no result depends on it.  One launch of one workgroup; experts <= 4096.
+ *   no result depends on it.  pair_wgt (fp32 [n * top], may be NULL): the choice's weight wgt[t, k] for every grouped row (row_scale of a
+ *   grouped Linear, where the weight belongs on the expert's input).  One launch of one workgroup; experts <= 4096.
  * i64h_moe_combine: out[t, :] = sum_k wgt[t, k] * (pair_row[t, k] >= 0 ? Y[pair_row[t, k], :] : h[t, :]) + (shared ? shared[t, :] : 0),
- *   summed in the order k = 0 .. top - 1, the shared row last.  Y fp32 [pairs, W].  shared_gate (fp32 [n], may be NULL) multiplies the shared row. */
+ *   summed in the order k = 0 .. top - 1, the shared row last (wgt NULL: weights of one).  Y fp32 [pairs, W].  shared_gate (fp32 [n], may be NULL) multiplies the shared row. */
 typedef struct {
     const int32_t* idx;
     int64_t n;
@@ -585,6 +604,8 @@ typedef struct {
     int32_t* group_off;
     int32_t* pair_token;
     int32_t* pair_row;
+    const float* wgt;
+    float* pair_wgt;
 } i64h_moe_plan_args;
 int i64h_moe_plan(const i64h_moe_plan_args* d, void* stream);
 typedef struct {

@@ -403,7 +403,7 @@ def test_dense_feed_forward_alone(dev, n):
     h = torch.randn(n, 42, generator=torch.Generator().manual_seed(n))
     B = model.buffers(n, 1)
     B.h.copy_(h)
-    model._dense_ff(B, model.layers[0], n)
+    model._dense_glu(B, model.layers[0], n, B.h, B.y2)
     assert close(B.y2, R.dense_ff(w, "l0.mlp.", h.double()), 2e-5)
 
 

@@ -241,7 +241,7 @@ class Linear(ctypes.Structure):
     """Mirror of i64h_linear (include/i64h_dense.h)."""
     _fields_ = [("A", _P), ("lda", _L), ("a_rows", _P), ("W", _P), ("C", _P), ("ldc", _L), ("M", _L), ("N", _I), ("K", _I), ("batch", _I),
                 ("a_batch", _L), ("w_batch", _L), ("c_batch", _L), ("exact", _I), ("epilogue", _I), ("E", _P), ("lde", _L), ("e_batch", _L),
-                ("softcap", _F), ("bias", _P), ("bias_batch", _L), ("scale", _F), ("act_a", _F), ("act_b", _F), ("group_off", _P)]
+                ("softcap", _F), ("bias", _P), ("bias_batch", _L), ("scale", _F), ("act_a", _F), ("act_b", _F), ("group_off", _P), ("row_scale", _P)]
 
 
 class PostNorm(ctypes.Structure):
@@ -255,7 +255,7 @@ class LatentPrep(ctypes.Structure):
     """Mirror of i64h_latent_prep_args (include/i64h_dense.h)."""
     _fields_ = [("P", _P), ("ldp", _L), ("q_off", _I), ("dkv_off", _I), ("heads", _I), ("dim", _I), ("rot_dim", _I), ("kv_rank", _I),
                 ("rot_dims", _I), ("c_norm_w", _P), ("eps", _F), ("inv_freq", _P), ("positions", _P), ("slot_ids", _P), ("block_table", _P),
-                ("max_blocks_per_seq", _I), ("block_size", _I), ("cache", _P), ("cache_dtype", _I), ("Q", _P), ("n", _L)]
+                ("max_blocks_per_seq", _I), ("block_size", _I), ("cache", _P), ("cache_dtype", _I), ("Q", _P), ("n", _L), ("Qsrc", _P), ("ldqs", _L), ("rot_mult", _F)]
 
 
 class LatentAttn(ctypes.Structure):
@@ -276,7 +276,7 @@ class Streams(ctypes.Structure):
     """Mirror of i64h_streams_args (include/i64h_dense.h)."""
     _fields_ = [("streams", _P), ("S", _I), ("n", _L), ("W", _I), ("y", _P), ("ldy", _L), ("y2", _P), ("ldy2", _L), ("yn_w", _P), ("y2n_w", _P),
                 ("y_eps", _F), ("mix", _P), ("out_w", _P), ("in_w", _P), ("norm_w", _P), ("norm_w_len", _I), ("eps", _F), ("h", _P), ("rows", _P),
-                ("m_rows", _L), ("post_w", _P), ("post_center", _I), ("h_center", _I), ("norm_b", _P)]
+                ("m_rows", _L), ("post_w", _P), ("post_center", _I), ("h_center", _I), ("norm_b", _P), ("y_scale", _P)]
 
 
 class CausalConv(ctypes.Structure):
@@ -331,7 +331,7 @@ class RotPrep(ctypes.Structure):
     _fields_ = [("P", _P), ("ldp", _L), ("q_off", _I), ("k_off", _I), ("v_off", _I), ("heads", _I), ("kv_heads", _I), ("dim", _I), ("vdim", _I),
                 ("q_norm_w", _P), ("k_norm_w", _P), ("eps", _F), ("rot_dims", _I), ("interleaved", _I), ("inv_freq", _P), ("rot_mult", _F),
                 ("head_norm", _I), ("v_freq", _P), ("scale", _F), ("positions", _P), ("slot_ids", _P), ("block_table", _P),
-                ("max_blocks_per_seq", _I), ("block_size", _I), ("cache", _P), ("cache_dtype", _I), ("Q", _P), ("n", _L)]
+                ("max_blocks_per_seq", _I), ("block_size", _I), ("cache", _P), ("cache_dtype", _I), ("Q", _P), ("n", _L), ("norm_heads", _I)]
 
 
 class RotPost(ctypes.Structure):
@@ -351,18 +351,18 @@ class Gla(ctypes.Structure):
     """Mirror of i64h_gla_args (include/i64h_dense.h)."""
     _fields_ = [("P", _P), ("ldp", _L), ("q_off", _I), ("f_off", _I), ("k_off", _I), ("v_off", _I), ("heads", _I), ("dim", _I), ("vdim", _I),
                 ("lower", _P), ("q_act", _I), ("seg_start", _P), ("nseg", _I), ("positions", _P), ("slot_ids", _P), ("state", _P), ("out", _P),
-                ("ldo", _L), ("n", _L)]
+                ("ldo", _L), ("n", _L), ("F", _P), ("ldf", _L), ("q_scale", _F)]
 
 
 class Route(ctypes.Structure):
     """Mirror of i64h_route_args (include/i64h_dense.h)."""
     _fields_ = [("logits", _P), ("ld", _L), ("E", _I), ("correction", _P), ("groups", _I), ("keep", _I), ("top", _I), ("scale", _F), ("idx", _P),
-                ("wgt", _P), ("n", _L), ("h", _P), ("ldh", _L), ("W", _P), ("K", _I), ("bias", _P), ("chosen_softmax", _I), ("gate_out", _P)]
+                ("wgt", _P), ("n", _L), ("h", _P), ("ldh", _L), ("W", _P), ("K", _I), ("bias", _P), ("chosen_softmax", _I), ("gate_out", _P), ("sigmoid_scores", _I), ("raw_weights", _I)]
 
 
 class MoePlan(ctypes.Structure):
     """Mirror of i64h_moe_plan_args (include/i64h_dense.h)."""
-    _fields_ = [("idx", _P), ("n", _L), ("top", _I), ("experts", _I), ("group_off", _P), ("pair_token", _P), ("pair_row", _P)]
+    _fields_ = [("idx", _P), ("n", _L), ("top", _I), ("experts", _I), ("group_off", _P), ("pair_token", _P), ("pair_row", _P), ("wgt", _P), ("pair_wgt", _P)]
 
 
 class MoeCombine(ctypes.Structure):

@@ -90,6 +90,9 @@ class LatentAttentionConfig:
     rot_base: float = 10000.0
     rot_dims: int = 0        # leading dimensions of the rotated part that are rotated (the rest pass through)
     sink: bool = False       # a learned score per head in the softmax's denominator, without key or value (tensor 'sink')
+    q_rank: int = 0          # > 0: the queries come through a normed low-rank row of their own (tensors 'dq', 'dq.norm', 'uq' in the place of 'q')
+    head_gate: bool = False  # a sigmoid gate per head on its output (tensor 'g')
+    rot: "RotaryConfig | None" = None      # the rotation with its scaling, where a design scales frequencies
 
     @property
     def q_width(self) -> int:
@@ -100,33 +103,54 @@ class LatentAttentionConfig:
         return self.kv_rank + self.rot_dim
 
     @classmethod
-    def from_dict(cls, m: dict, sink: bool = False) -> "LatentAttentionConfig":
+    def from_dict(cls, m: dict, sink: bool = False, scaled_rotation: bool = False, **design) -> "LatentAttentionConfig":
         rot = m.get("rot") or {}
         rot_dim = int(m.get("rot_dim", 0))
         mask = m.get("mask") or {}
         c = cls(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=rot_dim, vdim=int(m["vdim"]), kv_rank=int(m["kv_rank"]),
                 scale=float(m["scale"]), window=int(mask.get("size", 0)), rot_base=float(rot.get("base", 10000.0)),
-                rot_dims=int(rot.get("dims", rot_dim)) if rot_dim else 0, sink=bool(sink))
+                rot_dims=int(rot.get("dims", rot_dim)) if rot_dim else 0, sink=bool(sink), q_rank=int(m.get("q_rank") or 0), **design)
+        if scaled_rotation and c.rot_dims:
+            c.rot = RotaryConfig.from_dict(dict(rot, base=c.rot_base, dims=c.rot_dims))
         if c.rot_dims > c.rot_dim or c.rot_dims % 2:
             raise ValueError(f"latent_attention: {c.rot_dims} rotated dimensions do not fit a rotated part of {c.rot_dim}")
-        if min(c.heads, c.dim, c.vdim, c.kv_rank) <= 0 or c.window < 0:
+        if min(c.heads, c.dim, c.vdim, c.kv_rank) <= 0 or c.window < 0 or c.q_rank < 0 or c.rot_dim < 0:
             raise ValueError(f"latent_attention: bad sizes {m}")
         return c
+
+    def to_dict(self) -> dict:
+        d = {"heads": self.heads, "dim": self.dim, "rot_dim": self.rot_dim, "vdim": self.vdim, "kv_rank": self.kv_rank, "scale": self.scale}
+        if self.q_rank:
+            d["q_rank"] = self.q_rank
+        if self.rot_dim:
+            d["rot"] = self.rot.to_dict() if self.rot is not None else {"base": self.rot_base, "dims": self.rot_dims}
+        if self.window:
+            d["mask"] = {"size": self.window}
+        return d
 
 
 @dataclass
 class DenseMlpConfig:
     ff: int
     kind: str = "dense"
+    # > 0: the gate is bounded from above by `limit` and the other factor u from both sides, g sigmoid(glu_alpha g) (u + 1)
+    limit: float = 0.0
+    glu_alpha: float = 1.702
 
     @classmethod
     def from_dict(cls, m: dict) -> "DenseMlpConfig":
         if m.get("kind", "dense") != "dense":
             raise ValueError(f"feed-forward kind '{m.get('kind')}' is not built")
-        return cls(ff=int(m["ff"]))
+        c = cls(ff=int(m["ff"]), limit=float(m.get("limit") or 0.0))
+        if c.ff <= 0 or c.limit < 0:
+            raise ValueError(f"dense feed-forward: bad sizes {m}")
+        return c
 
     def to_dict(self) -> dict:
-        return {"kind": "dense", "ff": self.ff}
+        d = {"kind": "dense", "ff": self.ff}
+        if self.limit:
+            d["limit"] = self.limit
+        return d
 
 
 @dataclass
@@ -149,10 +173,14 @@ class MoeMlpConfig:
     shared_limit: float = 0.0
     glu_alpha: float = 1.702
     # fixed by a design: a bias on the router's logits ('router.b'), choice and softmax on the chosen logits alone, a sigmoid gate per token
-    # on the shared expert ('shared.sg')
+    # on the shared expert ('shared.sg'); sigmoid scores in the place of the softmax, weights that are not renormalised, weights that multiply
+    # an expert's input instead of its output
     router_bias: bool = False
     chosen_softmax: bool = False
     shared_gate: bool = False
+    sigmoid_scores: bool = False
+    raw_weights: bool = False
+    weigh_input: bool = False
 
     @property
     def entries(self) -> int:
@@ -267,16 +295,22 @@ class MinGruConfig:
 
 @dataclass
 class ParallelMixerConfig:
-    """Two mixers that read the same input; the result is the mean of their separately normed outputs."""
+    """Two mixers that read the same input.  What a design makes of their results is its own: the mean of the separately normed outputs, or
+    the sum with a factor on either side."""
     left: KeyAttentionConfig
     right: MinGruConfig
+    left_scale: float = 1.0
+    right_scale: float = 1.0
 
     @classmethod
     def from_dict(cls, m: dict) -> "ParallelMixerConfig":
         return cls(left=KeyAttentionConfig.from_dict(m["left"]), right=MinGruConfig.from_dict(m["right"]))
 
     def to_dict(self) -> dict:
-        return {"left": self.left.to_dict(), "right": self.right.to_dict()}
+        d = {"left": self.left.to_dict(), "right": self.right.to_dict()}
+        if (self.left_scale, self.right_scale) != (1.0, 1.0):
+            d.update(left_scale=self.left_scale, right_scale=self.right_scale)
+        return d
 
 
 @dataclass
@@ -296,6 +330,27 @@ class Hgrn2Config:
 
     def to_dict(self) -> dict:
         return {"heads": self.heads, "dim": self.dim, "vdim": self.vdim}
+
+
+@dataclass
+class GatedLinearConfig:
+    """Gated linear attention: per head a (dim x vdim) matrix that decays by a factor per key channel, sigmoid(z)^(1 / tau) with z from a
+    low-rank map with a bias ('a1', 'a2', 'a2.b'), and receives k v^T; read by the query (times dim^-1/2) after the write.  The head outputs
+    pass an RMS norm over vdim and a silu gate ('g')."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float = 1.0
+
+    @classmethod
+    def from_dict(cls, m: dict) -> "GatedLinearConfig":
+        c = cls(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), tau=float(m.get("tau", 1.0)))
+        if min(c.heads, c.dim, c.vdim) <= 0 or c.tau <= 0:
+            raise ValueError(f"gated linear attention: bad sizes {m}")
+        return c
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "tau": self.tau}
 
 
 @dataclass
@@ -589,7 +644,7 @@ class RotaryConfig:
 class RotaryAttentionConfig:
     """Causal softmax attention over grouped key / value heads with separate key and value sizes and rotated positions.  What a design
     fixes comes in as flags: qk_norm 'row' (RMS norm over the whole projection with weights 'q.norm' / 'k.norm', before the rotation),
-    'head' (per head, without weights, after it) or None; interleaved pairs (2i, 2i + 1) or halves (i, i + dims / 2); rotated values
+    'head' (per head, without weights, after it), 'head_weight' (per head, weights of dim values that the heads share, before it) or None; interleaved pairs (2i, 2i + 1) or halves (i, i + dims / 2); rotated values
     (all vdim dimensions by the value's own position, the head's sum turned back by the query's); a sigmoid gate per head ('g')."""
     heads: int
     kv_heads: int
@@ -755,6 +810,28 @@ class LayerLoop:
     stop: int
     times: int
 
+    @classmethod
+    def from_dict(cls, lp: "dict | None", num_layers: int) -> "LayerLoop | None":
+        if not lp:
+            return None
+        c = cls(int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not 0 <= c.start < c.stop <= num_layers or c.times < 1:
+            raise ValueError(f"loop {lp} over {num_layers} layers")
+        return c
+
+    def to_dict(self) -> dict:
+        return {"start": self.start, "stop": self.stop, "times": self.times}
+
+
+def layer_runs(num_layers: int, loop: "LayerLoop | None") -> list:
+    """[(layer, number of the pass that begins in front of it or None)] in the order they run; run r has cache and state number r."""
+    if loop is None:
+        return [(i, None) for i in range(num_layers)]
+    runs = [(i, None) for i in range(loop.start)]
+    for t in range(loop.times):
+        runs += [(i, t if i == loop.start else None) for i in range(loop.start, loop.stop)]
+    return runs + [(i, None) for i in range(loop.stop, num_layers)]
+
 
 @dataclass
 class PukatarConfig:
@@ -779,25 +856,15 @@ class PukatarConfig:
         return 1 << 30
 
     def layer_runs(self) -> list:
-        """[(layer, number of the pass that begins in front of it or None)] in the order they run; run r has cache and state number r."""
-        n, lp = len(self.layers), self.loop
-        if lp is None:
-            return [(i, None) for i in range(n)]
-        runs = [(i, None) for i in range(lp.start)]
-        for t in range(lp.times):
-            runs += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
-        return runs + [(i, None) for i in range(lp.stop, n)]
+        return layer_runs(len(self.layers), self.loop)
 
     @classmethod
     def from_dict(cls, d: dict) -> "PukatarConfig":
         layers = [DecoderLayerConfig.from_dict(l, PUKATAR_MIXERS, PUKATAR_MLPS) for l in d["layers"]]
-        lp = d.get("loop")
         c = cls(vocab=int(d["vocab"]), width=int(d["width"]), layers=layers, norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)),
-                loop=LayerLoop(int(lp["start"]), int(lp["stop"]), int(lp["times"])) if lp else None, name=str(d.get("architecture", "Pukatar")))
+                loop=LayerLoop.from_dict(d.get("loop"), len(layers)), name=str(d.get("architecture", "Pukatar")))
         if min(c.vocab, c.width) <= 0 or not layers:
             raise ValueError("bad sizes")
-        if c.loop is not None and (not 0 <= c.loop.start < c.loop.stop <= len(layers) or c.loop.times < 1):
-            raise ValueError(f"loop {lp} over {len(layers)} layers")
         for i, l in enumerate(layers):
             if l.weights_of is not None:
                 raise ValueError(f"layer {i}: this design has no layers that borrow tensors")
@@ -809,5 +876,75 @@ class PukatarConfig:
         d = {"architecture": "Pukatar", "vocab": self.vocab, "width": self.width, "norm": {"eps": self.norm_eps},
              "layers": [{"type": l.type, "mixer": l.mixer.to_dict(), "mlp": l.mlp.to_dict() if l.mlp else None} for l in self.layers]}
         if self.loop is not None:
-            d["loop"] = {"start": self.loop.start, "stop": self.loop.stop, "times": self.loop.times}
+            d["loop"] = self.loop.to_dict()
+        return d
+
+
+# ---------------------------------------------------------------------------------------------------------------------------
+# Vepelix: a pre-norm decoder (RMS norms whose weights are distances from one, a learned factor per column on every sublayer's result) with a
+# stretch of layers repeated with the same weights, every further pass starting from the residual plus the embedding; per layer one of two
+# mixers - latent attention with low-rank queries, a rotated shared key part, sinks and gated heads, or a windowed attention beside a gated
+# linear attention - and one of two feed-forwards, a clamped gated one or a mixture of experts whose weights multiply the experts' input.
+# Every size and constant comes from config.json.
+# ---------------------------------------------------------------------------------------------------------------------------
+def _vepelix_latent(m: dict) -> LatentAttentionConfig:
+    c = LatentAttentionConfig.from_dict(m, sink=True, scaled_rotation=True, head_gate=True)
+    if c.q_rank <= 0:
+        raise ValueError("latent attention of this design takes its queries through a latent: 'q_rank' is missing")
+    return c
+
+
+def _vepelix_parallel(m: dict) -> ParallelMixerConfig:
+    return ParallelMixerConfig(left=RotaryAttentionConfig.from_dict(m["left"], qk_norm="head_weight", interleaved=True), right=GatedLinearConfig.from_dict(m["right"]),
+                               left_scale=float(m.get("left_scale", 1.0)), right_scale=float(m.get("right_scale", 1.0)))
+
+
+VEPELIX_MIXERS = {"latent_attention": _vepelix_latent, "parallel": _vepelix_parallel}
+VEPELIX_MLPS = {"dense": DenseMlpConfig, "moe": lambda m: MoeMlpConfig.from_dict(m, sigmoid_scores=True, raw_weights=True, weigh_input=True)}
+
+
+@dataclass
+class VepelixConfig:
+    vocab: int
+    width: int
+    layers: list
+    norm_eps: float = 1e-6
+    loop: "LayerLoop | None" = None
+    name: str = "Vepelix"
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def vocab_size(self) -> int:
+        return self.vocab
+
+    @property
+    def max_pos(self) -> int:
+        """Positions are computed, not tabulated: a sequence is bounded by the page pool only."""
+        return 1 << 30
+
+    def layer_runs(self) -> list:
+        return layer_runs(len(self.layers), self.loop)
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "VepelixConfig":
+        layers = [DecoderLayerConfig.from_dict(l, VEPELIX_MIXERS, VEPELIX_MLPS) for l in d["layers"]]
+        c = cls(vocab=int(d["vocab"]), width=int(d["width"]), layers=layers, norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)),
+                loop=LayerLoop.from_dict(d.get("loop"), len(layers)), name=str(d.get("architecture", "Vepelix")))
+        if min(c.vocab, c.width) <= 0 or not layers:
+            raise ValueError("bad sizes")
+        for i, l in enumerate(layers):
+            if l.weights_of is not None:
+                raise ValueError(f"layer {i}: this design has no layers that borrow tensors")
+            if l.mlp is not None and l.mlp.kind == "dense" and l.mlp.limit <= 0:
+                raise ValueError(f"layer {i}: the dense feed-forwards of this design are clamped, 'limit' is missing")
+        return c
+
+    def to_dict(self) -> dict:
+        d = {"architecture": "Vepelix", "vocab": self.vocab, "width": self.width, "norm": {"eps": self.norm_eps},
+             "layers": [{"type": l.type, "mixer": l.mixer.to_dict(), "mlp": l.mlp.to_dict() if l.mlp else None} for l in self.layers]}
+        if self.loop is not None:
+            d["loop"] = self.loop.to_dict()
         return d

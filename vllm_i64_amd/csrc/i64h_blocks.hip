@@ -1,11 +1,13 @@
 // Kernels of libi64hip_dense.so for gated linear recurrences and mixtures of experts (include/i64h_dense.h):
 //   gla_gates_kernel   : query activation and bounded forget gate, in place on the projection rows
-//   gla_scan_kernel    : linear attention with a decay per key channel, a head's matrix in registers (16 lanes per value column)
+//   gla_scan_kernel    : linear attention with a decay per key channel whose keys are one minus the decay, a head's matrix in registers (16
+//                        lanes per value column)
 //   gdn_gates_kernel / gdn_scan_kernel : gated delta rule - unit-vector queries and keys, write strength and decay; the recurrence with the
-//                        correction S^T k summed over the DPP row before the write, the read-out after it; a decay per head or per key channel
+//                        correction S^T k summed over the DPP row before the write, the read-out after it; a decay per head or per key channel;
+//                        without the correction: gated linear attention with keys of its own
 //   gdn_tile_kernel    : the same recurrence for long runs, tokens staged through LDS
-//   route_topk_kernel  : softmax scores (over all entries or the chosen ones), corrected choice, groups of neighbours, top-k and normalised
-//                        weights, one wave per row
+//   route_topk_kernel  : softmax scores (over all entries or the chosen ones) or sigmoid scores, corrected choice, groups of neighbours, top-k and normalised
+//                        (or raw) weights, one wave per row
 //   moe_plan_kernel    : (token, choice) pairs grouped by expert: offsets, the token of every grouped row, the row of every pair
 //   moe_combine_kernel : weighted sum of the chosen experts' rows, pass-through entries and the shared expert's row
 // A row continues the row before it iff slot and position say so; state is taken as empty at position 0.  All arithmetic fp32.
@@ -29,13 +31,13 @@ __global__ __launch_bounds__(256) void gla_gates_kernel(const i64h_gla_args p) {
 }
 
 // One workgroup per (head, 16 * CPT value columns, run of rows).  The 16 lanes of a DPP row share CPT neighbouring value columns and hold
-// KPT consecutive key channels of each in registers; a wave has four such rows.  Per token a lane loads its slices of the query, the
-// decay and (where it is not one minus the decay) the key once for its CPT columns, updates its states with fused multiply-adds and
+// KPT consecutive key channels of each in registers; a wave has four such rows.  The key is one minus the decay (keys of their own: the
+// delta rule's kernels below, without its correction).  Per token a lane loads its slices of the query and the decay once for its CPT columns, updates its states with fused multiply-adds and
 // the row sums the partial outputs with DPP moves: no LDS and no barrier, the tokens of a run strictly in their order (the same sums in
 // the same order however a prompt is cut).  Loads run GL_TG tokens ahead in two alternating register sets, so that a wave that is alone
 // on its SIMD still has a group of tokens in flight while it computes one.  State layout [slot, head, value column, key channel].
 #define GL_TG 4
-template <int KPT, int CPT, bool HASK>
+template <int KPT, int CPT>
 __global__ __launch_bounds__(256) void gla_scan_kernel(const i64h_gla_args p, const int ctiles, const int vec) {
     const int N = p.dim, P = p.vdim;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -69,33 +71,33 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(const i64h_gla_args p, co
             }
         }
     }
-    const int qoff = p.q_off + a * N + n0, foff = p.f_off + a * N + n0, koff = HASK ? p.k_off + a * N + n0 : 0;
+    const int qoff = p.q_off + a * N + n0, foff = p.f_off + a * N + n0;
+    const float* const F = p.F ? p.F : p.P;
+    const int64_t ldf = p.F ? p.ldf : p.ldp;
     struct Tok {
-        float q[KPT], f[KPT], k[HASK ? KPT : 1], v[CPT];
+        float q[KPT], f[KPT], v[CPT];
     };
     auto fetch = [&](int64_t t, Tok& u) {
         if (t >= r1) return;
         const float* row = p.P + t * p.ldp;
+        const float* frow = F + t * ldf;
         if (vec) {      // KPT % 4 == 0 and every slice starts at a multiple of four floats and lies inside the row
 #pragma unroll
             for (int k = 0; k < KPT; k += 4) {
-                float4 q = make_float4(0, 0, 0, 0), f = make_float4(1, 1, 1, 1), kk = q;
+                float4 q = make_float4(0, 0, 0, 0), f = make_float4(1, 1, 1, 1);
                 if (n0 + k < N) {
                     q = *(const float4*)(row + qoff + k);
-                    f = *(const float4*)(row + foff + k);
-                    if (HASK) kk = *(const float4*)(row + koff + k);
+                    f = *(const float4*)(frow + foff + k);
                 }
                 u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
                 u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
-                if (HASK) u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
             }
         } else {
 #pragma unroll
             for (int k = 0; k < KPT; ++k) {
                 const bool ok = n0 + k < N;
                 u.q[k] = ok ? row[qoff + k] : 0.0f;
-                u.f[k] = ok ? row[foff + k] : 1.0f;
-                if (HASK) u.k[k] = ok ? row[koff + k] : 0.0f;
+                u.f[k] = ok ? frow[foff + k] : 1.0f;
             }
         }
 #pragma unroll
@@ -108,12 +110,11 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(const i64h_gla_args p, co
             float part = 0.0f;
 #pragma unroll
             for (int k = 0; k < KPT; ++k) {
-                const float kk = HASK ? u.k[k] : 1.0f - u.f[k];
-                S[j][k] = fmaf(u.f[k], S[j][k], kk * u.v[j]);
+                S[j][k] = fmaf(u.f[k], S[j][k], (1.0f - u.f[k]) * u.v[j]);
                 part = fmaf(S[j][k], u.q[k], part);
             }
             part = group_sum(part, 16);
-            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = part;
+            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = part * p.q_scale;
         }
     };
     Tok A[GL_TG], B[GL_TG];
@@ -177,14 +178,15 @@ __global__ __launch_bounds__(256) void gdn_gates_kernel(const i64h_gdn_args p) {
 // row share CPT value columns and hold KPT key channels of each in registers).  Per token the state decays, the row sums S^T k with DPP
 // moves (every lane of the row ends with the sum), the correction along k is written, and a second row sum reads the state out with
 // the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order; loads run TG tokens ahead.
-// CHD: a decay per head and key channel (F) in the place of one per head.
+// CHD: a decay per head and key channel (F) in the place of one per head.  RULE: the delta rule's correction and write strength; without it the
+// token writes k v^T as it is (gated linear attention) and the read-out is multiplied by q_scale.
 // TG is chosen so that two waves fit a SIMD's registers (the loads in flight are most of them); one where every run is a single row.
 // A lane's KPT channels: four neighbours in every stripe of 64 (so that 16 lanes read 256 consecutive bytes at a time).
 template <int KPT>
 __device__ __forceinline__ int gd_channel(int nlane, int k) {
     return KPT >= 4 ? 4 * (nlane + 16 * (k >> 2)) + (k & 3) : nlane * KPT + k;
 }
-template <int KPT, int CPT, bool CHD, int TG>
+template <int KPT, int CPT, bool CHD, int TG, bool RULE>
 __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, const int ctiles, const int vec) {
     const int N = p.dim, P = p.vdim;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -250,29 +252,37 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
         }
 #pragma unroll
         for (int j = 0; j < CPT; ++j) u.v[j] = cbase + j < P ? row[p.v_off + a * P + cbase + j] : 0.0f;
-        u.beta = p.G[t * 2 * p.heads + a];
+        if (RULE) u.beta = p.G[t * 2 * p.heads + a];
         if (!CHD) u.f[0] = p.G[t * 2 * p.heads + p.heads + a];
     };
     auto step = [&](int64_t t, const Tok& u) {
         if (t >= r1) return;
 #pragma unroll
         for (int j = 0; j < CPT; ++j) {
-            float seen = 0.0f;
-#pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                S[j][k] *= u.f[CHD ? k : 0];
-                seen = fmaf(S[j][k], u.k[k], seen);
-            }
-            seen = group_sum(seen, 16);
-            const float d = u.beta * (u.v[j] - seen);
             float part = 0.0f;
+            if (RULE) {
+                float seen = 0.0f;
 #pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                S[j][k] = fmaf(u.k[k], d, S[j][k]);
-                part = fmaf(S[j][k], u.q[k], part);
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] *= u.f[CHD ? k : 0];
+                    seen = fmaf(S[j][k], u.k[k], seen);
+                }
+                seen = group_sum(seen, 16);
+                const float d = u.beta * (u.v[j] - seen);
+#pragma unroll
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] = fmaf(u.k[k], d, S[j][k]);
+                    part = fmaf(S[j][k], u.q[k], part);
+                }
+            } else {
+#pragma unroll
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], u.k[k] * u.v[j]);
+                    part = fmaf(S[j][k], u.q[k], part);
+                }
             }
             part = group_sum(part, 16);
-            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = part;
+            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = RULE ? part : part * p.q_scale;
         }
     };
     Tok A[TG], B[TG];
@@ -307,7 +317,7 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
 // gdn_tile_kernel: the same recurrence, bit for bit, for runs of many rows.  What every wave of a workgroup reads of a token (query, key,
 // decays) is loaded once per workgroup, TT tokens at a time, into one of two LDS tiles while the other one is computed: the loads of a
 // tile have the arithmetic of a whole tile to arrive, and the waves read 16 bytes per lane from LDS one token ahead.  Needs 16-byte rows.
-template <int KPT, int CPT, bool CHD>
+template <int KPT, int CPT, bool CHD, bool RULE>
 __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, const int ctiles) {
     static_assert(KPT % 4 == 0, "whole 16-byte slices per lane");
     constexpr int TT = KPT > 8 ? 8 : 16;      // tokens per tile
@@ -360,7 +370,7 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
         }
         if (tid < 2 * TT) {
             const int64_t t = t0 + (tid >> 1);
-            sg = (t < r1 && !(CHD && (tid & 1))) ? p.G[t * 2 * p.heads + (tid & 1) * p.heads + a] : 0.0f;
+            sg = (t < r1 && (RULE || (tid & 1)) && !(CHD && (tid & 1))) ? p.G[t * 2 * p.heads + (tid & 1) * p.heads + a] : 0.0f;
         }
     };
     auto lstore = [&](int b) {
@@ -397,6 +407,23 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
     };
     auto step = [&](int64_t t, const Tok& u) {
         float seen[CPT], part[CPT], d[CPT];
+        if (!RULE) {
+#pragma unroll
+            for (int j = 0; j < CPT; ++j) {
+                part[j] = 0.0f;
+#pragma unroll
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], u.k[k] * u.v[j]);
+                    part[j] = fmaf(S[j][k], u.q[k], part[j]);
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < CPT; ++j) {
+                const float o = group_sum(part[j], 16);
+                if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = o * p.q_scale;
+            }
+            return;
+        }
 #pragma unroll
         for (int j = 0; j < CPT; ++j) {
             seen[j] = 0.0f;
@@ -516,7 +543,13 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
         const float* z = p.logits + t * p.ld;
         for (int e = lane; e < E; e += 64) ch[e] = p.bias ? z[e] + p.bias[e] : z[e];
     }
-    if (p.chosen_softmax) {     // the choice falls on the logits themselves
+    if (p.sigmoid_scores) {     // scores of their own, in the logits' order: the choice falls on the logits unless it is corrected
+        for (int e = lane; e < E; e += 64) {
+            const float s = bl_sigmoid(ch[e]);
+            sc[e] = s;
+            if (p.correction) ch[e] = s + p.correction[e];
+        }
+    } else if (p.chosen_softmax) {     // the choice falls on the logits themselves
         for (int e = lane; e < E; e += 64) {
             const float s = ch[e];
             sc[e] = s;
@@ -585,7 +618,7 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
     }
     if (lane < p.top) {
         p.idx[t * p.top + lane] = mine_i;
-        p.wgt[t * p.top + lane] = mine_w / (wsum + 1e-20f) * p.scale;
+        p.wgt[t * p.top + lane] = (p.raw_weights ? mine_w : mine_w / (wsum + 1e-20f)) * p.scale;
     }
 }
 
@@ -621,6 +654,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const i64h_moe_plan_args
         if (e >= 0 && e < p.experts) {
             r = atomicAdd(&cur[e], 1);
             p.pair_token[r] = (int)(i / p.top);
+            if (p.pair_wgt) p.pair_wgt[r] = p.wgt[i];
         }
         p.pair_row[i] = r;
     }
@@ -634,7 +668,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const i64h_moe_combine
         for (int k = 0; k < p.top; ++k) {
             const int r = p.pair_row[t * p.top + k];
             const float v = r >= 0 ? p.Y[(int64_t)r * W + c] : p.h[t * W + c];
-            a += p.wgt[t * p.top + k] * v;
+            a += p.wgt ? p.wgt[t * p.top + k] * v : v;
         }
         if (p.shared) a += p.shared_gate ? p.shared_gate[t] * p.shared[t * W + c] : p.shared[t * W + c];
         p.out[t * W + c] = a;
@@ -661,45 +695,10 @@ int i64h_gla_gates(const i64h_gla_args* dp, void* stream) {
     return 0;
 }
 
-int i64h_gla_scan(const i64h_gla_args* dp, void* stream) {
-    I64H_CHECK_ARG(dp != nullptr, "gla_scan: no descriptor");
-    const i64h_gla_args& d = *dp;
-    if (gla_check(d, "gla_scan")) return 1;
-    I64H_CHECK_ARG(d.seg_start && d.positions && d.slot_ids && d.state && d.out, "gla_scan: null operand");
-    I64H_CHECK_ARG(d.dim <= 16 * 16, "gla_scan: dim %d above 256", d.dim);
-    I64H_CHECK_ARG(d.nseg <= 65535, "gla_scan: %d runs in one launch", d.nseg);
-    if (d.nseg <= 0 || d.n == 0) return 0;
-    const int kpt = (d.dim + 15) / 16;
-    // columns per lane: query, decay and key are loaded once for both - unless the launch would then leave most of the chip idle
-    const int cpt = (d.vdim > 16 && (int64_t)d.heads * ((d.vdim + 31) / 32) * d.nseg >= 512) ? 2 : 1;
-    const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
-    const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
-    const bool hask = d.k_off >= 0;
-    auto launch = [&](auto kern, int K) {
-        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldp % 4 == 0 && d.q_off % 4 == 0 && d.f_off % 4 == 0 && (!hask || d.k_off % 4 == 0) &&
-                        (uintptr_t)d.P % 16 == 0 && (uintptr_t)d.state % 16 == 0;
-        hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
-    };
-#define GLA_PICK(C, HK)                                          \
-    if (kpt <= 1) launch(gla_scan_kernel<1, C, HK>, 1);          \
-    else if (kpt <= 2) launch(gla_scan_kernel<2, C, HK>, 2);     \
-    else if (kpt <= 4) launch(gla_scan_kernel<4, C, HK>, 4);     \
-    else if (kpt <= 8) launch(gla_scan_kernel<8, C, HK>, 8);     \
-    else launch(gla_scan_kernel<16, C, HK>, 16);
-    if (cpt == 2) {
-        if (hask) { GLA_PICK(2, true) } else { GLA_PICK(2, false) }
-    } else {
-        if (hask) { GLA_PICK(1, true) } else { GLA_PICK(1, false) }
-    }
-#undef GLA_PICK
-    I64H_CHECK_LAUNCH();
-    return 0;
-}
-
 static int gdn_check(const i64h_gdn_args& d, const char* what) {
     I64H_CHECK_ARG(d.heads > 0 && d.kv_heads > 0 && d.heads % d.kv_heads == 0 && d.dim > 0 && d.vdim > 0 && d.n >= 0, "%s: heads %d, query / key heads %d, dim %d, vdim %d",
                    what, d.heads, d.kv_heads, d.dim, d.vdim);
-    I64H_CHECK_ARG(d.X && d.G && d.q_off >= 0 && d.k_off >= 0 && d.v_off >= 0, "%s: null operand or negative column", what);
+    I64H_CHECK_ARG(d.X && d.q_off >= 0 && d.k_off >= 0 && d.v_off >= 0, "%s: null operand or negative column", what);
     return 0;
 }
 
@@ -707,7 +706,7 @@ int i64h_gdn_gates(const i64h_gdn_args* dp, void* stream) {
     I64H_CHECK_ARG(dp != nullptr, "gdn_gates: no descriptor");
     const i64h_gdn_args& d = *dp;
     if (gdn_check(d, "gdn_gates")) return 1;
-    I64H_CHECK_ARG(d.R && d.b_off >= 0 && (d.a_off < 0 || (d.A_log && d.dt_bias)), "gdn_gates: null operand or negative column");
+    I64H_CHECK_ARG(d.G && d.R && d.b_off >= 0 && (d.a_off < 0 || (d.A_log && d.dt_bias)), "gdn_gates: null operand or negative column");
     if (d.n == 0) return 0;
     hipLaunchKernelGGL(gdn_gates_kernel, dim3((unsigned)d.n), dim3(256), 0, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();
@@ -721,14 +720,10 @@ int i64h_set_gdn_scan_form(int32_t form) {
     return 0;
 }
 
-int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
-    I64H_CHECK_ARG(dp != nullptr, "gdn_scan: no descriptor");
-    const i64h_gdn_args& d = *dp;
-    if (gdn_check(d, "gdn_scan")) return 1;
-    I64H_CHECK_ARG(d.seg_start && d.positions && d.slot_ids && d.state && d.out, "gdn_scan: null operand");
-    I64H_CHECK_ARG(d.dim <= 16 * 16, "gdn_scan: dim %d above 256", d.dim);
-    I64H_CHECK_ARG(d.nseg <= 65535, "gdn_scan: %d runs in one launch", d.nseg);
-    if (d.nseg <= 0 || d.n == 0) return 0;
+// the recurrence's launch, with the delta rule's correction or (RULE = false: a decay per key channel, keys of every head's own) without it
+extern "C++" {
+template <bool RULE>
+static int gdn_launch(const i64h_gdn_args& d, void* stream) {
     const int kpt = (d.dim + 15) / 16;
     auto vec_ok = [&](int K) {
         return K % 4 == 0 && d.dim % 4 == 0 && d.ldx % 4 == 0 && d.q_off % 4 == 0 && d.k_off % 4 == 0 && (uintptr_t)d.X % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
@@ -741,13 +736,13 @@ int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
         const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
         const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
         auto launch = [&](auto kern) { hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles); };
-#define GDN_TILE(C, CHD)                                      \
-    if (kround == 4) launch(gdn_tile_kernel<4, C, CHD>);      \
-    else if (kround == 8) launch(gdn_tile_kernel<8, C, CHD>); \
-    else launch(gdn_tile_kernel<16, C, CHD>);
-        if (d.F) {
+#define GDN_TILE(C, CHD)                                            \
+    if (kround == 4) launch(gdn_tile_kernel<4, C, CHD, RULE>);      \
+    else if (kround == 8) launch(gdn_tile_kernel<8, C, CHD, RULE>); \
+    else launch(gdn_tile_kernel<16, C, CHD, RULE>);
+        if (!RULE || d.F) {
             if (cpt == 1) { GDN_TILE(1, true) } else if (cpt == 2) { GDN_TILE(2, true) } else { GDN_TILE(4, true) }
-        } else {
+        } else if constexpr (RULE) {
             if (cpt == 1) { GDN_TILE(1, false) } else if (cpt == 2) { GDN_TILE(2, false) } else { GDN_TILE(4, false) }
         }
 #undef GDN_TILE
@@ -763,21 +758,71 @@ int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
         const int vec = vec_ok(K);
         hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
     };
-#define GDN_PICK(C, CHD, ONE)                                                              \
-    if (kpt <= 1) launch(gdn_scan_kernel<1, C, CHD, ONE ? 1 : 4>, 1);                       \
-    else if (kpt <= 2) launch(gdn_scan_kernel<2, C, CHD, ONE ? 1 : 4>, 2);                  \
-    else if (kpt <= 4) launch(gdn_scan_kernel<4, C, CHD, ONE ? 1 : 4>, 4);                  \
-    else if (kpt <= 8) launch(gdn_scan_kernel<8, C, CHD, ONE ? 1 : (CHD ? 2 : 4)>, 8);      \
-    else launch(gdn_scan_kernel<16, C, CHD, ONE ? 1 : (CHD ? 1 : 2)>, 16);
+#define GDN_PICK(C, CHD, ONE)                                                                    \
+    if (kpt <= 1) launch(gdn_scan_kernel<1, C, CHD, ONE ? 1 : 4, RULE>, 1);                       \
+    else if (kpt <= 2) launch(gdn_scan_kernel<2, C, CHD, ONE ? 1 : 4, RULE>, 2);                  \
+    else if (kpt <= 4) launch(gdn_scan_kernel<4, C, CHD, ONE ? 1 : 4, RULE>, 4);                  \
+    else if (kpt <= 8) launch(gdn_scan_kernel<8, C, CHD, ONE ? 1 : (CHD ? 2 : 4), RULE>, 8);      \
+    else launch(gdn_scan_kernel<16, C, CHD, ONE ? 1 : (CHD ? 1 : 2), RULE>, 16);
 #define GDN_PICK2(C, CHD) \
     if (d.nseg == d.n) { GDN_PICK(C, CHD, true) } else { GDN_PICK(C, CHD, false) }
-    if (d.F) {
+    if (!RULE || d.F) {
         if (cpt == 2) { GDN_PICK2(2, true) } else { GDN_PICK2(1, true) }
-    } else {
+    } else if constexpr (RULE) {
         if (cpt == 2) { GDN_PICK2(2, false) } else { GDN_PICK2(1, false) }
     }
 #undef GDN_PICK2
 #undef GDN_PICK
+    I64H_CHECK_LAUNCH();
+    return 0;
+}
+}
+
+int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
+    I64H_CHECK_ARG(dp != nullptr, "gdn_scan: no descriptor");
+    const i64h_gdn_args& d = *dp;
+    if (gdn_check(d, "gdn_scan")) return 1;
+    I64H_CHECK_ARG(d.G && d.seg_start && d.positions && d.slot_ids && d.state && d.out, "gdn_scan: null operand");
+    I64H_CHECK_ARG(d.dim <= 16 * 16, "gdn_scan: dim %d above 256", d.dim);
+    I64H_CHECK_ARG(d.nseg <= 65535, "gdn_scan: %d runs in one launch", d.nseg);
+    if (d.nseg <= 0 || d.n == 0) return 0;
+    return gdn_launch<true>(d, stream);
+}
+
+int i64h_gla_scan(const i64h_gla_args* dp, void* stream) {
+    I64H_CHECK_ARG(dp != nullptr, "gla_scan: no descriptor");
+    const i64h_gla_args& d = *dp;
+    if (gla_check(d, "gla_scan")) return 1;
+    I64H_CHECK_ARG(d.seg_start && d.positions && d.slot_ids && d.state && d.out, "gla_scan: null operand");
+    I64H_CHECK_ARG(d.dim <= 16 * 16, "gla_scan: dim %d above 256", d.dim);
+    I64H_CHECK_ARG(d.nseg <= 65535, "gla_scan: %d runs in one launch", d.nseg);
+    I64H_CHECK_ARG(!d.F || d.ldf >= d.f_off + (int64_t)d.heads * d.dim, "gla_scan: the decays' rows are shorter than their columns");
+    if (d.nseg <= 0 || d.n == 0) return 0;
+    if (d.k_off >= 0) {      // keys of their own: the delta rule's kernels without the correction
+        i64h_gdn_args a = {};
+        a.X = d.P, a.ldx = d.ldp, a.q_off = d.q_off, a.k_off = d.k_off, a.v_off = d.v_off, a.heads = a.kv_heads = d.heads, a.dim = d.dim, a.vdim = d.vdim;
+        a.F = (d.F ? d.F : d.P) + d.f_off, a.ldf = d.F ? d.ldf : d.ldp, a.q_scale = d.q_scale, a.seg_start = d.seg_start, a.nseg = d.nseg;
+        a.positions = d.positions, a.slot_ids = d.slot_ids, a.state = d.state, a.out = d.out, a.ldo = d.ldo, a.n = d.n;
+        return gdn_launch<false>(a, stream);
+    }
+    const int kpt = (d.dim + 15) / 16;
+    // columns per lane: query and decay are loaded once for both - unless the launch would then leave most of the chip idle
+    const int cpt = (d.vdim > 16 && (int64_t)d.heads * ((d.vdim + 31) / 32) * d.nseg >= 512) ? 2 : 1;
+    const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
+    const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
+    auto launch = [&](auto kern, int K) {
+        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldp % 4 == 0 && d.q_off % 4 == 0 && d.f_off % 4 == 0 && (uintptr_t)d.P % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
+                        (!d.F || (d.ldf % 4 == 0 && (uintptr_t)d.F % 16 == 0));
+        hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
+    };
+#define GLA_PICK(C)                                          \
+    if (kpt <= 1) launch(gla_scan_kernel<1, C>, 1);          \
+    else if (kpt <= 2) launch(gla_scan_kernel<2, C>, 2);     \
+    else if (kpt <= 4) launch(gla_scan_kernel<4, C>, 4);     \
+    else if (kpt <= 8) launch(gla_scan_kernel<8, C>, 8);     \
+    else launch(gla_scan_kernel<16, C>, 16);
+    if (cpt == 2) { GLA_PICK(2) } else { GLA_PICK(1) }
+#undef GLA_PICK
     I64H_CHECK_LAUNCH();
     return 0;
 }
@@ -787,6 +832,7 @@ int i64h_route_topk(const i64h_route_args* dp, void* stream) {
     const i64h_route_args& d = *dp;
     I64H_CHECK_ARG(d.E > 0 && d.E <= 1024 && d.top > 0 && d.top <= RT_MAX_TOP && d.top <= d.E, "route_topk: %d entries (at most 1024), top %d (at most %d)", d.E, d.top, RT_MAX_TOP);
     I64H_CHECK_ARG(d.groups <= 1 || (d.E % d.groups == 0 && d.keep >= 1 && d.keep <= d.groups), "route_topk: %d entries in %d groups, %d kept", d.E, d.groups, d.keep);
+    I64H_CHECK_ARG(!d.sigmoid_scores || !d.chosen_softmax, "route_topk: sigmoid scores, or the softmax over the chosen logits");
     I64H_CHECK_ARG(!d.gate_out || d.W, "route_topk: the gate's row lies behind the router's rows");
     I64H_CHECK_ARG(d.groups <= 1 || d.keep * (d.E / d.groups) >= d.top, "route_topk: %d kept groups of %d entries hold fewer than top %d", d.keep, d.E / (d.groups > 0 ? d.groups : 1), d.top);
     I64H_CHECK_ARG(d.idx && d.wgt && ((d.logits && d.ld >= d.E) || (d.W && d.h && d.K > 0 && d.ldh >= d.K)), "route_topk: null operand or row stride below the row");
@@ -803,6 +849,7 @@ int i64h_moe_plan(const i64h_moe_plan_args* dp, void* stream) {
     I64H_CHECK_ARG(d.experts > 0 && d.experts <= 4096 && d.top > 0 && d.n >= 0, "moe_plan: %d experts (at most 4096), top %d", d.experts, d.top);
     I64H_CHECK_ARG(d.idx && d.group_off && d.pair_token && d.pair_row, "moe_plan: null operand");
     I64H_CHECK_ARG(d.n * d.top < (1ll << 31), "moe_plan: too many pairs");
+    I64H_CHECK_ARG(!d.pair_wgt || d.wgt, "moe_plan: weights per row come from the weights per choice");
     hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), (size_t)(2 * d.experts + 1) * 4, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();
     return 0;
@@ -812,7 +859,7 @@ int i64h_moe_combine(const i64h_moe_combine_args* dp, void* stream) {
     I64H_CHECK_ARG(dp != nullptr, "moe_combine: no descriptor");
     const i64h_moe_combine_args& d = *dp;
     I64H_CHECK_ARG(d.top > 0 && d.W > 0 && d.n >= 0, "moe_combine: top %d, width %d", d.top, d.W);
-    I64H_CHECK_ARG(d.Y && d.pair_row && d.wgt && d.h && d.out, "moe_combine: null operand");
+    I64H_CHECK_ARG(d.Y && d.pair_row && d.h && d.out, "moe_combine: null operand");
     if (d.n == 0) return 0;
     hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)d.n), dim3(256), 0, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();

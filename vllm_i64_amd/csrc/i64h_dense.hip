@@ -46,6 +46,10 @@ constexpr bool dn_dual(int epi) { return epi == I64H_EPI_GELU_MUL || epi == I64H
 
 template <int EPI>
 __device__ __forceinline__ float dn_epilogue(const i64h_linear& p, float acc, float acc2, int64_t b, int64_t r, int c) {
+    if (dn_dual(EPI) && p.row_scale) {      // a factor on the input row
+        const float s = p.row_scale[r];
+        acc *= s, acc2 *= s;
+    }
     if (EPI == I64H_EPI_GELU_MUL) return dn_gelu_tanh(acc) * acc2;
     if (EPI == I64H_EPI_SILU_MUL) return acc * dn_sigmoid(acc) * acc2;
     if (EPI == I64H_EPI_CLAMP_GLU) {
@@ -58,6 +62,7 @@ __device__ __forceinline__ float dn_epilogue(const i64h_linear& p, float acc, fl
     if (EPI == I64H_EPI_GELU_ERF) return dn_gelu_erf(acc);
     if (EPI == I64H_EPI_SCALE) return acc * p.scale;
     if (EPI == I64H_EPI_MUL_SIGMOID) return acc * dn_sigmoid(p.E[b * p.e_batch + r * p.lde + c]);
+    if (EPI == I64H_EPI_ROW_SIGMOID) return acc * dn_sigmoid(p.E[b * p.e_batch + r * p.lde]);
     if (EPI == I64H_EPI_SOFTCAP) return p.softcap * tanhf(acc / p.softcap);
     if (EPI == I64H_EPI_ADD) return acc + p.E[b * p.e_batch + r * p.lde + c];
     if (EPI == I64H_EPI_DECAY) return expf(-p.E[b * p.e_batch + r * p.lde + c] * dn_softplus(acc));
@@ -708,6 +713,7 @@ static void launch_tile(const i64h_linear& d, dim3 grid, hipStream_t s, int vecA
         case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_RELU_SQ>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_ADD: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_ADD>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_DECAY>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+        case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_ROW_SIGMOID>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_SCALE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         default: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_STORE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
     }
@@ -734,11 +740,12 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
     const i64h_linear& d = *dp;
     I64H_CHECK_ARG(d.M >= 0 && d.N > 0 && d.K > 0 && d.batch > 0, "linear: bad sizes M=%lld N=%d K=%d batch=%d", (long long)d.M, d.N, d.K, d.batch);
     I64H_CHECK_ARG(d.A && d.W && d.C, "linear: null operand");
-    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_DECAY, "linear: epilogue %d", d.epilogue);
-    I64H_CHECK_ARG((d.epilogue != I64H_EPI_MUL_SIGMOID && d.epilogue != I64H_EPI_ADD && d.epilogue != I64H_EPI_DECAY) || d.E, "linear: epilogue %d needs E", d.epilogue);
+    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_ROW_SIGMOID, "linear: epilogue %d", d.epilogue);
+    I64H_CHECK_ARG((d.epilogue != I64H_EPI_MUL_SIGMOID && d.epilogue != I64H_EPI_ADD && d.epilogue != I64H_EPI_DECAY && d.epilogue != I64H_EPI_ROW_SIGMOID) || d.E, "linear: epilogue %d needs E", d.epilogue);
     I64H_CHECK_ARG(d.epilogue != I64H_EPI_CLAMP_GLU || d.act_b > 0.0f, "linear: bound %g of the clamped gate / up epilogue", (double)d.act_b);
     I64H_CHECK_ARG(d.epilogue != I64H_EPI_SOFTCAP || d.softcap > 0.0f, "linear: soft cap %g", (double)d.softcap);
     I64H_CHECK_ARG(!dn_dual(d.epilogue) || !d.bias, "linear: the gate / up epilogues take no bias");
+    I64H_CHECK_ARG(dn_dual(d.epilogue) || !d.row_scale, "linear: row factors belong to the gate / up epilogues");
     I64H_CHECK_ARG(d.lda >= d.K || d.M <= 1, "linear: lda %lld < K %d", (long long)d.lda, d.K);
     I64H_CHECK_ARG(d.batch <= 65535 && (d.M + 63) / 64 <= 65535, "linear: grid too large");
     if (d.M == 0) return 0;
@@ -761,6 +768,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_RELU_SQ>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_ADD: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_ADD>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_DECAY>), grid, dim3(256), lds, s, d, cpb); break;
+            case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_ROW_SIGMOID>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_SCALE>), grid, dim3(256), lds, s, d, cpb); break;
             default: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_STORE>), grid, dim3(256), lds, s, d, cpb); break;
         }
@@ -781,6 +789,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_RELU_SQ, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_ADD: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_ADD, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_DECAY, 8>), grid, dim3(512), 0, s, d); break;
+            case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_ROW_SIGMOID, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_SCALE, 8>), grid, dim3(512), 0, s, d); break;
             default: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_STORE, 8>), grid, dim3(512), 0, s, d); break;
         }
@@ -801,6 +810,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             case I64H_EPI_RELU_SQ: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_RELU_SQ>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_ADD: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_ADD>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_DECAY>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+            case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_ROW_SIGMOID>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_SCALE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
             default: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_STORE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         }

@@ -134,7 +134,8 @@ __global__ __launch_bounds__(256) void streams_kernel(const i64h_streams_args p)
 #pragma unroll
         for (int s = 0; s < HY_MAX_STREAMS; ++s) x[s] = s < S ? xs[s * plane + c] : 0.0f;
         if (p.y) {
-            const float v = p.post_w ? (sv[c] - pmean) / pden * p.post_w[c] : result(c);
+            float v = p.post_w ? (sv[c] - pmean) / pden * p.post_w[c] : result(c);
+            if (p.y_scale) v *= p.y_scale[c];
             float nx[HY_MAX_STREAMS];
 #pragma unroll
             for (int t = 0; t < HY_MAX_STREAMS; ++t) {
@@ -599,7 +600,7 @@ __device__ __forceinline__ void rot_pair(int d, int dims, int interleaved, int& 
 }
 
 // One workgroup per token, two passes: the raw queries and keys go to LDS while their squares are summed (a rotation keeps the sum of
-// squares of a pair, so the per-head sums behind the rotation are those in front of it, the rotated part times rot_mult^2); the second
+// squares of a pair, so the per-head sums behind the rotation are those in front of it, the rotated part times rot_mult^2, and a norm per head in front of it needs them as they are); the second
 // pass norms and rotates out of LDS straight into the query rows and the cached row.
 template <int NT>
 __global__ __launch_bounds__(NT) void rot_prep_kernel(const i64h_rot_prep_args p) {
@@ -637,7 +638,7 @@ __global__ __launch_bounds__(NT) void rot_prep_kernel(const i64h_rot_prep_args p
         }
     }
     float qr = 1.0f, kr = 1.0f;
-    if (p.q_norm_w) {   // (both sums through one exchange)
+    if (p.q_norm_w && !p.norm_heads) {   // (both sums through one exchange)
         a = wave_sum(a), b = wave_sum(b);
         __syncthreads();
         if (lane == 0) red[wid] = a, red[4 + wid] = b;
@@ -649,8 +650,8 @@ __global__ __launch_bounds__(NT) void rot_prep_kernel(const i64h_rot_prep_args p
         kr = 1.0f / sqrtf(sb / (float)nk + p.eps);
     }
     __syncthreads();
-    if (p.head_norm) {
-        const float m2 = p.rot_mult * p.rot_mult;
+    if (p.head_norm || p.norm_heads) {
+        const float m2 = p.norm_heads ? 1.0f : p.rot_mult * p.rot_mult;
         for (int h = wid; h < p.heads + p.kv_heads; h += NT / 64) {
             float s = 0.0f;
             for (int d = lane; d < dim; d += 64) {
@@ -671,8 +672,8 @@ __global__ __launch_bounds__(NT) void rot_prep_kernel(const i64h_rot_prep_args p
         const bool isq = h < p.heads;
         const int h0 = h * dim;                      // (the keys' raw values lie behind the queries': head index heads + g)
         const float* nw = isq ? p.q_norm_w : p.k_norm_w;
-        const float r = isq ? qr : kr;
-        const int w0 = isq ? h0 : h0 - nq;
+        const float r = p.norm_heads ? inv[h] : (isq ? qr : kr);
+        const int w0 = p.norm_heads ? 0 : (isq ? h0 : h0 - nq);
         const float hn = (p.head_norm ? inv[h] : 1.0f) * (isq ? p.scale : 1.0f);
         const int g = h - p.heads;
         for (int d = lane; d < gs; d += 64) {
@@ -937,7 +938,8 @@ int i64h_rot_prep(const i64h_rot_prep_args* dp, void* stream) {
                    d.heads, d.kv_heads, d.dim, d.vdim);
     I64H_CHECK_ARG(d.rot_dims >= 0 && d.rot_dims <= d.dim && d.rot_dims % 2 == 0 && (d.rot_dims == 0 || d.inv_freq), "rot_prep: %d rotated dimensions of %d", d.rot_dims, d.dim);
     I64H_CHECK_ARG(!d.v_freq || d.vdim % 2 == 0, "rot_prep: rotated values of an odd size %d", d.vdim);
-    I64H_CHECK_ARG((d.q_norm_w == nullptr) == (d.k_norm_w == nullptr), "rot_prep: the whole-row norms come together");
+    I64H_CHECK_ARG((d.q_norm_w == nullptr) == (d.k_norm_w == nullptr), "rot_prep: the norms' weights come together");
+    I64H_CHECK_ARG(!d.norm_heads || (d.q_norm_w && !d.head_norm), "rot_prep: a norm per head in front of the rotation needs weights and excludes the one behind it");
     I64H_CHECK_ARG(d.P && d.Q && d.positions && d.slot_ids && d.block_table && d.cache, "rot_prep: null operand");
     I64H_CHECK_ARG(d.block_size > 0 && d.max_blocks_per_seq > 0 && (d.cache_dtype == 0 || d.cache_dtype == 2), "rot_prep: bad paging or cache type");
     const size_t lds = ((size_t)(d.heads + d.kv_heads) * (d.dim + 1) + 8 + d.rot_dims + (d.v_freq ? d.vdim : 0)) * 4;

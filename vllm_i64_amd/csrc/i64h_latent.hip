@@ -45,11 +45,12 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const i64h_latent_prep
     // the shared key part and every head's query part: index 0 is the key, 1 + h the heads
     for (int e = tid; e < (p.heads + 1) * rd; e += 256) {
         const int who = e / rd, c = e % rd;
-        const float* src = who == 0 ? dkv + r : pr + p.q_off + (int64_t)(who - 1) * (p.dim + rd) + p.dim;
+        const float* src = who == 0 ? dkv + r : (p.Qsrc ? p.Qsrc + t * p.ldqs : pr) + p.q_off + (int64_t)(who - 1) * (p.dim + rd) + p.dim;
         float v;
         if (c < 2 * half) {
             float sn, cs;
             sincosf(fpos * p.inv_freq[c >> 1], &sn, &cs);
+            sn *= p.rot_mult, cs *= p.rot_mult;
             const float a = src[c & ~1], b = src[c | 1];
             v = (c & 1) ? (b * cs + a * sn) : (a * cs - b * sn);
         } else {

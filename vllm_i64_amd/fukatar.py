@@ -97,14 +97,8 @@ class FukatarModel(HybridRunner):
         m = L.mixer
         if L.type == "latent_attention":
             H, r = m.heads, m.kv_rank
-            d["w_in"] = bf(torch.cat([need(p + "mix.q", (H * m.dim, W)), need(p + "mix.dkv", (r, W))], 0))
-            d["n_in"] = H * m.dim + r
-            # a head's score against a cached latent c is q_h . (U_h c) = (U_h^T q_h) . c: the key map transposed per head
-            d["uk_t"] = bf(need(p + "mix.uk", (H * m.dim, r)).reshape(H, m.dim, r).transpose(1, 2))      # [H, r, dim]
-            d["uv"] = bf(need(p + "mix.uv", (H * m.vdim, r)).reshape(H, m.vdim, r))                      # [H, vdim, r]
-            d["c_norm"] = f(need(p + "mix.dkv.norm", (r,)))
-            d["sink"] = f(need(p + "mix.sink", (H,))) if m.sink else None
-            d["o"] = bf(need(p + "mix.o", (W, H * m.vdim)))
+            d["w_in"] = bf(torch.cat(self._load_latent(p + "mix.", m, need, d), 0))
+            d["q_off"], d["dkv_off"], d["n_in"] = 0, H * m.dim, H * m.dim + r
             d["n_a"], d["n_b"] = H * r, max(H * r, H * m.vdim)
         else:
             a = m if L.type == "attention" else m.left
@@ -148,27 +142,9 @@ class FukatarModel(HybridRunner):
         self._rotary_attention(B, d, d["m"], P, l, n, positions, slot_ids, kvc, runs, ctx_hint, B.y)
 
     def _latent(self, B, d, l, n, positions, slot_ids, kvc, runs, ctx_hint) -> None:
-        m, ex = d["m"], self.exact
-        H, r, N1 = m.heads, m.kv_rank, d["n_in"]
-        P = B.p[: n * N1].view(n, N1)
-        D.linear(B.h, d["w_in"], P, exact=ex)
-        cache = kvc.rows[l]
-        Q = B.a[: n * H * r]
-        D.latent_prep(P, q_off=0, dkv_off=H * m.dim, heads=H, dim=m.dim, rot_dim=0, kv_rank=r, rot_dims=0, c_norm_w=d["c_norm"], eps=self.cfg.norm_eps,
-                      inv_freq=None, positions=positions, slot_ids=slot_ids, block_table=kvc.block_table, block_size=kvc.block, cache=cache, q=Q, n=n)
-        # queries into latent space, per head: Q[:, h, :] = q[:, h, :] @ U_h
-        D.linear(P, d["uk_t"], Q, m=n, n=r, k=m.dim, a_off=0, lda=N1, ldc=H * r, batch=H, a_batch=m.dim, w_batch=r * m.dim, c_batch=r, exact=ex)
-        olat = B.b[: n * H * r]
-        for r0, r1, one_per_seq in runs:
-            splits, ws = 1, None
-            if one_per_seq and not ex:
-                splits, ws = self._splits(B, r1 - r0, H, 1, r, r, ctx_hint, lambda s: D.latent_attn_workspace_floats(r1 - r0, H, r, s))
-            D.latent_attn(Q[r0 * H * r: r1 * H * r], cache, kvc.block_table, slot_ids[r0:r1], positions[r0:r1], window=0, scale=m.scale, heads=H, kv_rank=r,
-                          rot_dim=0, out=olat[r0 * H * r: r1 * H * r], n=r1 - r0, mode=2 if one_per_seq else 3, splits=splits, workspace=ws, sink=d["sink"])
-        # summed latents into value space, per head
-        og = B.c[: n * H * m.vdim]
-        D.linear(olat, d["uv"], og, m=n, n=m.vdim, k=r, lda=H * r, ldc=H * m.vdim, batch=H, a_batch=r, w_batch=m.vdim * r, c_batch=m.vdim, exact=ex)
-        D.linear(og, d["o"], B.y, m=n, k=H * m.vdim, lda=H * m.vdim, exact=ex)
+        P = B.p[: n * d["n_in"]].view(n, d["n_in"])
+        D.linear(B.h, d["w_in"], P, exact=self.exact)
+        self._latent_attention(B, d, d["m"], P, l, n, positions, slot_ids, kvc, runs, ctx_hint, B.y)
 
     def _parallel(self, B, d, l, n, positions, slot_ids, kvc, seg, nseg, runs, ctx_hint, single) -> None:
         a, r = d["m"].left, d["m"].right

@@ -1,10 +1,11 @@
 """What the runners over a HybridCache share: step buffers, the grouping of a step's rows, and the sublayers that more than one design is
-made of - rotated attention over [values | keys] rows, the gated delta rule, mixtures of experts - each with its options as parameters.
+made of - rotated attention over [values | keys] rows, latent attention, the gated delta rule, gated linear attention, clamped and mixture
+feed-forwards - each with its options as parameters.
 A design's own file holds its weight layout, its residual and the order in which its sublayers run."""
 from __future__ import annotations
 
 import os
-from contextlib import contextmanager
+from contextlib import contextmanager, nullcontext
 from typing import Callable, Dict, Optional
 
 import torch
@@ -68,6 +69,27 @@ class HybridRunner:
                 raise ValueError(f"'{name}': shape {tuple(weights[name].shape)}, config says {tuple(shape)}")
             return weights[name]
         return need
+
+    # ---- load-time layout ----
+    def _stack(self, parts):
+        """Rows of several projections as one weight, every part starting at a multiple of eight rows (rows of zeros between), so that the
+        columns of a projection row can be read 16 bytes at a time; returns (weight, first column of each part)."""
+        rows, offs, at = [], [], 0
+        for t in parts:
+            offs.append(at)
+            rows.append(t.float())
+            at = pad8(at + t.shape[0])
+            if at > offs[-1] + t.shape[0]:
+                rows.append(torch.zeros(at - offs[-1] - t.shape[0], t.shape[1]))
+        return self._bf(torch.cat([r.cpu() for r in rows], 0)), offs
+
+    def _low_rank(self, weights, need, first: str, second: str, out: int):
+        """A map of two factors: the rank is the tensors' own; the second factor's columns are padded to where the first one's rows end."""
+        if first not in weights or weights[first].dim() != 2:
+            raise KeyError(f"tensor '{first}' is missing or is no matrix")
+        r = weights[first].shape[0]
+        a, b = need(first, (r, self.cfg.width)), need(second, (out, r))
+        return a, self._bf(torch.nn.functional.pad(b.float(), (0, pad8(r) - r)))
 
     # ---- step buffers: the most recent row counts are kept, pinned sets stay for captured graphs ----
     def buffers(self, n: int, m: int):
@@ -156,22 +178,92 @@ class HybridRunner:
         if a.rot is not None and a.rotate_values:
             d["v_freq"] = self._f(torch.tensor([a.rot.base ** (-2.0 * i / a.vdim) for i in range(a.vdim // 2)], dtype=torch.float64))
 
-    def _rotary_attention(self, B, d, a, P, l, n, positions, slot_ids, kvc, runs, ctx_hint, out) -> None:
+    def _rotary_attention(self, B, d, a, P, l, n, positions, slot_ids, kvc, runs, ctx_hint, out, scale: float = 1.0) -> None:
         """Rotated attention on the projection rows P (already computed; columns d["q_off"], d["k_off"], d["v_off"]): prep -> paged
-        [values | keys] rows and query rows, attention, the turn back and the head gate, out-projection into `out`."""
+        [values | keys] rows and query rows, attention, the turn back and the head gate, out-projection (times `scale`) into `out`."""
         gs = a.vdim + a.dim
         Q = B.a[: n * a.heads * gs].view(n, a.heads * gs)
         rows = kvc.rows[l]
         D.rot_prep(P, q_off=d["q_off"], k_off=d["k_off"], v_off=d["v_off"], heads=a.heads, kv_heads=a.kv_heads, dim=a.dim, vdim=a.vdim, q_norm_w=d.get("q_norm"),
                    k_norm_w=d.get("k_norm"), eps=self.cfg.norm_eps, rot_dims=a.rot.dims if a.rot is not None else 0, interleaved=a.interleaved,
                    inv_freq=d["inv_freq"], rot_mult=d["rot_mult"], head_norm=a.qk_norm == "head", v_freq=d["v_freq"], scale=a.scale, positions=positions,
-                   slot_ids=slot_ids, block_table=kvc.block_table, cache=rows, q=Q, n=n)
+                   slot_ids=slot_ids, block_table=kvc.block_table, cache=rows, q=Q, n=n, norm_heads=a.qk_norm == "head_weight")
         O = B.b[: n * a.heads * a.vdim].view(n, a.heads * a.vdim)
         self._kattn(B, a, Q, O, rows, kvc, slot_ids, positions, runs, ctx_hint, softcap=a.softcap, window=a.window, keep_first=a.keep_first, sink_w=d.get("sink"))
         if d["v_freq"] is not None or a.head_gate:
             D.rot_post(O, heads=a.heads, vdim=a.vdim, interleaved=a.interleaved, v_freq=d["v_freq"], positions=positions,
                        gate=P if a.head_gate else None, gate_off=d.get("g_off", 0), ldg=P.shape[-1], n=n)
-        D.linear(O, d["o"], out, exact=self.exact)
+        self._out(O, d["o"], out, scale)
+
+    def _out(self, a, w, out, scale: float = 1.0) -> None:
+        D.linear(a, w, out, exact=self.exact, epilogue=D.EPI_STORE if scale == 1.0 else D.EPI_SCALE, scale=scale)
+
+    # ---- latent attention: one cached row per token that all heads share ----
+    def _load_latent(self, p: str, m, need, d: dict) -> list:
+        """Tensors of a latent attention under the prefix p behind its input projections, which are returned as parts of the layer's input
+        weight, in order: queries (or their low-rank row), latent + shared key part, head gates."""
+        W, bf, f, H, r = self.cfg.width, self._bf, self._f, m.heads, m.kv_rank
+        # a head's score against a cached latent c is q_h . (U_h c) = (U_h^T q_h) . c: the key map transposed per head
+        d["uk_t"] = bf(need(p + "uk", (H * m.dim, r)).reshape(H, m.dim, r).transpose(1, 2))      # [H, r, dim]
+        d["uv"] = bf(need(p + "uv", (H * m.vdim, r)).reshape(H, m.vdim, r))                      # [H, vdim, r]
+        d["c_norm"] = f(need(p + "dkv.norm", (r,)))
+        d["sink"] = f(need(p + "sink", (H,))) if m.sink else None
+        d["o"] = bf(need(p + "o", (W, H * m.vdim)))
+        d["inv_freq"], d["rot_mult"] = None, 1.0
+        if m.rot is not None:
+            fr, d["rot_mult"] = m.rot.frequencies()
+            d["inv_freq"] = f(torch.tensor(fr, dtype=torch.float64))
+        if m.q_rank:
+            d["q_norm"], d["uq"] = f(need(p + "dq.norm", (m.q_rank,))), bf(need(p + "uq", (m.q_width, m.q_rank)))
+        parts = [need(p + "dq", (m.q_rank, W)) if m.q_rank else need(p + "q", (m.q_width, W)), need(p + "dkv", (r + m.rot_dim, W))]
+        return parts + ([need(p + "g", (H, W))] if m.head_gate else [])
+
+    def _latent_attention(self, B, d, m, P, l, n, positions, slot_ids, kvc, runs, ctx_hint, out) -> None:
+        """Latent attention on the projection rows P (columns d["q_off"]: the queries, or their low-rank row; d["dkv_off"]: latent + shared
+        key part; d["g_off"]: head gates): norms and rotation -> paged rows and query rows, queries into latent space per head, attention,
+        summed latents into value space per head (times the head's gate), out-projection into `out`."""
+        ex, N1 = self.exact, P.shape[-1]
+        H, r, rd, qh = m.heads, m.kv_rank, m.rot_dim, m.dim + m.rot_dim
+        width = r + rd
+        src, q_off = P, d["q_off"]
+        if m.q_rank:
+            cq, src, q_off = B.cq[: n * m.q_rank].view(n, m.q_rank), B.q[: n * H * qh].view(n, H * qh), 0
+            D.gate_norm(P, d["q_norm"], cq, groups=1, eps=self.cfg.norm_eps, y_off=d["q_off"], ldy=N1, n=n)
+            D.linear(cq, d["uq"], src, exact=ex)
+        cache = kvc.rows[l]
+        Q = B.a[: n * H * width]
+        D.latent_prep(P, q_off=q_off, dkv_off=d["dkv_off"], heads=H, dim=m.dim, rot_dim=rd, kv_rank=r, rot_dims=m.rot_dims, c_norm_w=d["c_norm"], eps=self.cfg.norm_eps,
+                      inv_freq=d["inv_freq"], positions=positions, slot_ids=slot_ids, block_table=kvc.block_table, block_size=kvc.block, cache=cache, q=Q, n=n,
+                      q_src=src if m.q_rank else None, rot_mult=d["rot_mult"])
+        # queries into latent space, per head: Q[:, h, :r] = q_unrotated[:, h, :] @ U_h
+        D.linear(src, d["uk_t"], Q, m=n, n=r, k=m.dim, a_off=q_off, lda=src.shape[-1], ldc=H * width, batch=H, a_batch=qh, w_batch=r * m.dim, c_batch=width, exact=ex)
+        olat = B.b[: n * H * r]
+        keys = min(ctx_hint, m.window + 64) if m.window > 0 else ctx_hint
+        for r0, r1, one_per_seq in runs:
+            splits, ws = 1, None
+            if one_per_seq and not ex:
+                splits, ws = self._splits(B, r1 - r0, H, 1, r, width, keys, lambda s: D.latent_attn_workspace_floats(r1 - r0, H, r, s))
+            D.latent_attn(Q[r0 * H * width: r1 * H * width], cache, kvc.block_table, slot_ids[r0:r1], positions[r0:r1], window=m.window, scale=m.scale, heads=H, kv_rank=r,
+                          rot_dim=rd, out=olat[r0 * H * r: r1 * H * r], n=r1 - r0, mode=2 if one_per_seq else 3, splits=splits, workspace=ws, sink=d["sink"])
+        # summed latents into value space, per head
+        og = B.c[: n * H * m.vdim]
+        gate = dict(epilogue=D.EPI_ROW_SIGMOID, e=P, e_off=d["g_off"], lde=N1, e_batch=1) if m.head_gate else {}
+        D.linear(olat, d["uv"], og, m=n, n=m.vdim, k=r, lda=H * r, ldc=H * m.vdim, batch=H, a_batch=r, w_batch=m.vdim * r, c_batch=m.vdim, exact=ex, **gate)
+        D.linear(og, d["o"], out, m=n, k=H * m.vdim, lda=H * m.vdim, exact=ex)
+
+    # ---- gated linear attention ----
+    def _gated_linear(self, B, d, r, P, l, n, positions, slot_ids, kvc, seg, nseg, out, scale: float = 1.0) -> None:
+        """Gated linear attention on the projection rows P (columns d["rq_off"], d["rk_off"], d["rv_off"], d["rg_off"]: queries, keys, values, output
+        gates; d["a1_off"]: the low-rank decay map's first factor).  sigmoid(z)^(1 / tau) = exp(-softplus(-z) / tau): the second factor and
+        its bias are held negated, the exponent's rate is d["a_rate"]."""
+        rv = r.heads * r.vdim
+        F = B.f[: n * r.heads * r.dim].view(n, r.heads * r.dim)
+        D.linear(P, d["a2"], F, m=n, a_off=d["a1_off"], exact=self.exact, bias=d["a2_b"], epilogue=D.EPI_DECAY, e=d["a_rate"])
+        R, Rn = B.r[: n * rv].view(n, rv), B.rn[: n * rv].view(n, rv)
+        D.gla_scan(P, f=F, q_off=d["rq_off"], k_off=d["rk_off"], f_off=0, v_off=d["rv_off"], heads=r.heads, dim=r.dim, vdim=r.vdim, seg_start=seg, nseg=nseg,
+                   positions=positions, slot_ids=slot_ids, state=kvc.state[l]["gla"], out=R, n=n, q_scale=r.dim ** -0.5)
+        D.gate_norm(R, d["r_norm"], Rn, groups=r.heads, eps=self.cfg.norm_eps, z=P, z_off=d["rg_off"], ldz=P.shape[-1], n=n, gate_after=True, width=rv)
+        self._out(Rn, d["o_right"], out, scale)
 
     # ---- gated delta rule ----
     def _gated_delta(self, B, d, r, P, l, n, positions, slot_ids, kvc, seg, nseg, single: bool, out) -> None:
@@ -227,6 +319,7 @@ class HybridRunner:
         B.wgt = torch.empty(n * max(t, 1), **f32)
         B.pair_token = torch.empty(n * max(t, 1), **i32)
         B.pair_row = torch.empty(n * max(t, 1), **i32)
+        B.pair_wgt = torch.empty(n * max(t, 1), **f32)
         B.group_off = torch.empty(model.max_experts + 1, **i32)
         B.sgate = torch.empty(n, **f32)
         B.sact = torch.empty(n * max(model.max_shared, 1), **f32)
@@ -238,25 +331,45 @@ class HybridRunner:
         self.max_shared = max([m.shared_ff for m in moes] or [0])
         self.max_act = max([m.ff for m in mlps if m is not None and m.kind == "dense"] + [m.ff * m.top for m in moes] + [0])
 
-    def _moe_ff(self, B, d, n, h, out, shared_out, record: Optional[dict] = None, tag: str = "") -> None:
-        """out <- the mixture of d["mlp"] on h fp32 [n, width]; shared_out [n, width] receives the shared expert's rows on the way."""
+    @staticmethod
+    def _glu(limit: float, alpha: float) -> dict:
+        """The gate / up epilogue of a feed-forward: clamped by `limit`, or silu."""
+        return dict(epilogue=D.EPI_CLAMP_GLU, act_a=alpha, act_b=limit) if limit > 0 else dict(epilogue=D.EPI_SILU_MUL)
+
+    def _load_dense(self, p: str, f, need, d: dict) -> None:
+        W = self.cfg.width
+        d["ff_gate_up"] = self._bf(torch.cat([need(p + "gate", (f.ff, W)), need(p + "up", (f.ff, W))], 0))
+        d["ff_down"] = self._bf(need(p + "down", (W, f.ff)))
+
+    def _dense_glu(self, B, d, n, h, out) -> None:
+        f = d["mlp"]
+        act = B.act[: n * f.ff].view(n, f.ff)
+        D.linear(h, d["ff_gate_up"], act, exact=self.exact, **self._glu(f.limit, f.glu_alpha))
+        D.linear(act, d["ff_down"], out, exact=self.exact)
+
+    def _moe_ff(self, B, d, n, h, out, shared_out, record: Optional[dict] = None, tag: str = "", beside: bool = False) -> None:
+        """out <- the mixture of d["mlp"] on h fp32 [n, width]; shared_out [n, width] receives the shared expert's rows on the way (beside: on
+        the side stream, while the routed experts run)."""
         f, ex, W = d["mlp"], self.exact, self.cfg.width
         E, top = f.experts, f.top
         gate = B.sgate if f.shared_ff and f.shared_gate else None
-        # the router's products in 32 bits in both modes (a choice between experts is not rounding's to make), inside the choice's launch
-        D.route_topk(None, h=h, w=d["router"], entries=f.entries, correction=d.get("correction"), groups=f.groups, keep=f.keep, top=top, scale=f.scale,
-                     idx=B.idx, wgt=B.wgt, n=n, bias=d["router_b"], chosen_softmax=f.chosen_softmax, gate_out=gate)
-        if record is not None:
-            record[f"{tag}.route"] = B.idx[: n * top].view(n, top).clone()
-        D.moe_plan(B.idx, n=n, top=top, experts=E, group_off=B.group_off, pair_token=B.pair_token, pair_row=B.pair_row)
-        glu = lambda limit: dict(epilogue=D.EPI_CLAMP_GLU, act_a=f.glu_alpha, act_b=limit) if limit > 0 else dict(epilogue=D.EPI_SILU_MUL)
-        # the (token, expert) pairs lie grouped by expert: one launch runs every expert over its own rows, the counts stay on the device
-        act = B.act[: n * top * f.ff].view(n * top, f.ff)
-        D.linear(h, d["gate_up"], act, m=n, a_rows=B.pair_token, batch=E, w_batch=2 * f.ff * W, exact=ex, group_off=B.group_off, **glu(f.limit))
-        D.linear(act, d["e_down"], B.ey, m=n, batch=E, w_batch=W * f.ff, exact=ex, group_off=B.group_off)
         shared = None
         if f.shared_ff:
-            sact = B.sact[: n * f.shared_ff].view(n, f.shared_ff)
-            D.linear(h, d["s_gate_up"], sact, exact=ex, **glu(f.shared_limit))
-            shared = D.linear(sact, d["s_down"], shared_out, exact=ex)
-        D.moe_combine(B.ey, B.pair_row, B.wgt, h, shared, out, n=n, top=top, width=W, shared_gate=gate)
+            with self._beside() if beside else nullcontext():
+                sact = B.sact[: n * f.shared_ff].view(n, f.shared_ff)
+                D.linear(h, d["s_gate_up"], sact, exact=ex, **self._glu(f.shared_limit, f.glu_alpha))
+                shared = D.linear(sact, d["s_down"], shared_out, exact=ex)
+        # the router's products in 32 bits in both modes (a choice between experts is not rounding's to make), inside the choice's launch
+        D.route_topk(None, h=h, w=d["router"], entries=f.entries, correction=d.get("correction"), groups=f.groups, keep=f.keep, top=top, scale=f.scale,
+                     idx=B.idx, wgt=B.wgt, n=n, bias=d["router_b"], chosen_softmax=f.chosen_softmax, gate_out=gate, sigmoid_scores=f.sigmoid_scores, raw_weights=f.raw_weights)
+        if record is not None:
+            record[f"{tag}.route"] = B.idx[: n * top].view(n, top).clone()
+        pair_wgt = B.pair_wgt if f.weigh_input else None      # the weight multiplies what the expert reads, not what it returns
+        D.moe_plan(B.idx, n=n, top=top, experts=E, group_off=B.group_off, pair_token=B.pair_token, pair_row=B.pair_row, wgt=B.wgt, pair_wgt=pair_wgt)
+        # the (token, expert) pairs lie grouped by expert: one launch runs every expert over its own rows, the counts stay on the device
+        act = B.act[: n * top * f.ff].view(n * top, f.ff)
+        D.linear(h, d["gate_up"], act, m=n, a_rows=B.pair_token, batch=E, w_batch=2 * f.ff * W, exact=ex, group_off=B.group_off, row_scale=pair_wgt, **self._glu(f.limit, f.glu_alpha))
+        D.linear(act, d["e_down"], B.ey, m=n, batch=E, w_batch=W * f.ff, exact=ex, group_off=B.group_off)
+        if shared is not None and beside:
+            self._meet()
+        D.moe_combine(B.ey, B.pair_row, None if f.weigh_input else B.wgt, h, shared, out, n=n, top=top, width=W, shared_gate=gate)

@@ -12,7 +12,7 @@ from ._lib import call_dense, ptr
 from .ops import _chk, _stream
 
 EPI_STORE, EPI_GELU_MUL, EPI_MUL_SIGMOID, EPI_SOFTCAP, EPI_GELU_ERF, EPI_SCALE, EPI_SILU_MUL, EPI_XIELU, EPI_RELU_SQ = 0, 1, 2, 3, 4, 5, 6, 7, 8
-EPI_CLAMP_GLU, EPI_ADD, EPI_DECAY = 9, 10, 11
+EPI_CLAMP_GLU, EPI_ADD, EPI_DECAY, EPI_ROW_SIGMOID = 9, 10, 11, 12
 _DUAL = (EPI_GELU_MUL, EPI_SILU_MUL, EPI_CLAMP_GLU)
 CACHE_DTYPE_CODE = {torch.float32: 0, torch.bfloat16: 2}
 
@@ -26,12 +26,13 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
            batch: int = 1, a_batch: int = 0, w_batch: int = 0, c_batch: int = 0, exact: bool = False, epilogue: int = EPI_STORE,
            e: Optional[torch.Tensor] = None, e_off: int = 0, lde: int = 0, e_batch: int = 0, softcap: float = 0.0,
            bias: Optional[torch.Tensor] = None, bias_batch: int = 0, scale: float = 1.0, act_a: float = 0.0, act_b: float = 0.0,
-           group_off: Optional[torch.Tensor] = None) -> torch.Tensor:
+           group_off: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out[b][:, c_off + b * c_batch : + n] = epilogue(a[b][rows, a_off + b * a_batch : + k] @ w[b]^T): see i64h_linear.  a, out and e are
     fp32 matrices addressed by (column offset, row stride; e with lde = 0 is one row for all); w is bf16 [n, k] (the gate / up epilogues: [2n, k], gate rows first), or a
     stack [batch, n, k] with w_batch = n * k.  bias fp32 [n] (per batch: bias_batch apart) is added before the epilogue.  group_off int32
     [batch + 1] on the device: batch b takes the rows [group_off[b], group_off[b + 1]) of a_rows (or a) and out; m is then the most rows a
-    batch may have, and a_rows / a / out must hold group_off[batch] rows (the caller's business: the counts stay on the device)."""
+    batch may have, and a_rows / a / out must hold group_off[batch] rows (the caller's business: the counts stay on the device).
+    row_scale fp32, one factor per row of out (the gate / up epilogues): the input row times that factor."""
     _chk(a, torch.float32, "a"), _chk(w, torch.bfloat16, "w"), _chk(out, torch.float32, "out")
     if a_rows is not None:
         _chk(a_rows, torch.int32, "a_rows")
@@ -48,12 +49,16 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
         raise _lib.I64HError("linear: weight smaller than the launch reads")
     if e is not None:
         _chk(e, torch.float32, "e")
-        if e.numel() < (M - 1) * lde + e_off + (batch - 1) * e_batch + N:
+        if e.numel() < (M - 1) * lde + e_off + (batch - 1) * e_batch + (1 if epilogue == EPI_ROW_SIGMOID else N):
             raise _lib.I64HError("linear: gate operand smaller than the launch reads")
     if bias is not None:
         _chk(bias, torch.float32, "bias")
         if bias.numel() < (batch - 1) * bias_batch + N:
             raise _lib.I64HError("linear: bias smaller than the launch reads")
+    if row_scale is not None:
+        _chk(row_scale, torch.float32, "row_scale")
+        if row_scale.numel() < M:
+            raise _lib.I64HError("linear: fewer row factors than rows")
     if group_off is not None:
         _chk(group_off, torch.int32, "group_off")
         if group_off.numel() < batch + 1:
@@ -61,7 +66,8 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
     d = _lib.Linear(A=ptr(a) + 4 * a_off, lda=lda, a_rows=ptr(a_rows), W=ptr(w), C=ptr(out) + 4 * c_off, ldc=ldc, M=M, N=N, K=K, batch=batch,
                     a_batch=a_batch, w_batch=w_batch, c_batch=c_batch, exact=int(exact), epilogue=epilogue,
                     E=(ptr(e) + 4 * e_off) if e is not None else 0, lde=lde, e_batch=e_batch, softcap=float(softcap),
-                    bias=ptr(bias), bias_batch=int(bias_batch), scale=float(scale), act_a=float(act_a), act_b=float(act_b), group_off=ptr(group_off))
+                    bias=ptr(bias), bias_batch=int(bias_batch), scale=float(scale), act_a=float(act_a), act_b=float(act_b), group_off=ptr(group_off),
+                    row_scale=ptr(row_scale))
     call_dense("i64h_linear_run", _ref(d), _stream())
     return out
 
@@ -100,7 +106,9 @@ def gated_postnorm(x: torch.Tensor, norm_w: torch.Tensor, groups: int, eps: floa
 
 def latent_prep(p: torch.Tensor, *, q_off: int, dkv_off: int, heads: int, dim: int, rot_dim: int, kv_rank: int, rot_dims: int,
                 c_norm_w: torch.Tensor, eps: float, inv_freq: Optional[torch.Tensor], positions: torch.Tensor, slot_ids: torch.Tensor,
-                block_table: torch.Tensor, block_size: int, cache: torch.Tensor, q: torch.Tensor, n: Optional[int] = None) -> None:
+                block_table: torch.Tensor, block_size: int, cache: torch.Tensor, q: torch.Tensor, n: Optional[int] = None,
+                q_src: Optional[torch.Tensor] = None, rot_mult: float = 1.0) -> None:
+    """See i64h_latent_prep.  q_src fp32 [n, ld]: the queries' rows, where they are no columns of p."""
     _chk(p, torch.float32, "p"), _chk(c_norm_w, torch.float32, "c_norm_w"), _chk(q, torch.float32, "q")
     _chk(positions, torch.int32, "positions"), _chk(slot_ids, torch.int32, "slot_ids"), _chk(block_table, torch.int32, "block_table")
     _chk(cache, None, "cache")
@@ -108,7 +116,11 @@ def latent_prep(p: torch.Tensor, *, q_off: int, dkv_off: int, heads: int, dim: i
     D = kv_rank + rot_dim
     if cache.shape[-1] != D or cache.shape[-2] != block_size or q.numel() < rows * heads * D or positions.numel() < rows or slot_ids.numel() < rows:
         raise _lib.I64HError("latent_prep: cache / query / position shapes do not fit the sizes")
-    if q_off + heads * (dim + rot_dim) > p.shape[-1] or dkv_off + D > p.shape[-1] or c_norm_w.numel() != kv_rank:
+    if q_src is not None:
+        _chk(q_src, torch.float32, "q_src")
+        if q_src.numel() < rows * q_src.shape[-1]:
+            raise _lib.I64HError("latent_prep: fewer query rows than the launch reads")
+    if q_off + heads * (dim + rot_dim) > (q_src if q_src is not None else p).shape[-1] or p.numel() < rows * p.shape[-1] or dkv_off + D > p.shape[-1] or c_norm_w.numel() != kv_rank:
         raise _lib.I64HError("latent_prep: projection columns outside the projection rows")
     if rot_dims:
         _chk(inv_freq, torch.float32, "inv_freq")
@@ -116,7 +128,8 @@ def latent_prep(p: torch.Tensor, *, q_off: int, dkv_off: int, heads: int, dim: i
     d = _lib.LatentPrep(P=ptr(p), ldp=p.shape[-1], q_off=q_off, dkv_off=dkv_off, heads=heads, dim=dim, rot_dim=rot_dim, kv_rank=kv_rank,
                         rot_dims=rot_dims, c_norm_w=ptr(c_norm_w), eps=float(eps), inv_freq=ptr(inv_freq) if rot_dims else 0,
                         positions=ptr(positions), slot_ids=ptr(slot_ids), block_table=ptr(block_table), max_blocks_per_seq=block_table.shape[1],
-                        block_size=block_size, cache=ptr(cache), cache_dtype=CACHE_DTYPE_CODE[cache.dtype], Q=ptr(q), n=rows)
+                        block_size=block_size, cache=ptr(cache), cache_dtype=CACHE_DTYPE_CODE[cache.dtype], Q=ptr(q), n=rows, Qsrc=ptr(q_src),
+                        ldqs=q_src.shape[-1] if q_src is not None else 0, rot_mult=float(rot_mult))
     call_dense("i64h_latent_prep", _ref(d), _stream())
 
 
@@ -195,14 +208,14 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
                  y2n_w: Optional[torch.Tensor] = None, y_eps: float = 0.0, mix: Optional[torch.Tensor] = None, out_w: Optional[torch.Tensor] = None,
                  in_w: Optional[torch.Tensor] = None, norm_w: Optional[torch.Tensor] = None, eps: float = 0.0, h: Optional[torch.Tensor] = None,
                  rows: Optional[torch.Tensor] = None, post_w: Optional[torch.Tensor] = None, post_center: bool = False,
-                 h_center: bool = False, norm_b: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                 h_center: bool = False, norm_b: Optional[torch.Tensor] = None, y_scale: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """See i64h_streams_step.  streams fp32 [S, n, W], updated in place when y is given; h fp32 [n, W] (or [rows, W]).  post_w fp32 [W]: a
     norm over the result as a whole (centred with post_center) before it is added; h_center: the read's norm is centred; norm_b: added behind
-    the read's norm weight.  y2 without norm weights is simply added to y."""
+    the read's norm weight.  y2 without norm weights is simply added to y.  y_scale fp32 [W]: a factor per column on what is added."""
     _chk(streams, torch.float32, "streams")
     S, n, W = streams.shape
     for t, name in ((y, "y"), (y2, "y2"), (yn_w, "yn_w"), (y2n_w, "y2n_w"), (mix, "mix"), (out_w, "out_w"), (in_w, "in_w"), (norm_w, "norm_w"), (h, "h"),
-                    (post_w, "post_w"), (norm_b, "norm_b")):
+                    (post_w, "post_w"), (norm_b, "norm_b"), (y_scale, "y_scale")):
         if t is not None:
             _chk(t, torch.float32, name)
     for t, name in ((y, "y"), (y2, "y2")):
@@ -212,8 +225,8 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
         raise _lib.I64HError("streams_step: stream weights do not fit the number of streams")
     if (yn_w is not None and yn_w.numel() != W) or (y2n_w is not None and y2n_w.numel() != W) or (post_w is not None and post_w.numel() != W):
         raise _lib.I64HError("streams_step: result norm weights are not [W]")
-    if norm_b is not None and norm_b.numel() != W:
-        raise _lib.I64HError("streams_step: the norm's offsets are not [W]")
+    if (norm_b is not None and norm_b.numel() != W) or (y_scale is not None and y_scale.numel() != W):
+        raise _lib.I64HError("streams_step: the norm's offsets or the result's factors are not [W]")
     m_rows = n
     if rows is not None:
         _chk(rows, torch.int32, "rows")
@@ -223,7 +236,7 @@ def streams_step(streams: torch.Tensor, *, y: Optional[torch.Tensor] = None, y2:
     d = _lib.Streams(streams=ptr(streams), S=S, n=n, W=W, y=ptr(y), ldy=W, y2=ptr(y2), ldy2=W, yn_w=ptr(yn_w), y2n_w=ptr(y2n_w), y_eps=float(y_eps),
                      mix=ptr(mix), out_w=ptr(out_w), in_w=ptr(in_w), norm_w=ptr(norm_w), norm_w_len=norm_w.numel() if norm_w is not None else 0,
                      eps=float(eps), h=ptr(h), rows=ptr(rows), m_rows=m_rows, post_w=ptr(post_w), post_center=int(bool(post_center)), h_center=int(bool(h_center)),
-                     norm_b=ptr(norm_b))
+                     norm_b=ptr(norm_b), y_scale=ptr(y_scale))
     call_dense("i64h_streams_step", _ref(d), _stream())
     return h
 
@@ -282,22 +295,25 @@ def ssm_scan(xbc: torch.Tensor, dt: torch.Tensor, *, dt_off: int, lddt: int, dt_
 
 
 def gate_norm(y: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, groups: int, eps: float, z: Optional[torch.Tensor] = None, z_off: int = 0,
-              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None, sigmoid: bool = False) -> torch.Tensor:
+              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None, sigmoid: bool = False,
+              y_off: int = 0, ldy: Optional[int] = None) -> torch.Tensor:
     """out = rms_groups(y * silu(z)) * w: see i64h_gate_norm.  y, out fp32 [n, width]; z the columns [z_off, + width) of a matrix of row stride ldz.
-    gate_after: out = rms_groups(y) * w * silu(z).  sigmoid: the gate is sigmoid(z).  width (default: w's length): the row's width, w then repeats over it."""
+    gate_after: out = rms_groups(y) * w * silu(z).  sigmoid: the gate is sigmoid(z).  width (default: w's length): the row's width, w then repeats over it.
+    y_off, ldy: the columns [y_off, + width) of a matrix of row stride ldy (default: y is [n, width])."""
     _chk(y, torch.float32, "y"), _chk(w, torch.float32, "w"), _chk(out, torch.float32, "out")
     w_len = w.numel()
     width = int(width if width is not None else w_len)
     if width % w_len:
         raise _lib.I64HError("gate_norm: the weights do not repeat evenly over the row")
     rows = int(n if n is not None else y.numel() // width)
-    if y.numel() < rows * width or out.numel() < rows * width:
+    ldy = int(ldy if ldy is not None else width)
+    if y_off + width > ldy or y.numel() < (rows - 1) * ldy + y_off + width or out.numel() < rows * width:
         raise _lib.I64HError("gate_norm: operand smaller than the launch reads or writes")
     if z is not None:
         _chk(z, torch.float32, "z")
         if z.numel() < (rows - 1) * ldz + z_off + width:
             raise _lib.I64HError("gate_norm: gate smaller than the launch reads")
-    d = _lib.GateNorm(y=ptr(y), ldy=width, z=(ptr(z) + 4 * z_off) if z is not None else 0, ldz=ldz, w=ptr(w), width=width, groups=groups, eps=float(eps),
+    d = _lib.GateNorm(y=ptr(y) + 4 * y_off, ldy=ldy, z=(ptr(z) + 4 * z_off) if z is not None else 0, ldz=ldz, w=ptr(w), width=width, groups=groups, eps=float(eps),
                       out=ptr(out), ldo=width, n=rows, gate_after=int(bool(gate_after)), w_len=w_len if w_len != width else 0, gate_act=int(bool(sigmoid)))
     call_dense("i64h_gate_norm", _ref(d), _stream())
     return out
@@ -411,9 +427,9 @@ def kv_prep(p: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int, 
 def rot_prep(p: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int, kv_heads: int, dim: int, vdim: int, q_norm_w: Optional[torch.Tensor],
              k_norm_w: Optional[torch.Tensor], eps: float, rot_dims: int, interleaved: bool, inv_freq: Optional[torch.Tensor], rot_mult: float,
              head_norm: bool, v_freq: Optional[torch.Tensor], scale: float, positions: torch.Tensor, slot_ids: torch.Tensor, block_table: torch.Tensor,
-             cache: torch.Tensor, q: torch.Tensor, n: Optional[int] = None) -> None:
+             cache: torch.Tensor, q: torch.Tensor, n: Optional[int] = None, norm_heads: bool = False) -> None:
     """See i64h_rot_prep.  cache [blocks, block, kv_heads * (vdim + dim)] fp32 / bf16; q fp32 [n, heads, vdim + dim]; inv_freq fp32 [rot_dims / 2];
-    v_freq fp32 [vdim / 2] or None."""
+    v_freq fp32 [vdim / 2] or None.  norm_heads: the norms in front of the rotation are per head, weights [dim]."""
     _chk(p, torch.float32, "p"), _chk(q, torch.float32, "q"), _chk(cache, None, "cache")
     _chk(positions, torch.int32, "positions"), _chk(slot_ids, torch.int32, "slot_ids"), _chk(block_table, torch.int32, "block_table")
     rows = int(n if n is not None else positions.numel())
@@ -422,7 +438,7 @@ def rot_prep(p: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int,
     if q.numel() < rows * heads * gs or max(q_off + heads * dim, k_off + kv_heads * dim, v_off + kv_heads * vdim) > p.shape[-1] or p.numel() < rows * p.shape[-1] or \
             cache.shape[-1] != kv_heads * gs:
         raise _lib.I64HError("rot_prep: shapes do not fit the sizes")
-    for t, name, size in ((q_norm_w, "q_norm_w", heads * dim), (k_norm_w, "k_norm_w", kv_heads * dim), (inv_freq, "inv_freq", rot_dims // 2), (v_freq, "v_freq", vdim // 2)):
+    for t, name, size in ((q_norm_w, "q_norm_w", dim if norm_heads else heads * dim), (k_norm_w, "k_norm_w", dim if norm_heads else kv_heads * dim), (inv_freq, "inv_freq", rot_dims // 2), (v_freq, "v_freq", vdim // 2)):
         if t is not None:
             _chk(t, torch.float32, name)
             if t.numel() < size:
@@ -433,7 +449,7 @@ def rot_prep(p: torch.Tensor, *, q_off: int, k_off: int, v_off: int, heads: int,
                      k_norm_w=ptr(k_norm_w), eps=float(eps), rot_dims=int(rot_dims), interleaved=int(bool(interleaved)), inv_freq=ptr(inv_freq), rot_mult=float(rot_mult),
                      head_norm=int(bool(head_norm)), v_freq=ptr(v_freq), scale=float(scale), positions=ptr(positions), slot_ids=ptr(slot_ids),
                      block_table=ptr(block_table), max_blocks_per_seq=block_table.shape[1], block_size=cache.shape[-2], cache=ptr(cache),
-                     cache_dtype=CACHE_DTYPE_CODE[cache.dtype], Q=ptr(q), n=rows)
+                     cache_dtype=CACHE_DTYPE_CODE[cache.dtype], Q=ptr(q), n=rows, norm_heads=int(bool(norm_heads)))
     call_dense("i64h_rot_prep", _ref(d), _stream())
 
 
@@ -503,17 +519,23 @@ def gdn_scan(x: torch.Tensor, g: torch.Tensor, *, q_off: int, k_off: int, v_off:
 
 
 def _gla_args(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int, dim: int, vdim: int, k_off: int = -1, lower: Optional[torch.Tensor] = None,
-              q_act: bool = False, n: int, **rest) -> "_lib.Gla":
+              q_act: bool = False, n: int, f: Optional[torch.Tensor] = None, q_scale: float = 1.0, **rest) -> "_lib.Gla":
     _chk(p, torch.float32, "p")
     if lower is not None:
         _chk(lower, torch.float32, "lower")
         if lower.numel() != heads * dim:
             raise _lib.I64HError("gla: the gate's lower bounds are not [heads * dim]")
     ld = p.shape[-1]
-    if max(q_off, f_off, max(k_off, 0)) + heads * dim > ld or v_off + heads * vdim > ld or p.numel() < n * ld:
+    fld = ld
+    if f is not None:
+        _chk(f, torch.float32, "f")
+        fld = f.shape[-1]
+        if f.numel() < n * fld:
+            raise _lib.I64HError("gla: fewer rows of decays than the launch reads")
+    if max(q_off, max(k_off, 0)) + heads * dim > ld or f_off + heads * dim > fld or v_off + heads * vdim > ld or p.numel() < n * ld:
         raise _lib.I64HError("gla: projection columns outside the projection rows")
     return _lib.Gla(P=ptr(p), ldp=ld, q_off=q_off, f_off=f_off, k_off=k_off, v_off=v_off, heads=heads, dim=dim, vdim=vdim, lower=ptr(lower),
-                    q_act=int(bool(q_act)), n=n, **rest)
+                    q_act=int(bool(q_act)), n=n, F=ptr(f), ldf=fld if f is not None else 0, q_scale=float(q_scale), **rest)
 
 
 def gla_gates(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int, dim: int, vdim: int, lower: Optional[torch.Tensor], q_act: bool,
@@ -524,14 +546,16 @@ def gla_gates(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int
 
 
 def gla_scan(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int, dim: int, vdim: int, seg_start: torch.Tensor, nseg: int,
-             positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n: int, k_off: int = -1) -> torch.Tensor:
-    """See i64h_gla_scan.  state fp32 [slots, heads, vdim, dim]; out fp32 [n, heads * vdim]; k_off < 0: the key is one minus the decay."""
+             positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n: int, k_off: int = -1,
+             f: Optional[torch.Tensor] = None, q_scale: float = 1.0) -> torch.Tensor:
+    """See i64h_gla_scan.  state fp32 [slots, heads, vdim, dim]; out fp32 [n, heads * vdim]; k_off < 0: the key is one minus the decay.
+    f fp32 [n, ld]: the decays, where they are no columns of p; q_scale multiplies the read-out."""
     _chk(state, torch.float32, "state"), _chk(out, torch.float32, "out")
     _chk(seg_start, torch.int32, "seg_start"), _chk(positions, torch.int32, "positions"), _chk(slot_ids, torch.int32, "slot_ids")
     _rows_ok("gla_scan", n, positions, slot_ids)
     if tuple(state.shape[1:]) != (heads, vdim, dim) or out.numel() < n * heads * vdim or seg_start.numel() < nseg + 1:
         raise _lib.I64HError("gla_scan: shapes do not fit the sizes")
-    d = _gla_args(p, q_off=q_off, f_off=f_off, v_off=v_off, heads=heads, dim=dim, vdim=vdim, k_off=k_off, n=n, seg_start=ptr(seg_start), nseg=nseg,
+    d = _gla_args(p, q_off=q_off, f_off=f_off, v_off=v_off, heads=heads, dim=dim, vdim=vdim, k_off=k_off, n=n, f=f, q_scale=q_scale, seg_start=ptr(seg_start), nseg=nseg,
                   positions=ptr(positions), slot_ids=ptr(slot_ids), state=ptr(state), out=ptr(out), ldo=heads * vdim)
     call_dense("i64h_gla_scan", _ref(d), _stream())
     return out
@@ -539,10 +563,11 @@ def gla_scan(p: torch.Tensor, *, q_off: int, f_off: int, v_off: int, heads: int,
 
 def route_topk(logits: Optional[torch.Tensor], *, entries: int, correction: Optional[torch.Tensor], groups: int, keep: int, top: int, scale: float, idx: torch.Tensor,
                wgt: torch.Tensor, n: Optional[int] = None, h: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None,
-               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, gate_out: Optional[torch.Tensor] = None) -> None:
+               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, gate_out: Optional[torch.Tensor] = None,
+               sigmoid_scores: bool = False, raw_weights: bool = False) -> None:
     """See i64h_route_topk.  logits fp32 [n, ld >= entries], or None with h fp32 [n, K] and w bf16 [entries, K]: the launch computes the
     logits itself in 32 bits; idx int32 [n, top]; wgt fp32 [n, top].  bias fp32 [entries]; gate_out fp32 [n]: w has one more row, whose
-    product's sigmoid it receives."""
+    product's sigmoid it receives.  sigmoid_scores: sigmoid in the softmax's place; raw_weights: scores as weights, not renormalised."""
     _chk(idx, torch.int32, "idx"), _chk(wgt, torch.float32, "wgt")
     if logits is None:
         if h is None or w is None:
@@ -573,30 +598,39 @@ def route_topk(logits: Optional[torch.Tensor], *, entries: int, correction: Opti
     d = _lib.Route(logits=ptr(logits), ld=logits.shape[-1] if logits is not None else 0, E=entries, correction=ptr(correction), groups=int(groups), keep=int(keep),
                    top=int(top), scale=float(scale), idx=ptr(idx), wgt=ptr(wgt), n=rows, h=ptr(h) if logits is None else 0,
                    ldh=h.shape[-1] if logits is None else 0, W=ptr(w) if logits is None else 0, K=w.shape[1] if logits is None else 0,
-                   bias=ptr(bias), chosen_softmax=int(bool(chosen_softmax)), gate_out=ptr(gate_out))
+                   bias=ptr(bias), chosen_softmax=int(bool(chosen_softmax)), gate_out=ptr(gate_out), sigmoid_scores=int(bool(sigmoid_scores)),
+                   raw_weights=int(bool(raw_weights)))
     call_dense("i64h_route_topk", _ref(d), _stream())
 
 
-def moe_plan(idx: torch.Tensor, *, n: int, top: int, experts: int, group_off: torch.Tensor, pair_token: torch.Tensor, pair_row: torch.Tensor) -> None:
-    """See i64h_moe_plan."""
+def moe_plan(idx: torch.Tensor, *, n: int, top: int, experts: int, group_off: torch.Tensor, pair_token: torch.Tensor, pair_row: torch.Tensor,
+             wgt: Optional[torch.Tensor] = None, pair_wgt: Optional[torch.Tensor] = None) -> None:
+    """See i64h_moe_plan.  pair_wgt fp32 [n * top] receives the choices' weights wgt fp32 [n, top] in the grouped order."""
+    if pair_wgt is not None:
+        _chk(wgt, torch.float32, "wgt"), _chk(pair_wgt, torch.float32, "pair_wgt")
+        if min(wgt.numel(), pair_wgt.numel()) < n * top:
+            raise _lib.I64HError("moe_plan: fewer weights than choices")
     for t, name in ((idx, "idx"), (group_off, "group_off"), (pair_token, "pair_token"), (pair_row, "pair_row")):
         _chk(t, torch.int32, name)
     if idx.numel() < n * top or group_off.numel() < experts + 1 or pair_token.numel() < n * top or pair_row.numel() < n * top:
         raise _lib.I64HError("moe_plan: shapes do not fit the sizes")
-    d = _lib.MoePlan(idx=ptr(idx), n=n, top=top, experts=experts, group_off=ptr(group_off), pair_token=ptr(pair_token), pair_row=ptr(pair_row))
+    d = _lib.MoePlan(idx=ptr(idx), n=n, top=top, experts=experts, group_off=ptr(group_off), pair_token=ptr(pair_token), pair_row=ptr(pair_row),
+                     wgt=ptr(wgt) if pair_wgt is not None else 0, pair_wgt=ptr(pair_wgt))
     call_dense("i64h_moe_plan", _ref(d), _stream())
 
 
-def moe_combine(y: torch.Tensor, pair_row: torch.Tensor, wgt: torch.Tensor, h: torch.Tensor, shared: Optional[torch.Tensor], out: torch.Tensor, *,
+def moe_combine(y: torch.Tensor, pair_row: torch.Tensor, wgt: Optional[torch.Tensor], h: torch.Tensor, shared: Optional[torch.Tensor], out: torch.Tensor, *,
                 n: int, top: int, width: int, shared_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """See i64h_moe_combine.  y fp32 [pairs, width]; h, shared, out fp32 [n, width]; shared_gate fp32 [n]."""
+    """See i64h_moe_combine.  y fp32 [pairs, width]; h, shared, out fp32 [n, width]; shared_gate fp32 [n]; wgt None: weights of one."""
     if shared_gate is not None:
         _chk(shared_gate, torch.float32, "shared_gate")
         _rows_ok("moe_combine", n, shared_gate)
-    _chk(y, torch.float32, "y"), _chk(pair_row, torch.int32, "pair_row"), _chk(wgt, torch.float32, "wgt"), _chk(h, torch.float32, "h"), _chk(out, torch.float32, "out")
+    _chk(y, torch.float32, "y"), _chk(pair_row, torch.int32, "pair_row"), _chk(h, torch.float32, "h"), _chk(out, torch.float32, "out")
+    if wgt is not None:
+        _chk(wgt, torch.float32, "wgt")
     if shared is not None:
         _chk(shared, torch.float32, "shared")
-    if min(h.numel(), out.numel(), shared.numel() if shared is not None else out.numel()) < n * width or min(pair_row.numel(), wgt.numel()) < n * top or \
+    if min(h.numel(), out.numel(), shared.numel() if shared is not None else out.numel()) < n * width or min(pair_row.numel(), wgt.numel() if wgt is not None else pair_row.numel()) < n * top or \
             y.numel() < n * top * width:
         raise _lib.I64HError("moe_combine: shapes do not fit the sizes")
     d = _lib.MoeCombine(Y=ptr(y), pair_row=ptr(pair_row), wgt=ptr(wgt), h=ptr(h), shared=ptr(shared), out=ptr(out), n=n, top=top, W=width,

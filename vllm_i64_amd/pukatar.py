@@ -27,7 +27,7 @@ import torch
 
 from . import ops_dense as D
 from .config import PukatarConfig
-from .hybrid_runner import HybridRunner, pad8
+from .hybrid_runner import HybridRunner
 from .model import attention_segments
 from .paged_cache import HybridCache
 
@@ -100,26 +100,6 @@ class PukatarModel(HybridRunner):
         self.kv = HybridCache(specs, num_kv_blocks, max_seqs, dev, dtype=cache_dtype, block=kv_block)
 
     # ---- load-time layout work: one weight for everything that reads the layer's input; small vectors and tables in fp32 ----
-    def _stack(self, parts):
-        """Rows of several projections as one weight, every part starting at a multiple of eight rows (rows of zeros between), so that the
-        columns of a projection row can be read 16 bytes at a time; returns (weight, first column of each part)."""
-        rows, offs, at = [], [], 0
-        for t in parts:
-            offs.append(at)
-            rows.append(t.float())
-            at = pad8(at + t.shape[0])
-            if at > offs[-1] + t.shape[0]:
-                rows.append(torch.zeros(at - offs[-1] - t.shape[0], t.shape[1]))
-        return self._bf(torch.cat([r.cpu() for r in rows], 0)), offs
-
-    def _low_rank(self, weights, need, first: str, second: str, out: int):
-        """A map of two factors: the rank is the tensors' own; the second factor's columns are padded to where the first one's rows end."""
-        if first not in weights or weights[first].dim() != 2:
-            raise KeyError(f"tensor '{first}' is missing or is no matrix")
-        r = weights[first].shape[0]
-        a, b = need(first, (r, self.cfg.width)), need(second, (out, r))
-        return a, self._bf(torch.nn.functional.pad(b.float(), (0, pad8(r) - r)))
-
     def _load_layer(self, i: int, L, weights, need) -> dict:
         W, p, bf, f = self.cfg.width, f"l{i}.", self._bf, self._f
         d = dict(type=L.type, m=L.mixer, mlp=L.mlp)
@@ -147,23 +127,16 @@ class PukatarModel(HybridRunner):
         d["ld"] = d["w_in"].shape[0]
         ff = L.mlp
         if ff is not None and ff.kind == "dense":
-            d["ff_gate_up"] = bf(torch.cat([need(p + "mlp.gate", (ff.ff, W)), need(p + "mlp.up", (ff.ff, W))], 0))
-            d["ff_down"] = bf(need(p + "mlp.down", (W, ff.ff)))
+            self._load_dense(p + "mlp.", ff, need, d)
         elif ff is not None:
             self._load_moe(p + "mlp.", ff, need, d)
         return d
 
     def _feed_forward(self, B, d, n, record, r) -> None:
         if d["mlp"].kind == "dense":
-            self._dense_ff(B, d, n)
+            self._dense_glu(B, d, n, B.h, B.y2)
         else:
             self._moe_ff(B, d, n, B.h, B.y2, B.y3, record, f"r{r}")
-
-    def _dense_ff(self, B, d, n) -> None:
-        ff = d["mlp"].ff
-        act = B.act[: n * ff].view(n, ff)
-        D.linear(B.h, d["ff_gate_up"], act, exact=self.exact, epilogue=D.EPI_SILU_MUL)
-        D.linear(act, d["ff_down"], B.y2, exact=self.exact)
 
     @torch.no_grad()
     def forward(self, token_ids: torch.Tensor, positions: torch.Tensor, slot_ids: torch.Tensor, ctx_len: Optional[torch.Tensor] = None,

@@ -97,6 +97,25 @@ def _load_pukatar(config: dict, tensors, *, device, dtype, max_seqs, max_tokens,
     return PukatarModel(cfg, tensors, device=device, dtype=dtype, max_seqs=max_seqs, num_kv_blocks=blocks, kv_block=kv_block)
 
 
+def _load_vepelix(config: dict, tensors, *, device, dtype, max_seqs, max_tokens, kv_block=16, **_):
+    from .config import VepelixConfig
+    from .vepelix import VepelixModel
+    config = dict(config)
+    for key, axis in (("vocab", 0), ("width", 1)):      # sizes that the file may leave to the tensors' shapes
+        if key not in config and "embed" in tensors:
+            config[key] = int(tensors["embed"].shape[axis])
+    layers = []
+    for i, l in enumerate(config.get("layers") or []):     # (the queries' rank likewise)
+        name = f"l{i}.mix.dq"
+        if l.get("type") == "latent_attention" and "q_rank" not in (l.get("mixer") or {"q_rank": 0}) and name in tensors:
+            l = dict(l, mixer=dict(l["mixer"], q_rank=int(tensors[name].shape[0])))
+        layers.append(l)
+    config["layers"] = layers
+    cfg = VepelixConfig.from_dict(config)
+    blocks = max(1, (int(max_tokens) + kv_block - 1) // kv_block)
+    return VepelixModel(cfg, tensors, device=device, dtype=dtype, max_seqs=max_seqs, num_kv_blocks=blocks, kv_block=kv_block)
+
+
 def _load_complexity_deep(config: dict, tensors, *, device, dtype, max_seqs, max_tokens, quant="int8", **_):
     import torch
     from .checkpoint import config_from_dict, native_to_weights
@@ -112,6 +131,7 @@ register("Dogalorn", _load_dogalorn)
 register("Zabutar", _load_zabutar)
 register("Fukatar", _load_fukatar)
 register("Pukatar", _load_pukatar)
+register("Vepelix", _load_vepelix)
 register("complexity-deep", _load_complexity_deep)
 register("ComplexityDeepModel", _load_complexity_deep)
 
