@@ -1,8 +1,9 @@
-"""`bench.py --design morilorn | dogalorn | zabutar | fukatar | pukatar`: prefill and decode throughput of a registered design at layer sizes of real models
+"""`bench.py --design morilorn | dogalorn | zabutar | fukatar | pukatar | vepelix`: prefill and decode throughput of a registered design at layer sizes of real models
 (random weights), beside the package's closest existing model at equal width, depth, feed-forward size and batch (Morilorn: the dense
 int8 decoder; Dogalorn: Morilorn, which shares its library, bf16 Linears and 32-bit residual; Zabutar: Dogalorn, the other design of
 recurrent layers beside attention with a distance bias; Fukatar: Zabutar, the other design with a norm behind every sublayer, a matrix-valued
-recurrence and attention over separate keys and values; Pukatar: Fukatar, the other design of rotated attention and a gated delta rule),
+recurrence and attention over separate keys and values; Pukatar: Fukatar, the other design of rotated attention and a gated delta rule;
+Vepelix: Pukatar, the other design of repeated layers, windowed attention, a recurrence with a decay per key channel and clamped experts),
 and the design's kernels one by one against their rooflines beside the like
 kernel of that model.  Prints one JSON line."""
 from __future__ import annotations
@@ -909,6 +910,218 @@ def run_pukatar(args) -> dict:
     return result
 
 
+VEPELIX_SIZES = {
+    "w1024": dict(width=1024, blocks=3, loop_blocks=1, heads=16, dim=64, rot_dim=32, vdim=64, kv_rank=256, q_rank=512, left_heads=16, left_kv_heads=4, left_dim=64, left_vdim=64,
+                  window=1024, rec_heads=8, rec_dim=128, rec_vdim=128, ff=2752, experts=8, top=2, expert_ff=896, shared_ff=896),
+    "w2048": dict(width=2048, blocks=1, loop_blocks=1, heads=32, dim=64, rot_dim=32, vdim=64, kv_rank=256, q_rank=768, left_heads=32, left_kv_heads=8, left_dim=64, left_vdim=64,
+                  window=1024, rec_heads=16, rec_dim=128, rec_vdim=128, ff=5504, experts=8, top=2, expert_ff=1792, shared_ff=1792),
+}
+
+
+def _vepelix_kernels(sz, rows, batch, ctx, dev):
+    """Single launches at the step's shapes with the share of their roofline (matrix products: bf16 matrix peak; recurrences: the larger of
+    bytes / HBM rate and flop / fp32 vector rate; everything else: bytes / HBM rate), each beside the like kernel of Pukatar (of Fukatar for
+    the latent attention)."""
+    from . import ops_dense as D
+    W, ff, H, dm, rd, dv, r, rq = sz["width"], sz["ff"], sz["heads"], sz["dim"], sz["rot_dim"], sz["vdim"], sz["kv_rank"], sz["q_rank"]
+    Hl, Gl, dl, vl, win = sz["left_heads"], sz["left_kv_heads"], sz["left_dim"], sz["left_vdim"], sz["window"]
+    Hr, dk, dr = sz["rec_heads"], sz["rec_dim"], sz["rec_vdim"]
+    E, top, eff, R = sz["experts"], sz["top"], sz["expert_ff"], PUKATAR_RANK
+    out = {}
+    g = torch.Generator(device=dev).manual_seed(1)
+    rn = lambda *s: torch.randn(*s, device=dev, generator=g)
+    wt = lambda *s: (rn(*s) * 0.02).to(torch.bfloat16)
+
+    def row(name, t, flops=0.0, bytes_=0.0, peak=BF16_TFLOPS):
+        share = max(flops / t / (peak * 1e12), bytes_ / t / (HBM_GBS * 1e9))
+        out[name] = {"us": round(t * 1e6, 1), "roofline_share": round(share, 3)}
+
+    seq = 512
+    warm_a, warm_w, warm_c = rn(rows, W), wt(W, W), torch.empty(rows, W, device=dev)
+    _time(lambda: D.linear(warm_a, warm_w, warm_c), 20)      # clocks and caches settle before the first timed launch
+    for n, tag in ((rows, "prefill"), (batch, "decode")):
+        nseq = n // seq if tag == "prefill" else n
+        per = seq if tag == "prefill" else 1
+        pos0 = 0 if tag == "prefill" else ctx - 1
+        pos = (torch.arange(per, dtype=torch.int32) + pos0).repeat(nseq).to(dev)
+        slots = torch.arange(nseq, dtype=torch.int32).repeat_interleave(per).to(dev)
+        seg = (torch.arange(nseq + 1, dtype=torch.int32) * per).to(dev)
+        reps = 5 if tag == "prefill" else 20
+        a = rn(n, W)
+        # dense feed-forward's clamped gate / up pair; beside Pukatar's silu pair
+        w_gu, act = wt(2 * ff, W), torch.empty(n, ff, device=dev)
+        for name, opts in (("linear_clamped_gate_up", dict(epilogue=D.EPI_CLAMP_GLU, act_a=1.702, act_b=7.0)), ("pukatar_linear_gate_up", dict(epilogue=D.EPI_SILU_MUL))):
+            t = _time(lambda: D.linear(a, w_gu, act, **opts), reps)
+            row(f"{name}_{tag}", t, flops=4.0 * n * ff * W, bytes_=4.0 * ff * W + 4.0 * n * (W + ff))
+        # mixture of experts: sigmoid scores, the weight on the experts' input; beside Pukatar's
+        w_r = (rn(E + 1, W) * 0.1).to(torch.bfloat16)
+        w_e = w_r[:E].contiguous()
+        idx, wgt, rb, sg = torch.empty(n, top, dtype=torch.int32, device=dev), torch.empty(n, top, device=dev), torch.zeros(E, device=dev), torch.empty(n, device=dev)
+        rbytes = 4.0 * n * (W + 2 * top) + 2.0 * E * W
+        rk_ = dict(entries=E, correction=None, groups=1, keep=1, top=top, scale=1.0, idx=idx, wgt=wgt, n=n)
+        t = _time(lambda: D.route_topk(None, h=a, w=w_r, bias=rb, chosen_softmax=True, gate_out=sg, **rk_), reps)
+        row(f"pukatar_route_{tag}", t, bytes_=rbytes)
+        t = _time(lambda: D.route_topk(None, h=a, w=w_e, sigmoid_scores=True, raw_weights=True, **rk_), reps)
+        row(f"route_sigmoid_{tag}", t, bytes_=rbytes)
+        i32 = dict(dtype=torch.int32, device=dev)
+        goff, ptok, prow, pwgt = torch.empty(E + 1, **i32), torch.empty(n * top, **i32), torch.empty(n * top, **i32), torch.empty(n * top, device=dev)
+        pl = dict(n=n, top=top, experts=E, group_off=goff, pair_token=ptok, pair_row=prow)
+        t = _time(lambda: D.moe_plan(idx, **pl), reps)
+        row(f"pukatar_moe_plan_{tag}", t, bytes_=4.0 * n * top * 3)
+        t = _time(lambda: D.moe_plan(idx, wgt=wgt, pair_wgt=pwgt, **pl), reps)
+        row(f"moe_plan_weights_{tag}", t, bytes_=4.0 * n * top * 5)
+        pairs = int(goff[-1])
+        w_egu, eact, ey = wt(E, 2 * eff, W), torch.empty(n * top, eff, device=dev), torch.empty(n * top, W, device=dev)
+        ek = dict(m=n, a_rows=ptok, batch=E, w_batch=2 * eff * W, group_off=goff)
+        for name, opts in (("experts_weighed_gate_up", dict(epilogue=D.EPI_SILU_MUL, row_scale=pwgt)), ("pukatar_experts_gate_up", dict(epilogue=D.EPI_CLAMP_GLU, act_a=1.702, act_b=7.0))):
+            t = _time(lambda: D.linear(a, w_egu, eact, **ek, **opts), reps)
+            row(f"{name}_{tag}", t, flops=4.0 * pairs * eff * W, bytes_=4.0 * E * eff * W + 4.0 * pairs * (W + eff))
+        sh, yo = rn(n, W), torch.empty(n, W, device=dev)
+        for name, wg, opts in (("moe_combine_plain", None, {}), ("pukatar_moe_combine", wgt, dict(shared_gate=sg))):
+            t = _time(lambda: D.moe_combine(ey, prow, wg, a, sh, yo, n=n, top=top, width=W, **opts), reps)
+            row(f"{name}_{tag}", t, bytes_=4.0 * n * W * (top + 2))
+        # residual: one result / two summed, a factor per column, the next norm; what a further pass starts from; beside Pukatar's
+        st, y, y2, h = rn(1, n, W), rn(n, W), rn(n, W), torch.empty(n, W, device=dev)
+        wn, bn, ls, one = torch.ones(W, device=dev), torch.zeros(W, device=dev), torch.ones(W, device=dev), torch.ones(1, device=dev)
+        nk_ = dict(out_w=one, norm_w=wn, eps=1e-6, h=h)
+        t = _time(lambda: D.streams_step(st, y=y, y_scale=ls, **nk_), reps)
+        row(f"residual_scaled_norm_{tag}", t, bytes_=4.0 * n * W * 4)
+        t = _time(lambda: D.streams_step(st, y=y, y2=y2, y_scale=ls, **nk_), reps)
+        row(f"residual_two_results_scaled_norm_{tag}", t, bytes_=4.0 * n * W * 5)
+        t = _time(lambda: D.streams_step(st, y=y, y2=y2, norm_b=bn, h_center=True, **nk_), reps)
+        row(f"pukatar_residual_two_results_norm_{tag}", t, bytes_=4.0 * n * W * 5)
+        t = _time(lambda: D.streams_step(st, y=y, **nk_), reps)
+        row(f"loop_entry_{tag}", t, bytes_=4.0 * n * W * 4)
+        # latent attention: the queries' low-rank norm + map, norm / rotation / cache write, attention, value map with the heads' gates; beside Fukatar's
+        plen = seq if tag == "prefill" else ctx
+        nb = (plen + 15) // 16
+        bt = torch.arange(nseq * nb, dtype=torch.int32, device=dev).view(nseq, nb).contiguous()
+        ld = rq + r + rd + (H + 7) // 8 * 8
+        P = rn(n, ld) * 0.3
+        qh, width = dm + rd, r + rd
+        qn, cn, inv = torch.ones(rq, device=dev), torch.ones(r, device=dev), torch.rand(rd // 2, device=dev, generator=g)
+        w_uq, Qs = wt(H * qh, rq), torch.empty(n, H * qh, device=dev)
+        qb = 2.0 * H * qh * rq + 4.0 * n * (rq + H * qh)
+        t = _time(lambda: _query_map(D, P, qn, w_uq, Qs, n, rq), reps)
+        row(f"latent_query_norm_and_map_{tag}", t, flops=2.0 * n * H * qh * rq, bytes_=qb)
+        t = _time(lambda: D.linear(P, w_uq, Qs, m=n), reps)
+        row(f"pukatar_linear_same_size_{tag}", t, flops=2.0 * n * H * qh * rq, bytes_=qb)
+        lc, lc0 = (rn(nseq * nb, 16, width) * 0.5).to(torch.bfloat16), (rn(nseq * nb, 16, r) * 0.5).to(torch.bfloat16)
+        Q = rn(n, H * width) * 0.1
+        pk = dict(heads=H, dim=dm, kv_rank=r, c_norm_w=cn, eps=1e-6, positions=pos, slot_ids=slots, block_table=bt, block_size=16, q=Q, n=n)
+        t = _time(lambda: D.latent_prep(P, q_off=0, dkv_off=rq, rot_dim=rd, rot_dims=rd, inv_freq=inv, cache=lc, q_src=Qs, rot_mult=1.1, **pk), reps)
+        row(f"latent_prep_rotated_{tag}", t, bytes_=4.0 * n * (width + 2 * H * rd) + 2.0 * n * width)
+        P0 = rn(n, H * dm + r)
+        t = _time(lambda: D.latent_prep(P0, q_off=0, dkv_off=H * dm, rot_dim=0, rot_dims=0, inv_freq=None, cache=lc0, **pk), reps)
+        row(f"fukatar_latent_prep_{tag}", t, bytes_=4.0 * n * r + 2.0 * n * r)
+        P1 = rn(n, H * qh + width)
+        t = _time(lambda: D.latent_prep(P1, q_off=0, dkv_off=H * qh, rot_dim=rd, rot_dims=rd, inv_freq=inv, cache=lc, **pk), reps)
+        row(f"morilorn_latent_prep_{tag}", t, bytes_=4.0 * n * (width + 2 * H * rd) + 2.0 * n * width)
+        keys = seq * (seq + 1) / 2 * nseq if tag == "prefill" else float(ctx) * n
+        mode = 3 if tag == "prefill" else 2
+        sink, ol = torch.zeros(H, device=dev), torch.empty(n, H * r, device=dev)
+        sp = 1 if tag == "prefill" else max(1, min(1024 // max(1, n * ((H + 15) // 16)), int(keys / n) // 64, 64))
+        ws = torch.empty(max(1, D.latent_attn_workspace_floats(n, H, r, sp)), device=dev) if sp > 1 else None
+        for name, cache, rr in (("latent_attention_rotated_sink", lc, rd), ("fukatar_latent_attention_sink", lc0, 0)):
+            t = _time(lambda: D.latent_attn(Q, cache, bt, slots, pos, window=0, scale=0.1, heads=H, kv_rank=r, rot_dim=rr, out=ol, n=n, mode=mode, splits=sp, workspace=ws, sink=sink), reps)
+            row(f"{name}_{tag}", t, flops=2.0 * keys * H * (2 * r + rr), bytes_=(2.0 * keys * (r + rr) if tag == "decode" else 0.0) + 4.0 * n * H * (2 * r + rr))
+        w_uv, og = wt(H, dv, r), torch.empty(n, H * dv, device=dev)
+        uvk = dict(m=n, n=dv, k=r, lda=H * r, ldc=H * dv, batch=H, a_batch=r, w_batch=dv * r, c_batch=dv)
+        for name, opts in (("latent_values_gated", dict(epilogue=D.EPI_ROW_SIGMOID, e=P, e_off=rq + r + rd, lde=ld, e_batch=1)), ("fukatar_latent_values", {})):
+            t = _time(lambda: D.linear(ol, w_uv, og, **uvk, **opts), reps)
+            row(f"{name}_{tag}", t, flops=2.0 * n * H * dv * r, bytes_=2.0 * H * dv * r + 4.0 * n * H * (r + dv))
+        # left attention: prep (norms per head, rotation, cache write), window; beside Pukatar's (no norms; kept first positions and sinks)
+        gs, nq, nk, nv = dl + vl, Hl * dl, Gl * dl, Gl * vl
+        kc = (rn(nseq * nb, 16, Gl * gs) * 0.5).to(torch.bfloat16)
+        Pl = rn(n, nq + nk + nv) * 0.3
+        ql, oa = torch.empty(n, Hl * gs, device=dev), torch.empty(n, Hl * vl, device=dev)
+        invl, hw = torch.rand(dl // 2, device=dev, generator=g), torch.ones(dl, device=dev)
+        pk = dict(q_off=0, k_off=nq, v_off=nq + nk, heads=Hl, kv_heads=Gl, dim=dl, vdim=vl, eps=1e-6, rot_dims=dl, inv_freq=invl, head_norm=False, v_freq=None, scale=0.125,
+                  positions=pos, slot_ids=slots, block_table=bt, cache=kc, q=ql, n=n)
+        pbytes = 4.0 * n * (nq + nk + nv + Hl * gs) + 2.0 * n * Gl * gs
+        t = _time(lambda: D.rot_prep(Pl, q_norm_w=hw, k_norm_w=hw, norm_heads=True, interleaved=True, rot_mult=1.1, **pk), reps)
+        row(f"rot_prep_head_norms_{tag}", t, bytes_=pbytes)
+        t = _time(lambda: D.rot_prep(Pl, q_norm_w=None, k_norm_w=None, interleaved=False, rot_mult=1.0, **pk), reps)
+        row(f"pukatar_rot_prep_{tag}", t, bytes_=pbytes)
+        waves = 3072 if gs <= 64 else (2048 if gs <= 128 else 1024)
+        sinkl = torch.zeros(Hl, device=dev)
+        kk = dict(chunk=0, bias=None, heads=Hl, kv_heads=Gl, dim=dl, vdim=vl, out=oa, n=n, mode=mode)
+        for name, opts in (("window_attention", dict(sink=False, window=win)), ("pukatar_window_attention", dict(sink=True, sink_w=sinkl, window=win, keep_first=4))):
+            kf = opts.get("keep_first", 0)
+            seen = sum(min(p + 1, win + kf) for p in range(seq)) * nseq if tag == "prefill" else float(min(ctx, win + kf)) * n
+            sp = 1 if tag == "prefill" else max(1, min(waves // max(1, n * Gl * ((Hl // Gl + 15) // 16)), int(seen / n) // 64, 64))
+            ws = torch.empty(max(1, D.kattn_workspace_floats(n, Hl, Gl, vl, sp)), device=dev) if sp > 1 else None
+            t = _time(lambda: D.kattn(ql, kc, None, bt, slots, pos, splits=sp, workspace=ws, **kk, **opts), reps)
+            row(f"{name}_{tag}", t, flops=2.0 * seen * Hl * (dl + vl), bytes_=(2.0 * seen * Gl * gs if tag == "decode" else 0.0) + 4.0 * n * Hl * (gs + vl))
+        # right: low-rank decay, scan, gated head norm; beside Pukatar's delta rule
+        nd, rv = Hr * dk, Hr * dr
+        Pr = rn(n, 2 * nd + 2 * rv + R) * 0.5
+        a2, F, rate, dtb = wt(nd, R), torch.empty(n, nd, device=dev), torch.full((nd,), 1.0 / 8, device=dev), torch.linspace(-2.0, 6.0, nd, device=dev)
+        t = _time(lambda: D.linear(Pr, a2, F, m=n, a_off=2 * nd + 2 * rv, bias=dtb, epilogue=D.EPI_DECAY, e=rate), reps)
+        row(f"channel_decay_linear_{tag}", t, flops=2.0 * n * nd * R, bytes_=2.0 * nd * R + 4.0 * n * (R + nd))
+        state, ro, rg = torch.zeros(nseq, Hr, dr, dk, device=dev), torch.empty(n, rv, device=dev), torch.empty(n, rv, device=dev)
+        sc = dict(seg_start=seg, nseg=nseq, positions=pos, slot_ids=slots, state=state, out=ro, n=n)
+        sbytes = 4.0 * n * (3 * nd + 2 * rv) + 8.0 * nseq * Hr * dk * dr
+        t = _time(lambda: D.gla_scan(Pr, f=F, q_off=0, k_off=nd, f_off=0, v_off=2 * nd, heads=Hr, dim=dk, vdim=dr, q_scale=dk ** -0.5, **sc), reps)
+        row(f"gated_linear_scan_{tag}", t, flops=5.0 * n * Hr * dk * dr, bytes_=sbytes, peak=F32_TFLOPS)
+        Gt = torch.rand(n, 2 * Hr, device=dev, generator=g)
+        Xu = Pr * 0.1
+        t = _time(lambda: D.gdn_scan(Xu, Gt, f=F, q_off=0, k_off=nd, v_off=2 * nd, heads=Hr, kv_heads=Hr, dim=dk, vdim=dr, **sc), reps)
+        row(f"pukatar_channel_delta_scan_{tag}", t, flops=7.0 * n * Hr * dk * dr, bytes_=sbytes, peak=F32_TFLOPS)
+        nwv = torch.ones(dr, device=dev)
+        for name, sig in (("gated_head_norm", False), ("pukatar_gated_head_norm", True)):
+            t = _time(lambda: D.gate_norm(ro, nwv, rg, groups=Hr, eps=1e-6, z=Pr, z_off=2 * nd + rv, ldz=Pr.shape[-1], n=n, gate_after=True, width=rv, sigmoid=sig), reps)
+            row(f"{name}_{tag}", t, bytes_=4.0 * n * rv * 3)
+    return out
+
+
+def _query_map(D, P, qn, w_uq, out, n, rq):
+    cq = torch.empty(n, rq, device=P.device)
+    D.gate_norm(P, qn, cq, groups=1, eps=1e-6, y_off=0, ldy=P.shape[-1], n=n)
+    D.linear(cq, w_uq, out)
+
+
+def run_vepelix(args) -> dict:
+    from . import _lib, synth
+    from .model import GreedyDecoder
+    from .pukatar import PukatarModel
+    from .vepelix import VepelixModel
+    _lib.load(), _lib.load_dense()
+    dev = torch.device("cuda:0")
+    torch.cuda.set_device(dev)
+    batch, ctx, rows = args.batch, args.prompt_len, 4096
+    result = {"metric": "prefill / decode tokens/s of the Vepelix design beside Pukatar at equal sizes", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+              "warmup": args.warmup, "dtype": "bf16 matrix products, fp32 residual / norms / recurrences / attention math (both designs)", "data": "synthetic",
+              "config": {"batch": batch, "context": ctx, "prefill_step": f"{rows} rows = {rows // 512} prompts of 512 tokens"}, "sizes": {}}
+    for name in (args.design_sizes.split(",") if args.design_sizes else sorted(VEPELIX_SIZES)):
+        sz = VEPELIX_SIZES[name]
+        need_tokens = batch * (ctx + args.steps + args.warmup + 64)
+
+        def fill(m):
+            g = torch.Generator(device=dev).manual_seed(5)
+            for t in {id(t): t for t in m.kv.rows if t is not None}.values():
+                t.copy_((0.5 * torch.randn(t.shape, device=dev, generator=g)).to(t.dtype))
+            for d in m.kv.state:
+                for t in d.values():
+                    t.copy_(0.1 * torch.randn(t.shape, device=dev, generator=g))
+
+        entry = {}
+        for label, cfg, cls, weights in (("vepelix", synth.vepelix_config(**sz), VepelixModel, lambda c: synth.make_vepelix_weights(c, rank=PUKATAR_RANK)),
+                                         ("pukatar", synth.pukatar_config(**PUKATAR_SIZES[name]), PukatarModel, lambda c: synth.make_pukatar_weights(c, rank=PUKATAR_RANK))):
+            model = cls(cfg, weights(cfg), device=dev, dtype="bfloat16", max_seqs=batch, num_kv_blocks=need_tokens // 16)
+            p, d, ms = _steps(model, GreedyDecoder, batch, ctx, rows, 512, args.steps, args.warmup, fill, cfg.vocab, dev)
+            entry[label] = {"prefill_tokens_per_s": round(p, 1), "decode_tokens_per_s": round(d, 1), "decode_ms_per_step": round(ms, 3), "layers": cfg.num_layers,
+                            "layer_runs": len(cfg.layer_runs()), "shape": sz if label == "vepelix" else PUKATAR_SIZES[name]}
+            del model
+            torch.cuda.empty_cache()
+        entry["kernels"] = _vepelix_kernels(sz, rows, batch, ctx, dev)
+        result["sizes"][name] = entry
+    first = result["sizes"][sorted(result["sizes"])[0]]["vepelix"]
+    result["value"], result["ms_per_step"] = first["decode_tokens_per_s"], first["decode_ms_per_step"]
+    result["higher_is_better"], result["scaling"], result["vs_baseline"] = True, "weak", None
+    return result
+
+
 def main(args) -> int:
-    print(json.dumps({"dogalorn": run_dogalorn, "zabutar": run_zabutar, "fukatar": run_fukatar, "pukatar": run_pukatar}.get(args.design, run)(args)), flush=True)
+    print(json.dumps({"dogalorn": run_dogalorn, "zabutar": run_zabutar, "fukatar": run_fukatar, "pukatar": run_pukatar, "vepelix": run_vepelix}.get(args.design, run)(args)), flush=True)
     return 0

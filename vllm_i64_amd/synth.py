@@ -339,3 +339,71 @@ def make_pukatar_weights(cfg, seed: int = 0, std: float = 0.02, rank: int = 128)
                 glu(p + "mlp.shared.", f.shared_ff)
                 w[p + "mlp.shared.sg"] = rn(1, W)
     return w
+
+
+def vepelix_config(width: int = 1024, blocks: int = 3, loop_blocks: int = 1, heads: int = 16, dim: int = 64, rot_dim: int = 32, vdim: int = 64, kv_rank: int = 256,
+                   q_rank: int = 512, left_heads: int = 16, left_kv_heads: int = 4, left_dim: int = 64, left_vdim: int = 64, window: int = 1024, rec_heads: int = 8,
+                   rec_dim: int = 128, rec_vdim: int = 128, tau: float = 8.0, ff: int = 2752, experts: int = 8, top: int = 2, expert_ff: int = 896, shared_ff: int = 896,
+                   vocab: int = 32000):
+    """A Vepelix configuration with layers of a real model's proportions: `blocks` times (latent attention with a dense feed-forward, attention
+    beside gated linear attention with a mixture of experts, latent attention with a mixture, attention beside linear attention with a
+    mixture), the first loop_blocks of them run twice; random weights: make_vepelix_weights."""
+    from .config import VepelixConfig
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "shared": {"ff": shared_ff}, "router": {"experts": experts, "top": top}}
+    rot = lambda dims: {"base": 100000.0, "dims": dims, "scaling": {"factor": 4.0, "original": 1024, "fast": 32.0, "slow": 1.0}}
+    lat = {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank,
+                                                 "scale": (dim + rot_dim) ** -0.5, "rot": rot(rot_dim)}}
+    par = {"type": "parallel", "mixer": {"left": {"heads": left_heads, "kv_heads": left_kv_heads, "dim": left_dim, "vdim": left_vdim, "scale": left_dim ** -0.5,
+                                                  "rot": rot(left_dim), "mask": {"size": window}},
+                                         "right": {"heads": rec_heads, "dim": rec_dim, "vdim": rec_vdim, "tau": tau}, "left_scale": 0.7, "right_scale": 0.6}}
+    layers = []
+    for _ in range(blocks):
+        layers += [dict(lat, mlp=dense), dict(par, mlp=moe), dict(lat, mlp=moe), dict(par, mlp=moe)]
+    d = {"architecture": "Vepelix", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers}
+    if loop_blocks:
+        d["loop"] = {"start": 0, "stop": 4 * loop_blocks, "times": 2}
+    return VepelixConfig.from_dict(d)
+
+
+def make_vepelix_weights(cfg, seed: int = 0, std: float = 0.02, rank: int = 128) -> Dict[str, torch.Tensor]:
+    """bf16 N(0, std) matrices, norms of one (stored as zero where the weight is a distance from one), factors per column of one, sinks zero, a
+    low-rank decay map of `rank` with biases spread over the channels, a router wide enough that the experts' loads differ from token to
+    token."""
+    g = torch.Generator().manual_seed(seed)
+    W = cfg.width
+
+    def rn(*shape, s=std):
+        return torch.empty(*shape, dtype=torch.float32).normal_(0.0, s, generator=g).to(torch.bfloat16)
+
+    one, zero = (lambda *n: torch.ones(*n, dtype=torch.bfloat16)), (lambda *n: torch.zeros(*n, dtype=torch.bfloat16))
+    w = {"embed": rn(cfg.vocab, W), "head": rn(cfg.vocab, W), "final.norm": zero(W)}
+
+    def glu(p, ff):
+        w.update({p + "gate": rn(ff, W), p + "up": rn(ff, W), p + "down": rn(W, ff)})
+
+    for i, L in enumerate(cfg.layers):
+        p, m, f = f"l{i}.", L.mixer, L.mlp
+        mp = p + "mix."
+        w.update({p + "norm1": zero(W), p + "norm2": zero(W), p + "ls1": one(W), p + "ls2": one(W)})
+        if L.type == "latent_attention":
+            H = m.heads
+            w.update({mp + "dq": rn(m.q_rank, W), mp + "dq.norm": one(m.q_rank), mp + "uq": rn(m.q_width, m.q_rank), mp + "dkv": rn(m.cache_width, W),
+                      mp + "dkv.norm": one(m.kv_rank), mp + "uk": rn(H * m.dim, m.kv_rank), mp + "uv": rn(H * m.vdim, m.kv_rank), mp + "sink": zero(H), mp + "g": rn(H, W),
+                      mp + "o": rn(W, H * m.vdim)})
+        else:
+            a, r, lp, rp = m.left, m.right, mp + "left.", mp + "right."
+            rk, rv = r.heads * r.dim, r.heads * r.vdim
+            w.update({lp + "q": rn(a.heads * a.dim, W), lp + "k": rn(a.kv_heads * a.dim, W), lp + "v": rn(a.kv_heads * a.vdim, W), lp + "q.norm": one(a.dim),
+                      lp + "k.norm": one(a.dim), lp + "o": rn(W, a.heads * a.vdim), rp + "q": rn(rk, W), rp + "k": rn(rk, W), rp + "v": rn(rv, W), rp + "g": rn(rv, W),
+                      rp + "a1": rn(rank, W), rp + "a2": rn(rk, rank), rp + "a2.b": torch.linspace(-2.0, 6.0, rk).to(torch.bfloat16), rp + "norm": one(r.vdim),
+                      rp + "o": rn(W, rv)})
+        if f is not None and f.kind == "dense":
+            glu(p + "mlp.", f.ff)
+        elif f is not None:
+            w[p + "mlp.router"] = rn(f.experts, W, s=0.1)
+            for e in range(f.experts):
+                glu(f"{p}mlp.e{e}.", f.ff)
+            if f.shared_ff:
+                glu(p + "mlp.shared.", f.shared_ff)
+    return w
