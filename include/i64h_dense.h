@@ -38,6 +38,8 @@ int i64h_device_check(void);
  *   I64H_EPI_CLAMP_GLU: u = min(A W^T, act_b), w = clamp(A W2^T, -act_b, act_b), u * sigmoid(act_a * u) * (w + 1), laid out as I64H_EPI_GELU_MUL;
  *   I64H_EPI_ADD: v + E[b][m, n];  I64H_EPI_DECAY: exp(-E[b][m, n] * softplus(v))  (with lde = 0 E is one row for all m);
  *   I64H_EPI_ROW_SIGMOID: v * sigmoid(E[b][m]), one gate for all columns of a row (a head's gate where the batch is the heads).
+ *   I64H_EPI_IN_NORM: the input row is RMS-normed over its K columns first, A[m] / sqrt(mean(A[m]^2) + in_eps) * in_norm_w (fp32 [K], given
+ *   exactly with this epilogue): the weights multiply what is staged, the row's factor the sums.
  *   row_scale (may be NULL; fp32, one per row of C, the gate / up epilogues only): both sums are multiplied by row_scale[m] first - the
  *   input row times that factor.
  *   bias (may be NULL; fp32 [N], batch stride bias_batch) is added to the sum before any epilogue but the three gate / up ones.
@@ -60,6 +62,7 @@ int i64h_device_check(void);
 #define I64H_EPI_ADD 10
 #define I64H_EPI_DECAY 11
 #define I64H_EPI_ROW_SIGMOID 12
+#define I64H_EPI_IN_NORM 13
 #define I64H_SKINNY_ROWS 8
 typedef struct {
     const float* A;
@@ -83,6 +86,8 @@ typedef struct {
     float act_a, act_b;
     const int32_t* group_off;
     const float* row_scale;
+    const float* in_norm_w;
+    float in_eps;
 } i64h_linear;
 int i64h_linear_run(const i64h_linear* d, void* stream);
 
@@ -264,6 +269,7 @@ typedef struct {
     const float* y_scale;
 } i64h_streams_args;
 int i64h_streams_step(const i64h_streams_args* d, void* stream);
+int i64h_set_residual_form(int32_t on); /* tuning / test knob: 1 (default) = one stream and results without norms of their own take the kernel that keeps the row in registers (16-byte rows) */
 
 /* ---- causal per-channel convolution with carried inputs + silu ---------------------------------------------------------------------
  * out[t, c] = silu(bias[c] + sum_k w[c, k] * in(t, taps - 1 - k)),  in(t, d) = the input of channel c d positions before row t:

@@ -229,6 +229,7 @@ DENSE_SIGNATURES: Dict[str, str] = {
     "i64h_gdn_gates": "pp",
     "i64h_gdn_scan": "pp",
     "i64h_set_gdn_scan_form": "i",
+    "i64h_set_residual_form": "i",
     "i64h_gla_gates": "pp",
     "i64h_gla_scan": "pp",
     "i64h_route_topk": "pp",
@@ -241,7 +242,7 @@ class Linear(ctypes.Structure):
     """Mirror of i64h_linear (include/i64h_dense.h)."""
     _fields_ = [("A", _P), ("lda", _L), ("a_rows", _P), ("W", _P), ("C", _P), ("ldc", _L), ("M", _L), ("N", _I), ("K", _I), ("batch", _I),
                 ("a_batch", _L), ("w_batch", _L), ("c_batch", _L), ("exact", _I), ("epilogue", _I), ("E", _P), ("lde", _L), ("e_batch", _L),
-                ("softcap", _F), ("bias", _P), ("bias_batch", _L), ("scale", _F), ("act_a", _F), ("act_b", _F), ("group_off", _P), ("row_scale", _P)]
+                ("softcap", _F), ("bias", _P), ("bias_batch", _L), ("scale", _F), ("act_a", _F), ("act_b", _F), ("group_off", _P), ("row_scale", _P), ("in_norm_w", _P), ("in_eps", _F)]
 
 
 class PostNorm(ctypes.Structure):

@@ -1002,8 +1002,8 @@ def _vepelix_kernels(sz, rows, batch, ctx, dev):
         qn, cn, inv = torch.ones(rq, device=dev), torch.ones(r, device=dev), torch.rand(rd // 2, device=dev, generator=g)
         w_uq, Qs = wt(H * qh, rq), torch.empty(n, H * qh, device=dev)
         qb = 2.0 * H * qh * rq + 4.0 * n * (rq + H * qh)
-        t = _time(lambda: _query_map(D, P, qn, w_uq, Qs, n, rq), reps)
-        row(f"latent_query_norm_and_map_{tag}", t, flops=2.0 * n * H * qh * rq, bytes_=qb)
+        t = _time(lambda: D.linear(P, w_uq, Qs, m=n, in_norm_w=qn, in_eps=1e-6), reps)
+        row(f"linear_normed_input_{tag}", t, flops=2.0 * n * H * qh * rq, bytes_=qb)
         t = _time(lambda: D.linear(P, w_uq, Qs, m=n), reps)
         row(f"pukatar_linear_same_size_{tag}", t, flops=2.0 * n * H * qh * rq, bytes_=qb)
         lc, lc0 = (rn(nseq * nb, 16, width) * 0.5).to(torch.bfloat16), (rn(nseq * nb, 16, r) * 0.5).to(torch.bfloat16)
@@ -1073,12 +1073,6 @@ def _vepelix_kernels(sz, rows, batch, ctx, dev):
             t = _time(lambda: D.gate_norm(ro, nwv, rg, groups=Hr, eps=1e-6, z=Pr, z_off=2 * nd + rv, ldz=Pr.shape[-1], n=n, gate_after=True, width=rv, sigmoid=sig), reps)
             row(f"{name}_{tag}", t, bytes_=4.0 * n * rv * 3)
     return out
-
-
-def _query_map(D, P, qn, w_uq, out, n, rq):
-    cq = torch.empty(n, rq, device=P.device)
-    D.gate_norm(P, qn, cq, groups=1, eps=1e-6, y_off=0, ldy=P.shape[-1], n=n)
-    D.linear(cq, w_uq, out)
 
 
 def run_vepelix(args) -> dict:

@@ -492,14 +492,19 @@ __device__ __forceinline__ int bl_wave_argmax(float v, int idx, float& best) {
 }
 
 #define RT_MAX_TOP 32
+#define RT_SPLIT_ROWS 512      // launches of at most so many rows give every row a workgroup
+// SPLIT: a workgroup per row - its four waves share the columns of the router's products, the first one goes on with their sums (few
+// rows: one wave's chain of loads is what a launch would wait for).
+template <bool SPLIT>
 __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p) {
-    extern __shared__ float rt_lds[];   // per wave: [E] scores, [E] choice values, [groups] group flags
+    extern __shared__ float rt_lds[];   // per wave: [E] scores, [E] choice values, [groups] group flags; SPLIT: once, and [4][E + 1] partial products
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-    const int64_t t = (int64_t)blockIdx.x * 4 + wid;
-    if (t >= p.n) return;     // (a whole wave leaves; no workgroup barrier below)
+    const int64_t t = SPLIT ? (int64_t)blockIdx.x : (int64_t)blockIdx.x * 4 + wid;
+    if (t >= p.n) return;     // (a whole wave leaves; without SPLIT there is no workgroup barrier below)
     const int E = p.E, G = p.groups > 1 ? p.groups : 1, gsz = E / G;
     // volatile: lanes read what another lane of the wave wrote (one wave: program order is enough, no barrier)
-    volatile float* sc = rt_lds + (size_t)wid * (2 * E + G);
+    volatile float* sc = rt_lds + (SPLIT ? 0 : (size_t)wid * (2 * E + G));
+    float* part = rt_lds + 2 * E + G;
     volatile float* ch = sc + E;
     volatile float* gflag = ch + E;
     if (p.W) {      // the router's own products: eight entries at a time, every lane a share of the columns, fp32 throughout
@@ -511,7 +516,7 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
         for (int e0 = 0; e0 < rows; e0 += 8) {
             float acc[8] = {0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f, 0.0f};
             if (vec) {
-                for (int k = lane * 4; k < K; k += 256) {
+                for (int k = (SPLIT ? threadIdx.x : lane) * 4; k < K; k += SPLIT ? 1024 : 256) {
                     const float4 x = *(const float4*)(h + k);
 #pragma unroll
                     for (int j = 0; j < 8; ++j) {
@@ -525,7 +530,7 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
                     }
                 }
             } else {
-                for (int k = lane; k < K; k += 64) {
+                for (int k = SPLIT ? threadIdx.x : lane; k < K; k += SPLIT ? 256 : 64) {
                     const float x = h[k];
 #pragma unroll
                     for (int j = 0; j < 8; ++j)
@@ -535,8 +540,21 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const i64h_route_args p
 #pragma unroll
             for (int j = 0; j < 8; ++j) {
                 const float v = wave_sum(acc[j]);
+                if (SPLIT) {
+                    if (lane == 0 && e0 + j < rows) part[wid * rows + e0 + j] = v;
+                    continue;
+                }
                 if (lane == 0 && e0 + j < E) ch[e0 + j] = p.bias ? v + p.bias[e0 + j] : v;
                 if (lane == 0 && e0 + j == E && p.gate_out) p.gate_out[t] = bl_sigmoid(v);
+            }
+        }
+        if (SPLIT) {
+            __syncthreads();
+            if (wid > 0) return;
+            for (int e = lane; e < rows; e += 64) {
+                const float v = (part[e] + part[rows + e]) + (part[2 * rows + e] + part[3 * rows + e]);
+                if (e < E) ch[e] = p.bias ? v + p.bias[e] : v;
+                else p.gate_out[t] = bl_sigmoid(v);
             }
         }
     } else {
@@ -837,8 +855,11 @@ int i64h_route_topk(const i64h_route_args* dp, void* stream) {
     I64H_CHECK_ARG(d.groups <= 1 || d.keep * (d.E / d.groups) >= d.top, "route_topk: %d kept groups of %d entries hold fewer than top %d", d.keep, d.E / (d.groups > 0 ? d.groups : 1), d.top);
     I64H_CHECK_ARG(d.idx && d.wgt && ((d.logits && d.ld >= d.E) || (d.W && d.h && d.K > 0 && d.ldh >= d.K)), "route_topk: null operand or row stride below the row");
     if (d.n == 0) return 0;
-    const size_t lds = 4 * (size_t)(2 * d.E + (d.groups > 1 ? d.groups : 1)) * 4;
-    hipLaunchKernelGGL(route_topk_kernel, dim3((unsigned)((d.n + 3) / 4)), dim3(256), lds, (hipStream_t)stream, d);
+    const size_t own = (size_t)(2 * d.E + (d.groups > 1 ? d.groups : 1));
+    if (d.W && d.n <= RT_SPLIT_ROWS)
+        hipLaunchKernelGGL(route_topk_kernel<true>, dim3((unsigned)d.n), dim3(256), (own + 4 * (size_t)(d.E + 1)) * 4, (hipStream_t)stream, d);
+    else
+        hipLaunchKernelGGL(route_topk_kernel<false>, dim3((unsigned)((d.n + 3) / 4)), dim3(256), 4 * own * 4, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();
     return 0;
 }

@@ -94,15 +94,29 @@ __global__ __launch_bounds__(256) void linear_tile_kernel(const i64h_linear p, c
     const int M = (int)min((int64_t)64, rows - m0);  // rows of this tile
     const int N = p.N, K = p.K;
     const int lr = tid >> 2, lc = (tid & 3) * 8;
+    constexpr bool INN = EPI == I64H_EPI_IN_NORM;
+    __shared__ float sRow[INN ? 64 : 1];
+    float ssq = 0.0f;
     const bool aok = lr < M, bok = n0 + lr < N;
     const int64_t arow = aok ? (p.a_rows ? (int64_t)p.a_rows[m0 + lr] : m0 + lr) : 0;
     const float* pa = p.A + b * p.a_batch + arow * p.lda;
     const uint16_t* pw = (const uint16_t*)p.W + b * p.w_batch + (int64_t)(bok ? n0 + lr : 0) * K;
     const uint16_t* pw2 = pw + (int64_t)N * K;
-    float ra[8];
+    float ra[8], rn[INN ? 8 : 1];
     uint16_t rb[8], rb2[8];
     auto gload = [&](int k0) {
         const int k = k0 + lc;
+        if (INN) {
+            if (vecA && k + 8 <= K) {
+                const float4 u = *(const float4*)(p.in_norm_w + k), v = *(const float4*)(p.in_norm_w + k + 4);
+                const float w[8] = {u.x, u.y, u.z, u.w, v.x, v.y, v.z, v.w};
+#pragma unroll
+                for (int i = 0; i < 8; ++i) rn[INN ? i : 0] = w[i];
+            } else {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) rn[INN ? i : 0] = k + i < K ? p.in_norm_w[k + i] : 0.0f;
+            }
+        }
         if (aok && vecA && k + 8 <= K) {
             const float4 u = *(const float4*)(pa + k), v = *(const float4*)(pa + k + 4);
             ra[0] = u.x; ra[1] = u.y; ra[2] = u.z; ra[3] = u.w; ra[4] = v.x; ra[5] = v.y; ra[6] = v.z; ra[7] = v.w;
@@ -122,6 +136,13 @@ __global__ __launch_bounds__(256) void linear_tile_kernel(const i64h_linear p, c
         }
     };
     auto lstore = [&](int buf) {
+        if (INN) {      // the row's squares as they come, the norm's weights on what is staged
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                ssq = fmaf(ra[i], ra[i], ssq);
+                ra[i] *= rn[INN ? i : 0];
+            }
+        }
         if (EXACT) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
@@ -193,6 +214,12 @@ __global__ __launch_bounds__(256) void linear_tile_kernel(const i64h_linear p, c
         if (kt + 1 < KT) lstore(cur ^ 1);
         __syncthreads();
     }
+    if (INN) {      // four neighbouring lanes hold a row's shares
+        ssq += __shfl_xor(ssq, 1);
+        ssq += __shfl_xor(ssq, 2);
+        if ((tid & 3) == 0) sRow[INN ? lr : 0] = 1.0f / sqrtf(ssq / (float)K + p.in_eps);
+        __syncthreads();
+    }
     float* C = p.C + b * p.c_batch;
 #pragma unroll
     for (int i = 0; i < 2; ++i)
@@ -204,7 +231,7 @@ __global__ __launch_bounds__(256) void linear_tile_kernel(const i64h_linear p, c
 #pragma unroll
             for (int j = 0; j < 2; ++j) {
                 const int c = n0 + wn * 32 + j * 16 + fr;
-                if (c < N) C[r * p.ldc + c] = dn_epilogue<EPI>(p, acc[i][j][reg], acc2[i][j][reg], b, r, c);
+                if (c < N) C[r * p.ldc + c] = dn_epilogue<EPI>(p, INN ? acc[i][j][reg] * sRow[INN ? rl : 0] : acc[i][j][reg], acc2[i][j][reg], b, r, c);
             }
         }
 }
@@ -337,6 +364,8 @@ template <int EPI>
 __global__ __launch_bounds__(256) void linear_skinny_kernel(const i64h_linear p, const int cols_per_block) {
     constexpr bool DUAL = dn_dual(EPI);
     constexpr int CPW = 4, MR = I64H_SKINNY_ROWS;
+    constexpr bool INN = EPI == I64H_EPI_IN_NORM;
+    __shared__ float sRow[INN ? MR : 1][4];
     extern __shared__ __attribute__((aligned(16))) uint16_t sa[];  // [M][K]
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int64_t b = blockIdx.z;
@@ -344,9 +373,19 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(const i64h_linear p,
     for (int m = 0; m < M; ++m) {
         const int64_t arow = p.a_rows ? (int64_t)p.a_rows[m] : m;
         const float* pa = p.A + b * p.a_batch + arow * p.lda;
+        float ssq = 0.0f;
         for (int k = tid * 4; k < K; k += 1024) {
-            const float4 v = *(const float4*)(pa + k);
+            float4 v = *(const float4*)(pa + k);
+            if (INN) {
+                ssq = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ssq))));
+                const float4 w = *(const float4*)(p.in_norm_w + k);
+                v.x *= w.x, v.y *= w.y, v.z *= w.z, v.w *= w.w;
+            }
             *(uint2*)&sa[m * K + k] = make_uint2(dn_bf16_rne(v.x) | (dn_bf16_rne(v.y) << 16), dn_bf16_rne(v.z) | (dn_bf16_rne(v.w) << 16));
+        }
+        if (INN) {
+            ssq = wave_sum(ssq);
+            if (lane == 0) sRow[INN ? m : 0][wid] = ssq;
         }
     }
     __syncthreads();
@@ -403,7 +442,11 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(const i64h_linear p,
 #pragma unroll
             for (int m = 0; m < MR; ++m) {
                 if (m >= M) break;
-                const float s = wave_sum(acc[j][m]);
+                float s = wave_sum(acc[j][m]);
+                if (INN) {
+                    const float* q = sRow[INN ? m : 0];
+                    s *= 1.0f / sqrtf(((q[0] + q[1]) + (q[2] + q[3])) / (float)K + p.in_eps);
+                }
                 const float s2 = DUAL ? wave_sum(acc2[j][m]) : 0.0f;
                 const int c = c0 + j;
                 if (lane == 0 && c < c_end) C[(int64_t)m * p.ldc + c] = dn_epilogue<EPI>(p, s, s2, b, m, c);
@@ -420,7 +463,10 @@ __global__ __launch_bounds__(256) void linear_skinny_kernel(const i64h_linear p,
 template <int EPI, int NW>
 __global__ __launch_bounds__(64 * NW) void linear_rows64_kernel(const i64h_linear p) {
     constexpr bool DUAL = dn_dual(EPI);
+    constexpr bool INN = EPI == I64H_EPI_IN_NORM;
     __shared__ float red[DUAL ? 2 : 1][NW][64][17];
+    __shared__ float sRow[INN ? NW : 1][64];
+    float ssq[4] = {0.0f, 0.0f, 0.0f, 0.0f};
     const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
     const int n = lane & 15, kg = lane >> 4;
     const int64_t b = blockIdx.z;
@@ -458,12 +504,16 @@ __global__ __launch_bounds__(64 * NW) void linear_rows64_kernel(const i64h_linea
     constexpr int U = 2;
     for (int kt = wv; kt < KT; kt += U * NW) {
         uint4 wf[U], wf2[U];
-        float4 au[U][4], av[U][4];
+        float4 au[U][4], av[U][4], nu[INN ? U : 1], nv[INN ? U : 1];
 #pragma unroll
         for (int h = 0; h < U; ++h) {
             const int k = (kt + h * NW) * 32 + kg * 8;
             const bool kin = kt + h * NW < KT && k < K;
             wf[h] = wf2[h] = make_uint4(0, 0, 0, 0);
+            if (INN) {
+                nu[INN ? h : 0] = kin ? *(const float4*)(p.in_norm_w + k) : make_float4(0, 0, 0, 0);
+                nv[INN ? h : 0] = kin ? *(const float4*)(p.in_norm_w + k + 4) : make_float4(0, 0, 0, 0);
+            }
             if (cok && kin) {
                 wf[h] = *(const uint4*)(pw + k);
                 if (DUAL) wf2[h] = *(const uint4*)(pw2 + k);
@@ -482,7 +532,13 @@ __global__ __launch_bounds__(64 * NW) void linear_rows64_kernel(const i64h_linea
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 if (i < mblocks) {
-                    const float4 u = au[h][i], v = av[h][i];
+                    float4 u = au[h][i], v = av[h][i];
+                    if (INN) {
+                        ssq[i] = fmaf(u.x, u.x, fmaf(u.y, u.y, fmaf(u.z, u.z, fmaf(u.w, u.w, ssq[i]))));
+                        ssq[i] = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ssq[i]))));
+                        u.x *= nu[INN ? h : 0].x, u.y *= nu[INN ? h : 0].y, u.z *= nu[INN ? h : 0].z, u.w *= nu[INN ? h : 0].w;
+                        v.x *= nv[INN ? h : 0].x, v.y *= nv[INN ? h : 0].y, v.z *= nv[INN ? h : 0].z, v.w *= nv[INN ? h : 0].w;
+                    }
                     const uint4 af = make_uint4(dn_bf16_rne(u.x) | (dn_bf16_rne(u.y) << 16), dn_bf16_rne(u.z) | (dn_bf16_rne(u.w) << 16),
                                                 dn_bf16_rne(v.x) | (dn_bf16_rne(v.y) << 16), dn_bf16_rne(v.z) | (dn_bf16_rne(v.w) << 16));
                     acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dn_v8bf, af), __builtin_bit_cast(dn_v8bf, wf[h]), acc[i], 0, 0, 0);
@@ -497,6 +553,15 @@ __global__ __launch_bounds__(64 * NW) void linear_rows64_kernel(const i64h_linea
             red[0][wv][i * 16 + kg * 4 + g][n] = acc[i][g];
             if (DUAL) red[DUAL ? 1 : 0][wv][i * 16 + kg * 4 + g][n] = acc2[i][g];
         }
+    if (INN) {      // lanes n, n + 16, n + 32, n + 48 hold shares of row n of a block
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            float q = ssq[i];
+            q += __shfl_xor(q, 16);
+            q += __shfl_xor(q, 32);
+            if (kg == 0) sRow[INN ? wv : 0][i * 16 + n] = q;
+        }
+    }
     __syncthreads();
     float* C = p.C + b * p.c_batch;
     for (int e = tid; e < 64 * 16; e += 64 * NW) {
@@ -507,6 +572,12 @@ __global__ __launch_bounds__(64 * NW) void linear_rows64_kernel(const i64h_linea
         for (int w = 0; w < NW; ++w) {
             s += red[0][w][m][c];
             if (DUAL) s2 += red[DUAL ? 1 : 0][w][m][c];
+        }
+        if (INN) {
+            float q = 0.0f;
+#pragma unroll
+            for (int w = 0; w < NW; ++w) q += sRow[INN ? w : 0][m];
+            s *= 1.0f / sqrtf(q / (float)K + p.in_eps);
         }
         C[(g0 + m) * p.ldc + n0 + c] = dn_epilogue<EPI>(p, s, s2, b, g0 + m, n0 + c);
     }
@@ -714,6 +785,7 @@ static void launch_tile(const i64h_linear& d, dim3 grid, hipStream_t s, int vecA
         case I64H_EPI_ADD: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_ADD>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_DECAY>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_ROW_SIGMOID>), grid, dim3(256), 0, s, d, vecA, vecW); break;
+        case I64H_EPI_IN_NORM: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_IN_NORM>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_SCALE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
         default: hipLaunchKernelGGL((linear_tile_kernel<EXACT, I64H_EPI_STORE>), grid, dim3(256), 0, s, d, vecA, vecW); break;
     }
@@ -740,16 +812,17 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
     const i64h_linear& d = *dp;
     I64H_CHECK_ARG(d.M >= 0 && d.N > 0 && d.K > 0 && d.batch > 0, "linear: bad sizes M=%lld N=%d K=%d batch=%d", (long long)d.M, d.N, d.K, d.batch);
     I64H_CHECK_ARG(d.A && d.W && d.C, "linear: null operand");
-    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_ROW_SIGMOID, "linear: epilogue %d", d.epilogue);
+    I64H_CHECK_ARG(d.epilogue >= 0 && d.epilogue <= I64H_EPI_IN_NORM, "linear: epilogue %d", d.epilogue);
     I64H_CHECK_ARG((d.epilogue != I64H_EPI_MUL_SIGMOID && d.epilogue != I64H_EPI_ADD && d.epilogue != I64H_EPI_DECAY && d.epilogue != I64H_EPI_ROW_SIGMOID) || d.E, "linear: epilogue %d needs E", d.epilogue);
     I64H_CHECK_ARG(d.epilogue != I64H_EPI_CLAMP_GLU || d.act_b > 0.0f, "linear: bound %g of the clamped gate / up epilogue", (double)d.act_b);
     I64H_CHECK_ARG(d.epilogue != I64H_EPI_SOFTCAP || d.softcap > 0.0f, "linear: soft cap %g", (double)d.softcap);
     I64H_CHECK_ARG(!dn_dual(d.epilogue) || !d.bias, "linear: the gate / up epilogues take no bias");
+    I64H_CHECK_ARG((d.epilogue == I64H_EPI_IN_NORM) == (d.in_norm_w != nullptr), "linear: the normed input and its weights come together");
     I64H_CHECK_ARG(dn_dual(d.epilogue) || !d.row_scale, "linear: row factors belong to the gate / up epilogues");
     I64H_CHECK_ARG(d.lda >= d.K || d.M <= 1, "linear: lda %lld < K %d", (long long)d.lda, d.K);
     I64H_CHECK_ARG(d.batch <= 65535 && (d.M + 63) / 64 <= 65535, "linear: grid too large");
     if (d.M == 0) return 0;
-    const int vecA = (uintptr_t)d.A % 16 == 0 && d.lda % 4 == 0 && d.a_batch % 4 == 0;
+    const int vecA = (uintptr_t)d.A % 16 == 0 && d.lda % 4 == 0 && d.a_batch % 4 == 0 && (uintptr_t)d.in_norm_w % 16 == 0;
     const int vecW = (uintptr_t)d.W % 16 == 0 && d.K % 8 == 0 && d.w_batch % 8 == 0;
     hipStream_t s = (hipStream_t)stream;
     const size_t lds = (size_t)d.M * d.K * 2;
@@ -769,6 +842,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             case I64H_EPI_ADD: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_ADD>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_DECAY>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_ROW_SIGMOID>), grid, dim3(256), lds, s, d, cpb); break;
+            case I64H_EPI_IN_NORM: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_IN_NORM>), grid, dim3(256), lds, s, d, cpb); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_SCALE>), grid, dim3(256), lds, s, d, cpb); break;
             default: hipLaunchKernelGGL((linear_skinny_kernel<I64H_EPI_STORE>), grid, dim3(256), lds, s, d, cpb); break;
         }
@@ -790,6 +864,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
             case I64H_EPI_ADD: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_ADD, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_DECAY: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_DECAY, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_ROW_SIGMOID: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_ROW_SIGMOID, 8>), grid, dim3(512), 0, s, d); break;
+            case I64H_EPI_IN_NORM: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_IN_NORM, 8>), grid, dim3(512), 0, s, d); break;
             case I64H_EPI_SCALE: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_SCALE, 8>), grid, dim3(512), 0, s, d); break;
             default: hipLaunchKernelGGL((linear_rows64_kernel<I64H_EPI_STORE, 8>), grid, dim3(512), 0, s, d); break;
         }
@@ -797,7 +872,7 @@ int i64h_linear_run(const i64h_linear* dp, void* stream) {
         return 0;
     }
     const int64_t tiles128 = ((d.N + 127) / 128) * ((d.M + 127) / 128) * (int64_t)d.batch;
-    if (g_tile128 && !d.group_off && !d.exact && tiles128 >= 256) {     // at least a workgroup per CU: the large tile pays
+    if (g_tile128 && !d.group_off && !d.exact && d.epilogue != I64H_EPI_IN_NORM && tiles128 >= 256) {     // at least a workgroup per CU: the large tile pays
         const dim3 grid((unsigned)((d.N + 127) / 128), (unsigned)((d.M + 127) / 128), (unsigned)d.batch);
         switch (d.epilogue) {
             case I64H_EPI_GELU_MUL: hipLaunchKernelGGL((linear_tile128_kernel<I64H_EPI_GELU_MUL>), grid, dim3(256), 0, s, d, vecA, vecW); break;

@@ -182,6 +182,71 @@ __global__ __launch_bounds__(256) void streams_kernel(const i64h_streams_args p)
     }
 }
 
+// The ordinary residual sum (one stream, results without norms of their own) with rows of whole 16-byte slices: the row stays in registers
+// between the write and the norm, NV slices of four columns per thread.
+template <int NV>
+__global__ __launch_bounds__(256) void residual_kernel(const i64h_streams_args p) {
+    __shared__ float red[4];
+    const int tid = threadIdx.x, W = p.W;
+    const int64_t m = blockIdx.x;
+    float* xs = p.streams + (p.rows ? (int64_t)p.rows[m] : m) * W;
+    const float ow = p.y ? p.out_w[0] : 0.0f;
+    float v[NV][4];
+    float ss = 0.0f, su = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = (i * 256 + tid) * 4;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[i][k] = 0.0f;
+        if (c >= W) continue;
+        const float4 x = *(const float4*)(xs + c);
+        v[i][0] = x.x, v[i][1] = x.y, v[i][2] = x.z, v[i][3] = x.w;
+        if (p.y) {
+            const float4 y = *(const float4*)(p.y + m * p.ldy + c);
+            float u[4] = {y.x, y.y, y.z, y.w};
+            if (p.y2) {
+                const float4 z = *(const float4*)(p.y2 + m * p.ldy2 + c);
+                u[0] += z.x, u[1] += z.y, u[2] += z.z, u[3] += z.w;
+            }
+            if (p.y_scale) {
+                const float4 s = *(const float4*)(p.y_scale + c);
+                u[0] *= s.x, u[1] *= s.y, u[2] *= s.z, u[3] *= s.w;
+            }
+#pragma unroll
+            for (int k = 0; k < 4; ++k) v[i][k] += ow * u[k];
+            *(float4*)(xs + c) = make_float4(v[i][0], v[i][1], v[i][2], v[i][3]);
+        }
+#pragma unroll
+        for (int k = 0; k < 4; ++k) ss += v[i][k] * v[i][k], su += v[i][k];
+    }
+    if (!p.h) return;
+    float mean = 0.0f;
+    if (p.h_center) {
+        mean = hy_block_sum(su, red) / (float)W;
+        ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+            if ((i * 256 + tid) * 4 < W) {
+#pragma unroll
+                for (int k = 0; k < 4; ++k) ss += (v[i][k] - mean) * (v[i][k] - mean);
+            }
+    }
+    ss = hy_block_sum(ss, red);
+    const float den = sqrtf(ss / (float)W + p.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int c = (i * 256 + tid) * 4;
+        if (c >= W) continue;
+        const float4 w = *(const float4*)(p.norm_w + c);
+        float4 o = make_float4((v[i][0] - mean) / den * w.x, (v[i][1] - mean) / den * w.y, (v[i][2] - mean) / den * w.z, (v[i][3] - mean) / den * w.w);
+        if (p.norm_b) {
+            const float4 b = *(const float4*)(p.norm_b + c);
+            o.x += b.x, o.y += b.y, o.z += b.z, o.w += b.w;
+        }
+        *(float4*)(p.h + m * W + c) = o;
+    }
+}
+
 // ---------------------------------------------------------------------------------------------------------------------------
 // the input of channel c, d positions before row t (d >= 1); `before` = rows of this step that continue into row t (at most taps - 1 counted)
 __device__ __forceinline__ float conv_input(const i64h_causal_conv_args& p, int64_t t, int d, int before, int c) {
@@ -759,6 +824,12 @@ int i64h_embed_bigram(const i64h_embed_bigram_args* dp, void* stream) {
     return 0;
 }
 
+static int g_residual_form = 1;
+int i64h_set_residual_form(int32_t on) {
+    g_residual_form = on != 0;
+    return 0;
+}
+
 int i64h_streams_step(const i64h_streams_args* dp, void* stream) {
     I64H_CHECK_ARG(dp != nullptr, "streams: no descriptor");
     const i64h_streams_args& d = *dp;
@@ -772,6 +843,17 @@ int i64h_streams_step(const i64h_streams_args* dp, void* stream) {
     const size_t lds = ((size_t)d.W + 4) * 4;
     I64H_CHECK_ARG(lds <= 64 * 1024, "streams: a row of %d values does not fit the kernel's LDS buffer", d.W);
     if (rows == 0) return 0;
+    const uintptr_t at = (uintptr_t)d.streams | (uintptr_t)d.y | (uintptr_t)d.y2 | (uintptr_t)d.y_scale | (uintptr_t)d.norm_w | (uintptr_t)d.norm_b | (uintptr_t)d.h;
+    if (g_residual_form && d.S == 1 && !d.mix && !d.in_w && !d.yn_w && !d.post_w && d.W % 4 == 0 && d.W <= 8 * 1024 && at % 16 == 0 && (!d.y || d.ldy % 4 == 0) &&
+        (!d.y2 || d.ldy2 % 4 == 0) && (!d.h || d.norm_w_len == d.W)) {
+        const dim3 grid((unsigned)rows);
+        if (d.W <= 1024) hipLaunchKernelGGL(residual_kernel<1>, grid, dim3(256), 0, (hipStream_t)stream, d);
+        else if (d.W <= 2048) hipLaunchKernelGGL(residual_kernel<2>, grid, dim3(256), 0, (hipStream_t)stream, d);
+        else if (d.W <= 4096) hipLaunchKernelGGL(residual_kernel<4>, grid, dim3(256), 0, (hipStream_t)stream, d);
+        else hipLaunchKernelGGL(residual_kernel<8>, grid, dim3(256), 0, (hipStream_t)stream, d);
+        I64H_CHECK_LAUNCH();
+        return 0;
+    }
     hipLaunchKernelGGL(streams_kernel, dim3((unsigned)rows), dim3(256), lds, (hipStream_t)stream, d);
     I64H_CHECK_LAUNCH();
     return 0;

@@ -227,9 +227,8 @@ class HybridRunner:
         width = r + rd
         src, q_off = P, d["q_off"]
         if m.q_rank:
-            cq, src, q_off = B.cq[: n * m.q_rank].view(n, m.q_rank), B.q[: n * H * qh].view(n, H * qh), 0
-            D.gate_norm(P, d["q_norm"], cq, groups=1, eps=self.cfg.norm_eps, y_off=d["q_off"], ldy=N1, n=n)
-            D.linear(cq, d["uq"], src, exact=ex)
+            src, q_off = B.q[: n * H * qh].view(n, H * qh), 0
+            D.linear(P, d["uq"], src, m=n, a_off=d["q_off"], exact=ex, in_norm_w=d["q_norm"], in_eps=self.cfg.norm_eps)
         cache = kvc.rows[l]
         Q = B.a[: n * H * width]
         D.latent_prep(P, q_off=q_off, dkv_off=d["dkv_off"], heads=H, dim=m.dim, rot_dim=rd, kv_rank=r, rot_dims=m.rot_dims, c_norm_w=d["c_norm"], eps=self.cfg.norm_eps,

@@ -12,7 +12,7 @@ from ._lib import call_dense, ptr
 from .ops import _chk, _stream
 
 EPI_STORE, EPI_GELU_MUL, EPI_MUL_SIGMOID, EPI_SOFTCAP, EPI_GELU_ERF, EPI_SCALE, EPI_SILU_MUL, EPI_XIELU, EPI_RELU_SQ = 0, 1, 2, 3, 4, 5, 6, 7, 8
-EPI_CLAMP_GLU, EPI_ADD, EPI_DECAY, EPI_ROW_SIGMOID = 9, 10, 11, 12
+EPI_CLAMP_GLU, EPI_ADD, EPI_DECAY, EPI_ROW_SIGMOID, EPI_IN_NORM = 9, 10, 11, 12, 13
 _DUAL = (EPI_GELU_MUL, EPI_SILU_MUL, EPI_CLAMP_GLU)
 CACHE_DTYPE_CODE = {torch.float32: 0, torch.bfloat16: 2}
 
@@ -26,13 +26,15 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
            batch: int = 1, a_batch: int = 0, w_batch: int = 0, c_batch: int = 0, exact: bool = False, epilogue: int = EPI_STORE,
            e: Optional[torch.Tensor] = None, e_off: int = 0, lde: int = 0, e_batch: int = 0, softcap: float = 0.0,
            bias: Optional[torch.Tensor] = None, bias_batch: int = 0, scale: float = 1.0, act_a: float = 0.0, act_b: float = 0.0,
-           group_off: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+           group_off: Optional[torch.Tensor] = None, row_scale: Optional[torch.Tensor] = None,
+           in_norm_w: Optional[torch.Tensor] = None, in_eps: float = 0.0) -> torch.Tensor:
     """out[b][:, c_off + b * c_batch : + n] = epilogue(a[b][rows, a_off + b * a_batch : + k] @ w[b]^T): see i64h_linear.  a, out and e are
     fp32 matrices addressed by (column offset, row stride; e with lde = 0 is one row for all); w is bf16 [n, k] (the gate / up epilogues: [2n, k], gate rows first), or a
     stack [batch, n, k] with w_batch = n * k.  bias fp32 [n] (per batch: bias_batch apart) is added before the epilogue.  group_off int32
     [batch + 1] on the device: batch b takes the rows [group_off[b], group_off[b + 1]) of a_rows (or a) and out; m is then the most rows a
     batch may have, and a_rows / a / out must hold group_off[batch] rows (the caller's business: the counts stay on the device).
-    row_scale fp32, one factor per row of out (the gate / up epilogues): the input row times that factor."""
+    row_scale fp32, one factor per row of out (the gate / up epilogues): the input row times that factor.
+    in_norm_w fp32 [k] with in_eps: the input rows are RMS-normed first (plain result: the epilogue is then EPI_IN_NORM)."""
     _chk(a, torch.float32, "a"), _chk(w, torch.bfloat16, "w"), _chk(out, torch.float32, "out")
     if a_rows is not None:
         _chk(a_rows, torch.int32, "a_rows")
@@ -55,6 +57,11 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
         _chk(bias, torch.float32, "bias")
         if bias.numel() < (batch - 1) * bias_batch + N:
             raise _lib.I64HError("linear: bias smaller than the launch reads")
+    if in_norm_w is not None:
+        _chk(in_norm_w, torch.float32, "in_norm_w")
+        if epilogue != EPI_STORE or in_norm_w.numel() != K:
+            raise _lib.I64HError("linear: the input norm's weights are not [k], or another epilogue is asked for beside it")
+        epilogue = EPI_IN_NORM
     if row_scale is not None:
         _chk(row_scale, torch.float32, "row_scale")
         if row_scale.numel() < M:
@@ -67,7 +74,7 @@ def linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, m: Optional[i
                     a_batch=a_batch, w_batch=w_batch, c_batch=c_batch, exact=int(exact), epilogue=epilogue,
                     E=(ptr(e) + 4 * e_off) if e is not None else 0, lde=lde, e_batch=e_batch, softcap=float(softcap),
                     bias=ptr(bias), bias_batch=int(bias_batch), scale=float(scale), act_a=float(act_a), act_b=float(act_b), group_off=ptr(group_off),
-                    row_scale=ptr(row_scale))
+                    row_scale=ptr(row_scale), in_norm_w=ptr(in_norm_w), in_eps=float(in_eps))
     call_dense("i64h_linear_run", _ref(d), _stream())
     return out
 

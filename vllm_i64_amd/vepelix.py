@@ -41,8 +41,7 @@ class _StepBuffers:
         self.y = torch.empty(n, W, **f32)                       # a sublayer's result
         self.y2 = torch.empty(n, W, **f32)                      # that of the right one of two side-by-side mixers / the shared expert's
         self.p = torch.empty(n * model.max_proj, **f32)         # everything projected from the mixer's input
-        self.cq = torch.empty(n * model.max_q_rank, **f32)      # the normed low-rank row of the queries
-        self.q = torch.empty(n * model.max_q, **f32)            # ... and the queries
+        self.q = torch.empty(n * model.max_q, **f32)            # the queries of the latent heads
         self.a = torch.empty(n * model.max_a, **f32)            # query rows of the attention
         self.b = torch.empty(n * model.max_b, **f32)            # attention output
         self.c = torch.empty(n * model.max_c, **f32)            # values of the latent heads
@@ -85,7 +84,6 @@ class VepelixModel(HybridRunner):
         self.max_a = max(d["n_a"] for d in self.layers)
         self.max_b = max(d["n_b"] for d in self.layers)
         self.max_c = max([m.heads * m.vdim for m in latents] or [0])
-        self.max_q_rank = max([m.q_rank for m in latents] or [0])
         self.max_q = max([m.q_width for m in latents] or [0])
         self.max_rk = max([r.heads * r.dim for r in rights] or [0])
         self.max_rv = max([r.heads * r.vdim for r in rights] or [0])
