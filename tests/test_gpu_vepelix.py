@@ -374,9 +374,10 @@ def test_gated_linear_attention_under_cuts(dev, H, d, dv, tau, cut_sizes):
 
 @pytest.mark.parametrize("H,d,dv", [(4, 64, 32), (3, 40, 24), (2, 128, 128), (2, 200, 40), (1, 12, 5)])
 @pytest.mark.parametrize("own_matrix", [True, False])
-def test_gated_linear_scan_forms_agree_bit_for_bit(dev, H, d, dv, own_matrix):
+@pytest.mark.parametrize("own_keys", [True, False])
+def test_gated_linear_scan_forms_agree_bit_for_bit(dev, H, d, dv, own_matrix, own_keys):
     """Loads straight into registers, or tokens staged through LDS with one, two or four value columns per lane; decays in a matrix of their own or
-    as columns of the projections: runs of unequal length, continued from slots' states or fresh, in scattered slots."""
+    as columns of the projections; keys of their own or one minus the decay: runs of unequal length, continued from slots' states or fresh, in scattered slots."""
     from vllm_i64_amd import _lib, ops_dense as D
     g = torch.Generator().manual_seed(d + dv)
     runs = [(4, 0, 33), (1, 7, 1), (0, 3, 16), (3, 0, 17), (2, 50, 70)]
@@ -391,7 +392,7 @@ def test_gated_linear_scan_forms_agree_bit_for_bit(dev, H, d, dv, own_matrix):
         for form in (1, 2, 3, 4, 0):
             _lib.call_dense("i64h_set_gdn_scan_form", form)
             S, O = S0.to(dev).clone(), torch.full((r.n, H * dv), 7.0, device=dev)
-            D.gla_scan(Pd, f=Fd if own_matrix else None, q_off=0, k_off=nd, f_off=0 if own_matrix else 2 * nd + H * dv, v_off=2 * nd, heads=H, dim=d, vdim=dv, seg_start=r.seg,
+            D.gla_scan(Pd, f=Fd if own_matrix else None, q_off=0, k_off=nd if own_keys else -1, f_off=0 if own_matrix else 2 * nd + H * dv, v_off=2 * nd, heads=H, dim=d, vdim=dv, seg_start=r.seg,
                        nseg=r.nseg, positions=r.pos, slot_ids=r.slots, state=S, out=O, n=r.n, q_scale=0.3)
             got.append((O.cpu(), S.cpu()))
     finally:
@@ -402,7 +403,8 @@ def test_gated_linear_scan_forms_agree_bit_for_bit(dev, H, d, dv, own_matrix):
     for slot, p, c in runs:      # (the fresh runs against the oracle's recurrence)
         x, f = P[at:at + c].double(), F[at:at + c].double()
         if p == 0:
-            o = R.gated_linear_recurrence(0.3 * x[:, :nd].reshape(c, H, d), x[:, nd:2 * nd].reshape(c, H, d), x[:, 2 * nd:2 * nd + H * dv].reshape(c, H, dv), f.reshape(c, H, d))
+            k = x[:, nd:2 * nd] if own_keys else 1.0 - f
+            o = R.gated_linear_recurrence(0.3 * x[:, :nd].reshape(c, H, d), k.reshape(c, H, d), x[:, 2 * nd:2 * nd + H * dv].reshape(c, H, dv), f.reshape(c, H, d))
             assert close(got[0][0][at:at + c], o.reshape(c, H * dv), 2e-5)
         at += c
 

@@ -4,7 +4,8 @@ libi64hip.so        the quantized token-routed-MoE forward (include/i64h.h)
 libi64hip_dense.so  models with bf16 weights and a 32-bit residual: Linear, gated post-norm, latent attention, multi-stream
                     residual, state-space / gated recurrences, key-valued chunked attention, attention with separate keys and values,
                     gated linear recurrence, rotated attention with capped scores, windows with kept first positions, gated delta rule (a decay
-                    per head or key channel), expert routing and grouped expert Linears, sampling
+                    per head or key channel), gated linear attention, Linears that norm their input, expert routing (softmax or sigmoid scores)
+                    and grouped expert Linears, sampling
                     (include/i64h_dense.h) - a library of its own, so that serving such a model builds nothing else
 """
 from __future__ import annotations

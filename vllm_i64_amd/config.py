@@ -644,8 +644,8 @@ class RotaryConfig:
 class RotaryAttentionConfig:
     """Causal softmax attention over grouped key / value heads with separate key and value sizes and rotated positions.  What a design
     fixes comes in as flags: qk_norm 'row' (RMS norm over the whole projection with weights 'q.norm' / 'k.norm', before the rotation),
-    'head' (per head, without weights, after it), 'head_weight' (per head, weights of dim values that the heads share, before it) or None; interleaved pairs (2i, 2i + 1) or halves (i, i + dims / 2); rotated values
-    (all vdim dimensions by the value's own position, the head's sum turned back by the query's); a sigmoid gate per head ('g')."""
+    'head' (per head, without weights, after it), 'head_weight' (per head, weights of dim values that the heads share, before it) or None;
+    interleaved pairs (2i, 2i + 1) or halves (i, i + dims / 2); rotated values (all vdim dimensions by the value's own position, the head's sum turned back by the query's); a sigmoid gate per head ('g')."""
     heads: int
     kv_heads: int
     dim: int

@@ -1,13 +1,11 @@
 // Kernels of libi64hip_dense.so for gated linear recurrences and mixtures of experts (include/i64h_dense.h):
 //   gla_gates_kernel   : query activation and bounded forget gate, in place on the projection rows
-//   gla_scan_kernel    : linear attention with a decay per key channel whose keys are one minus the decay, a head's matrix in registers (16
-//                        lanes per value column)
 //   gdn_gates_kernel / gdn_scan_kernel : gated delta rule - unit-vector queries and keys, write strength and decay; the recurrence with the
 //                        correction S^T k summed over the DPP row before the write, the read-out after it; a decay per head or per key channel;
-//                        without the correction: gated linear attention with keys of its own
+//                        without the correction: gated linear attention, with keys of its own or one minus the decay as the key
 //   gdn_tile_kernel    : the same recurrence for long runs, tokens staged through LDS
-//   route_topk_kernel  : softmax scores (over all entries or the chosen ones) or sigmoid scores, corrected choice, groups of neighbours, top-k and normalised
-//                        (or raw) weights, one wave per row
+//   route_topk_kernel  : softmax scores (over all entries or the chosen ones) or sigmoid scores, corrected choice, groups of
+//                        neighbours, top-k and normalised (or raw) weights, one wave per row (few rows: a workgroup per row)
 //   moe_plan_kernel    : (token, choice) pairs grouped by expert: offsets, the token of every grouped row, the row of every pair
 //   moe_combine_kernel : weighted sum of the chosen experts' rows, pass-through entries and the shared expert's row
 // A row continues the row before it iff slot and position say so; state is taken as empty at position 0.  All arithmetic fp32.
@@ -28,122 +26,6 @@ __global__ __launch_bounds__(256) void gla_gates_kernel(const i64h_gla_args p) {
     }
     const float lo = p.lower ? p.lower[c] : 0.0f;
     row[p.f_off + c] = lo + (1.0f - lo) * bl_sigmoid(row[p.f_off + c]);
-}
-
-// One workgroup per (head, 16 * CPT value columns, run of rows).  The 16 lanes of a DPP row share CPT neighbouring value columns and hold
-// KPT consecutive key channels of each in registers; a wave has four such rows.  The key is one minus the decay (keys of their own: the
-// delta rule's kernels below, without its correction).  Per token a lane loads its slices of the query and the decay once for its CPT columns, updates its states with fused multiply-adds and
-// the row sums the partial outputs with DPP moves: no LDS and no barrier, the tokens of a run strictly in their order (the same sums in
-// the same order however a prompt is cut).  Loads run GL_TG tokens ahead in two alternating register sets, so that a wave that is alone
-// on its SIMD still has a group of tokens in flight while it computes one.  State layout [slot, head, value column, key channel].
-#define GL_TG 4
-template <int KPT, int CPT>
-__global__ __launch_bounds__(256) void gla_scan_kernel(const i64h_gla_args p, const int ctiles, const int vec) {
-    const int N = p.dim, P = p.vdim;
-    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
-    const int nlane = lane & 15, cl = lane >> 4;
-    const int a = blockIdx.x / ctiles, seg = blockIdx.y;
-    const int cbase = (blockIdx.x % ctiles) * 16 * CPT + (w * 4 + cl) * CPT;
-    const int64_t r0 = p.seg_start[seg], r1 = p.seg_start[seg + 1];
-    if (r1 <= r0) return;
-    const int n0 = nlane * KPT;
-    float S[CPT][KPT];
-    float* gS = p.state + ((int64_t)p.slot_ids[r0] * p.heads + a) * P * N + n0;      // + column * N
-    const bool fresh = p.positions[r0] == 0;
-#pragma unroll
-    for (int j = 0; j < CPT; ++j) {
-        const bool cok = cbase + j < P;
-        const float* src = gS + (int64_t)(cok ? cbase + j : 0) * N;
-#pragma unroll
-        for (int k = 0; k < KPT; ++k) S[j][k] = 0.0f;
-        if (!fresh && cok) {
-            if (vec) {
-#pragma unroll
-                for (int k = 0; k < KPT; k += 4)
-                    if (n0 + k < N) {
-                        const float4 v = *(const float4*)(src + k);
-                        S[j][k] = v.x, S[j][k + 1] = v.y, S[j][k + 2] = v.z, S[j][k + 3] = v.w;
-                    }
-            } else {
-#pragma unroll
-                for (int k = 0; k < KPT; ++k)
-                    if (n0 + k < N) S[j][k] = src[k];
-            }
-        }
-    }
-    const int qoff = p.q_off + a * N + n0, foff = p.f_off + a * N + n0;
-    const float* const F = p.F ? p.F : p.P;
-    const int64_t ldf = p.F ? p.ldf : p.ldp;
-    struct Tok {
-        float q[KPT], f[KPT], v[CPT];
-    };
-    auto fetch = [&](int64_t t, Tok& u) {
-        if (t >= r1) return;
-        const float* row = p.P + t * p.ldp;
-        const float* frow = F + t * ldf;
-        if (vec) {      // KPT % 4 == 0 and every slice starts at a multiple of four floats and lies inside the row
-#pragma unroll
-            for (int k = 0; k < KPT; k += 4) {
-                float4 q = make_float4(0, 0, 0, 0), f = make_float4(1, 1, 1, 1);
-                if (n0 + k < N) {
-                    q = *(const float4*)(row + qoff + k);
-                    f = *(const float4*)(frow + foff + k);
-                }
-                u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
-                u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
-            }
-        } else {
-#pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                const bool ok = n0 + k < N;
-                u.q[k] = ok ? row[qoff + k] : 0.0f;
-                u.f[k] = ok ? frow[foff + k] : 1.0f;
-            }
-        }
-#pragma unroll
-        for (int j = 0; j < CPT; ++j) u.v[j] = cbase + j < P ? row[p.v_off + a * P + cbase + j] : 0.0f;
-    };
-    auto step = [&](int64_t t, const Tok& u) {
-        if (t >= r1) return;
-#pragma unroll
-        for (int j = 0; j < CPT; ++j) {
-            float part = 0.0f;
-#pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                S[j][k] = fmaf(u.f[k], S[j][k], (1.0f - u.f[k]) * u.v[j]);
-                part = fmaf(S[j][k], u.q[k], part);
-            }
-            part = group_sum(part, 16);
-            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = part * p.q_scale;
-        }
-    };
-    Tok A[GL_TG], B[GL_TG];
-#pragma unroll
-    for (int i = 0; i < GL_TG; ++i) fetch(r0 + i, A[i]);
-    for (int64_t t = r0; t < r1; t += 2 * GL_TG) {
-#pragma unroll
-        for (int i = 0; i < GL_TG; ++i) fetch(t + GL_TG + i, B[i]);
-#pragma unroll
-        for (int i = 0; i < GL_TG; ++i) step(t + i, A[i]);
-#pragma unroll
-        for (int i = 0; i < GL_TG; ++i) fetch(t + 2 * GL_TG + i, A[i]);
-#pragma unroll
-        for (int i = 0; i < GL_TG; ++i) step(t + GL_TG + i, B[i]);
-    }
-#pragma unroll
-    for (int j = 0; j < CPT; ++j) {
-        if (cbase + j >= P) continue;
-        float* dst = gS + (int64_t)(cbase + j) * N;
-        if (vec) {
-#pragma unroll
-            for (int k = 0; k < KPT; k += 4)
-                if (n0 + k < N) *(float4*)(dst + k) = make_float4(S[j][k], S[j][k + 1], S[j][k + 2], S[j][k + 3]);
-        } else {
-#pragma unroll
-            for (int k = 0; k < KPT; ++k)
-                if (n0 + k < N) dst[k] = S[j][k];
-        }
-    }
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -174,19 +56,21 @@ __global__ __launch_bounds__(256) void gdn_gates_kernel(const i64h_gdn_args p) {
     }
 }
 
-// gdn_scan_kernel: the layout of gla_scan_kernel (one workgroup per (head, 16 * CPT value columns, run of rows); the 16 lanes of a DPP
-// row share CPT value columns and hold KPT key channels of each in registers).  Per token the state decays, the row sums S^T k with DPP
+// gdn_scan_kernel: one workgroup per (head, 16 * CPT value columns, run of rows); the 16 lanes of a DPP row share CPT value columns and hold
+// KPT key channels of each in registers, a wave has four such rows.  Per token the state decays, the row sums S^T k with DPP
 // moves (every lane of the row ends with the sum), the correction along k is written, and a second row sum reads the state out with
-// the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order; loads run TG tokens ahead.
-// CHD: a decay per head and key channel (F) in the place of one per head.  RULE: the delta rule's correction and write strength; without it the
-// token writes k v^T as it is (gated linear attention) and the read-out is multiplied by q_scale.
+// the query - after the write.  No LDS and no barrier, the tokens of a run strictly in their order (the same sums in the same order however
+// a prompt is cut); loads run TG tokens ahead in two alternating register sets.  State layout [slot, head, value column, key channel].
+// CHD: a decay per head and key channel (F) in the place of one per head.  RULE: the delta rule's correction and write strength, or gated
+// linear attention: the token writes k v^T as it is, the read-out is multiplied by q_scale; the keys are the row's own or one minus the decay.
+enum { GD_DELTA = 0, GD_KEYS = 1, GD_FORGET = 2 };
 // TG is chosen so that two waves fit a SIMD's registers (the loads in flight are most of them); one where every run is a single row.
 // A lane's KPT channels: four neighbours in every stripe of 64 (so that 16 lanes read 256 consecutive bytes at a time).
 template <int KPT>
 __device__ __forceinline__ int gd_channel(int nlane, int k) {
     return KPT >= 4 ? 4 * (nlane + 16 * (k >> 2)) + (k & 3) : nlane * KPT + k;
 }
-template <int KPT, int CPT, bool CHD, int TG, bool RULE>
+template <int KPT, int CPT, bool CHD, int TG, int RULE>
 __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, const int ctiles, const int vec) {
     const int N = p.dim, P = p.vdim;
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -222,7 +106,7 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
     }
     const int qoff = p.q_off + kh * N, koff = p.k_off + kh * N, foff = a * N;
     struct Tok {
-        float q[KPT], k[KPT], f[CHD ? KPT : 1], v[CPT], beta;
+        float q[KPT], k[RULE == GD_FORGET ? 1 : KPT], f[CHD ? KPT : 1], v[CPT], beta;
     };
     auto fetch = [&](int64_t t, Tok& u) {
         if (t >= r1) return;
@@ -230,14 +114,14 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
         if (vec) {      // KPT % 4 == 0 and every slice starts at a multiple of four floats and lies inside the row
 #pragma unroll
             for (int k = 0; k < KPT; k += 4) {
-                float4 q = make_float4(0, 0, 0, 0), kk = q, f = q;
+                float4 q = make_float4(0, 0, 0, 0), kk = q, f = RULE == GD_FORGET ? make_float4(1, 1, 1, 1) : q;
                 if (gd_channel<KPT>(nlane, k) < N) {
                     q = *(const float4*)(row + qoff + gd_channel<KPT>(nlane, k));
-                    kk = *(const float4*)(row + koff + gd_channel<KPT>(nlane, k));
+                    if (RULE != GD_FORGET) kk = *(const float4*)(row + koff + gd_channel<KPT>(nlane, k));
                     if (CHD) f = *(const float4*)(p.F + t * p.ldf + foff + gd_channel<KPT>(nlane, k));
                 }
                 u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
-                u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
+                if (RULE != GD_FORGET) u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
                 if (CHD) u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
             }
         } else {
@@ -246,13 +130,13 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
                 const int c = gd_channel<KPT>(nlane, k);
                 const bool ok = c < N;
                 u.q[k] = ok ? row[qoff + c] : 0.0f;
-                u.k[k] = ok ? row[koff + c] : 0.0f;
-                if (CHD) u.f[k] = ok ? p.F[t * p.ldf + foff + c] : 0.0f;
+                if (RULE != GD_FORGET) u.k[k] = ok ? row[koff + c] : 0.0f;
+                if (CHD) u.f[k] = ok ? p.F[t * p.ldf + foff + c] : (RULE == GD_FORGET ? 1.0f : 0.0f);
             }
         }
 #pragma unroll
         for (int j = 0; j < CPT; ++j) u.v[j] = cbase + j < P ? row[p.v_off + a * P + cbase + j] : 0.0f;
-        if (RULE) u.beta = p.G[t * 2 * p.heads + a];
+        if (RULE == GD_DELTA) u.beta = p.G[t * 2 * p.heads + a];
         if (!CHD) u.f[0] = p.G[t * 2 * p.heads + p.heads + a];
     };
     auto step = [&](int64_t t, const Tok& u) {
@@ -260,7 +144,7 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
 #pragma unroll
         for (int j = 0; j < CPT; ++j) {
             float part = 0.0f;
-            if (RULE) {
+            if constexpr (RULE == GD_DELTA) {
                 float seen = 0.0f;
 #pragma unroll
                 for (int k = 0; k < KPT; ++k) {
@@ -277,12 +161,13 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
             } else {
 #pragma unroll
                 for (int k = 0; k < KPT; ++k) {
-                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], u.k[k] * u.v[j]);
+                    const float kk = RULE == GD_FORGET ? 1.0f - u.f[CHD ? k : 0] : u.k[RULE == GD_FORGET ? 0 : k];
+                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], kk * u.v[j]);
                     part = fmaf(S[j][k], u.q[k], part);
                 }
             }
             part = group_sum(part, 16);
-            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = RULE ? part : part * p.q_scale;
+            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = RULE == GD_DELTA ? part : part * p.q_scale;
         }
     };
     Tok A[TG], B[TG];
@@ -317,11 +202,11 @@ __global__ __launch_bounds__(256) void gdn_scan_kernel(const i64h_gdn_args p, co
 // gdn_tile_kernel: the same recurrence, bit for bit, for runs of many rows.  What every wave of a workgroup reads of a token (query, key,
 // decays) is loaded once per workgroup, TT tokens at a time, into one of two LDS tiles while the other one is computed: the loads of a
 // tile have the arithmetic of a whole tile to arrive, and the waves read 16 bytes per lane from LDS one token ahead.  Needs 16-byte rows.
-template <int KPT, int CPT, bool CHD, bool RULE>
+template <int KPT, int CPT, bool CHD, int RULE>
 __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, const int ctiles) {
     static_assert(KPT % 4 == 0, "whole 16-byte slices per lane");
     constexpr int TT = KPT > 8 ? 8 : 16;      // tokens per tile
-    constexpr int NP = 16 * KPT, PARTS = CHD ? 3 : 2, LPP = TT * NP / 4 / 256, WC = 16 * CPT;     // LPP: 16-byte loads per thread and part
+    constexpr int NP = 16 * KPT, PARTS = CHD && RULE != GD_FORGET ? 3 : 2, LPP = TT * NP / 4 / 256, WC = 16 * CPT;     // LPP: 16-byte loads per thread and part
     constexpr int VPT = (TT * WC + 255) / 256;
     __shared__ __attribute__((aligned(16))) float sX[2][PARTS][TT][NP];
     __shared__ float sV[2][TT][WC];
@@ -359,8 +244,9 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
             const bool ok = t < r1 && c < N;
             const float* row = p.X + t * p.ldx;
             st[0][u] = ok ? *(const float4*)(row + p.q_off + kh * N + c) : make_float4(0, 0, 0, 0);
-            st[1][u] = ok ? *(const float4*)(row + p.k_off + kh * N + c) : make_float4(0, 0, 0, 0);
-            if (CHD) st[PARTS - 1][u] = ok ? *(const float4*)(p.F + t * p.ldf + a * N + c) : make_float4(0, 0, 0, 0);
+            if (RULE != GD_FORGET) st[1][u] = ok ? *(const float4*)(row + p.k_off + kh * N + c) : make_float4(0, 0, 0, 0);
+            const float pad = RULE == GD_FORGET ? 1.0f : 0.0f;
+            if (CHD) st[PARTS - 1][u] = ok ? *(const float4*)(p.F + t * p.ldf + a * N + c) : make_float4(pad, pad, pad, pad);
         }
 #pragma unroll
         for (int u = 0; u < VPT; ++u) {
@@ -370,7 +256,7 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
         }
         if (tid < 2 * TT) {
             const int64_t t = t0 + (tid >> 1);
-            sg = (t < r1 && (RULE || (tid & 1)) && !(CHD && (tid & 1))) ? p.G[t * 2 * p.heads + (tid & 1) * p.heads + a] : 0.0f;
+            sg = (t < r1 && (RULE == GD_DELTA || (tid & 1)) && !(CHD && (tid & 1))) ? p.G[t * 2 * p.heads + (tid & 1) * p.heads + a] : 0.0f;
         }
     };
     auto lstore = [&](int b) {
@@ -386,15 +272,18 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
         if (tid < 2 * TT) sG[b][tid >> 1][tid & 1] = sg;
     };
     struct Tok {
-        float q[KPT], k[KPT], f[CHD ? KPT : 1], v[CPT], beta;
+        float q[KPT], k[RULE == GD_FORGET ? 1 : KPT], f[CHD ? KPT : 1], v[CPT], beta;
     };
     auto fetch = [&](int b, int i, Tok& u) {
 #pragma unroll
         for (int k = 0; k < KPT; k += 4) {
             const int c = gd_channel<KPT>(nlane, k);
-            const float4 q = *(const float4*)&sX[b][0][i][c], kk = *(const float4*)&sX[b][1][i][c];
+            const float4 q = *(const float4*)&sX[b][0][i][c];
             u.q[k] = q.x, u.q[k + 1] = q.y, u.q[k + 2] = q.z, u.q[k + 3] = q.w;
-            u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
+            if (RULE != GD_FORGET) {
+                const float4 kk = *(const float4*)&sX[b][1][i][c];
+                u.k[k] = kk.x, u.k[k + 1] = kk.y, u.k[k + 2] = kk.z, u.k[k + 3] = kk.w;
+            }
             if (CHD) {
                 const float4 f = *(const float4*)&sX[b][PARTS - 1][i][c];
                 u.f[k] = f.x, u.f[k + 1] = f.y, u.f[k + 2] = f.z, u.f[k + 3] = f.w;
@@ -407,13 +296,14 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
     };
     auto step = [&](int64_t t, const Tok& u) {
         float seen[CPT], part[CPT], d[CPT];
-        if (!RULE) {
+        if constexpr (RULE != GD_DELTA) {
 #pragma unroll
             for (int j = 0; j < CPT; ++j) {
                 part[j] = 0.0f;
 #pragma unroll
                 for (int k = 0; k < KPT; ++k) {
-                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], u.k[k] * u.v[j]);
+                    const float kk = RULE == GD_FORGET ? 1.0f - u.f[CHD ? k : 0] : u.k[RULE == GD_FORGET ? 0 : k];
+                    S[j][k] = fmaf(u.f[CHD ? k : 0], S[j][k], kk * u.v[j]);
                     part[j] = fmaf(S[j][k], u.q[k], part[j]);
                 }
             }
@@ -422,32 +312,32 @@ __global__ __launch_bounds__(256) void gdn_tile_kernel(const i64h_gdn_args p, co
                 const float o = group_sum(part[j], 16);
                 if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = o * p.q_scale;
             }
-            return;
-        }
+        } else {
 #pragma unroll
-        for (int j = 0; j < CPT; ++j) {
-            seen[j] = 0.0f;
+            for (int j = 0; j < CPT; ++j) {
+                seen[j] = 0.0f;
 #pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                S[j][k] *= u.f[CHD ? k : 0];
-                seen[j] = fmaf(S[j][k], u.k[k], seen[j]);
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] *= u.f[CHD ? k : 0];
+                    seen[j] = fmaf(S[j][k], u.k[k], seen[j]);
+                }
             }
-        }
 #pragma unroll
-        for (int j = 0; j < CPT; ++j) d[j] = u.beta * (u.v[j] - group_sum(seen[j], 16));
+            for (int j = 0; j < CPT; ++j) d[j] = u.beta * (u.v[j] - group_sum(seen[j], 16));
 #pragma unroll
-        for (int j = 0; j < CPT; ++j) {
-            part[j] = 0.0f;
+            for (int j = 0; j < CPT; ++j) {
+                part[j] = 0.0f;
 #pragma unroll
-            for (int k = 0; k < KPT; ++k) {
-                S[j][k] = fmaf(u.k[k], d[j], S[j][k]);
-                part[j] = fmaf(S[j][k], u.q[k], part[j]);
+                for (int k = 0; k < KPT; ++k) {
+                    S[j][k] = fmaf(u.k[k], d[j], S[j][k]);
+                    part[j] = fmaf(S[j][k], u.q[k], part[j]);
+                }
             }
-        }
 #pragma unroll
-        for (int j = 0; j < CPT; ++j) {
-            const float o = group_sum(part[j], 16);
-            if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = o;
+            for (int j = 0; j < CPT; ++j) {
+                const float o = group_sum(part[j], 16);
+                if (nlane == 0 && cbase + j < P) p.out[t * p.ldo + a * P + cbase + j] = o;
+            }
         }
     };
     gload(r0);
@@ -738,9 +628,9 @@ int i64h_set_gdn_scan_form(int32_t form) {
     return 0;
 }
 
-// the recurrence's launch, with the delta rule's correction or (RULE = false: a decay per key channel, keys of every head's own) without it
+// the recurrence's launch, with the delta rule's correction or (a decay per key channel, every head its own keys) without it
 extern "C++" {
-template <bool RULE>
+template <int RULE>
 static int gdn_launch(const i64h_gdn_args& d, void* stream) {
     const int kpt = (d.dim + 15) / 16;
     auto vec_ok = [&](int K) {
@@ -758,9 +648,9 @@ static int gdn_launch(const i64h_gdn_args& d, void* stream) {
     if (kround == 4) launch(gdn_tile_kernel<4, C, CHD, RULE>);      \
     else if (kround == 8) launch(gdn_tile_kernel<8, C, CHD, RULE>); \
     else launch(gdn_tile_kernel<16, C, CHD, RULE>);
-        if (!RULE || d.F) {
+        if (RULE != GD_DELTA || d.F) {
             if (cpt == 1) { GDN_TILE(1, true) } else if (cpt == 2) { GDN_TILE(2, true) } else { GDN_TILE(4, true) }
-        } else if constexpr (RULE) {
+        } else if constexpr (RULE == GD_DELTA) {
             if (cpt == 1) { GDN_TILE(1, false) } else if (cpt == 2) { GDN_TILE(2, false) } else { GDN_TILE(4, false) }
         }
 #undef GDN_TILE
@@ -784,9 +674,9 @@ static int gdn_launch(const i64h_gdn_args& d, void* stream) {
     else launch(gdn_scan_kernel<16, C, CHD, ONE ? 1 : (CHD ? 1 : 2), RULE>, 16);
 #define GDN_PICK2(C, CHD) \
     if (d.nseg == d.n) { GDN_PICK(C, CHD, true) } else { GDN_PICK(C, CHD, false) }
-    if (!RULE || d.F) {
+    if (RULE != GD_DELTA || d.F) {
         if (cpt == 2) { GDN_PICK2(2, true) } else { GDN_PICK2(1, true) }
-    } else if constexpr (RULE) {
+    } else if constexpr (RULE == GD_DELTA) {
         if (cpt == 2) { GDN_PICK2(2, false) } else { GDN_PICK2(1, false) }
     }
 #undef GDN_PICK2
@@ -804,7 +694,7 @@ int i64h_gdn_scan(const i64h_gdn_args* dp, void* stream) {
     I64H_CHECK_ARG(d.dim <= 16 * 16, "gdn_scan: dim %d above 256", d.dim);
     I64H_CHECK_ARG(d.nseg <= 65535, "gdn_scan: %d runs in one launch", d.nseg);
     if (d.nseg <= 0 || d.n == 0) return 0;
-    return gdn_launch<true>(d, stream);
+    return gdn_launch<GD_DELTA>(d, stream);
 }
 
 int i64h_gla_scan(const i64h_gla_args* dp, void* stream) {
@@ -816,33 +706,11 @@ int i64h_gla_scan(const i64h_gla_args* dp, void* stream) {
     I64H_CHECK_ARG(d.nseg <= 65535, "gla_scan: %d runs in one launch", d.nseg);
     I64H_CHECK_ARG(!d.F || d.ldf >= d.f_off + (int64_t)d.heads * d.dim, "gla_scan: the decays' rows are shorter than their columns");
     if (d.nseg <= 0 || d.n == 0) return 0;
-    if (d.k_off >= 0) {      // keys of their own: the delta rule's kernels without the correction
-        i64h_gdn_args a = {};
-        a.X = d.P, a.ldx = d.ldp, a.q_off = d.q_off, a.k_off = d.k_off, a.v_off = d.v_off, a.heads = a.kv_heads = d.heads, a.dim = d.dim, a.vdim = d.vdim;
-        a.F = (d.F ? d.F : d.P) + d.f_off, a.ldf = d.F ? d.ldf : d.ldp, a.q_scale = d.q_scale, a.seg_start = d.seg_start, a.nseg = d.nseg;
-        a.positions = d.positions, a.slot_ids = d.slot_ids, a.state = d.state, a.out = d.out, a.ldo = d.ldo, a.n = d.n;
-        return gdn_launch<false>(a, stream);
-    }
-    const int kpt = (d.dim + 15) / 16;
-    // columns per lane: query and decay are loaded once for both - unless the launch would then leave most of the chip idle
-    const int cpt = (d.vdim > 16 && (int64_t)d.heads * ((d.vdim + 31) / 32) * d.nseg >= 512) ? 2 : 1;
-    const int ctiles = (d.vdim + 16 * cpt - 1) / (16 * cpt);
-    const dim3 grid((unsigned)(d.heads * ctiles), (unsigned)d.nseg);
-    auto launch = [&](auto kern, int K) {
-        const int vec = K % 4 == 0 && d.dim % 4 == 0 && d.ldp % 4 == 0 && d.q_off % 4 == 0 && d.f_off % 4 == 0 && (uintptr_t)d.P % 16 == 0 && (uintptr_t)d.state % 16 == 0 &&
-                        (!d.F || (d.ldf % 4 == 0 && (uintptr_t)d.F % 16 == 0));
-        hipLaunchKernelGGL(kern, grid, dim3(256), 0, (hipStream_t)stream, d, ctiles, vec);
-    };
-#define GLA_PICK(C)                                          \
-    if (kpt <= 1) launch(gla_scan_kernel<1, C>, 1);          \
-    else if (kpt <= 2) launch(gla_scan_kernel<2, C>, 2);     \
-    else if (kpt <= 4) launch(gla_scan_kernel<4, C>, 4);     \
-    else if (kpt <= 8) launch(gla_scan_kernel<8, C>, 8);     \
-    else launch(gla_scan_kernel<16, C>, 16);
-    if (cpt == 2) { GLA_PICK(2) } else { GLA_PICK(1) }
-#undef GLA_PICK
-    I64H_CHECK_LAUNCH();
-    return 0;
+    i64h_gdn_args a = {};
+    a.X = d.P, a.ldx = d.ldp, a.q_off = d.q_off, a.k_off = d.k_off >= 0 ? d.k_off : 0, a.v_off = d.v_off, a.heads = a.kv_heads = d.heads, a.dim = d.dim, a.vdim = d.vdim;
+    a.F = (d.F ? d.F : d.P) + d.f_off, a.ldf = d.F ? d.ldf : d.ldp, a.q_scale = d.q_scale, a.seg_start = d.seg_start, a.nseg = d.nseg;
+    a.positions = d.positions, a.slot_ids = d.slot_ids, a.state = d.state, a.out = d.out, a.ldo = d.ldo, a.n = d.n;
+    return d.k_off >= 0 ? gdn_launch<GD_KEYS>(a, stream) : gdn_launch<GD_FORGET>(a, stream);
 }
 
 int i64h_route_topk(const i64h_route_args* dp, void* stream) {

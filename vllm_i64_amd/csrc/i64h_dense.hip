@@ -2,7 +2,7 @@
 //   linear_tile_kernel   : C = epilogue(A W^T), 64 x 64 tiles, four waves of 32 x 32, on v_mfma_f32_16x16x32_bf16 (A rounded to
 //                          bf16 while staged) or v_mfma_f32_16x16x4_f32 (W widened while staged: true 32-bit); batched over
 //                          blockIdx.z (per-head weights on column blocks of wider matrices); epilogues: gelu_tanh(gate) * up
-//                          on two accumulators, * sigmoid(E), logit soft cap
+//                          on two accumulators, * sigmoid(E), logit soft cap and others; an RMS norm of its input on the way
 //   linear_tile128_kernel: bf16 form, 128 x 128 tiles (waves of 64 x 64); behind a knob, measured slower at the sizes tried
 //   linear_skinny_kernel : the same product for at most I64H_SKINNY_ROWS rows (decode steps): the rows sit in LDS as bf16, every
 //                          wave streams four weight rows at a time with 16-byte loads and reduces over its lanes

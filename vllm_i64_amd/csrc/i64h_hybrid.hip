@@ -3,6 +3,7 @@
 //   streams_kernel        : multi-stream residual write (a result may pass a norm of its own first, and the result as a whole an RMS or
 //                           centred norm) + the next sublayer's weighted read
 //                           and RMS norm, one workgroup per row
+//   residual_kernel       : the ordinary residual sum (one or two results, a factor per column) + the next norm, the row in registers
 //   causal_conv_kernel / conv_carry_kernel : per-channel causal convolution over rows and carried inputs (+ silu, or added to its input);
 //                           the carry update
 //   ssm_scan_kernel       : state-space recurrence with a scalar decay per head, a head's matrix in registers (16 lanes per value column)

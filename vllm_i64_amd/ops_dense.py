@@ -302,25 +302,22 @@ def ssm_scan(xbc: torch.Tensor, dt: torch.Tensor, *, dt_off: int, lddt: int, dt_
 
 
 def gate_norm(y: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, groups: int, eps: float, z: Optional[torch.Tensor] = None, z_off: int = 0,
-              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None, sigmoid: bool = False,
-              y_off: int = 0, ldy: Optional[int] = None) -> torch.Tensor:
+              ldz: int = 0, n: Optional[int] = None, gate_after: bool = False, width: Optional[int] = None, sigmoid: bool = False) -> torch.Tensor:
     """out = rms_groups(y * silu(z)) * w: see i64h_gate_norm.  y, out fp32 [n, width]; z the columns [z_off, + width) of a matrix of row stride ldz.
-    gate_after: out = rms_groups(y) * w * silu(z).  sigmoid: the gate is sigmoid(z).  width (default: w's length): the row's width, w then repeats over it.
-    y_off, ldy: the columns [y_off, + width) of a matrix of row stride ldy (default: y is [n, width])."""
+    gate_after: out = rms_groups(y) * w * silu(z).  sigmoid: the gate is sigmoid(z).  width (default: w's length): the row's width, w then repeats over it."""
     _chk(y, torch.float32, "y"), _chk(w, torch.float32, "w"), _chk(out, torch.float32, "out")
     w_len = w.numel()
     width = int(width if width is not None else w_len)
     if width % w_len:
         raise _lib.I64HError("gate_norm: the weights do not repeat evenly over the row")
     rows = int(n if n is not None else y.numel() // width)
-    ldy = int(ldy if ldy is not None else width)
-    if y_off + width > ldy or y.numel() < (rows - 1) * ldy + y_off + width or out.numel() < rows * width:
+    if y.numel() < rows * width or out.numel() < rows * width:
         raise _lib.I64HError("gate_norm: operand smaller than the launch reads or writes")
     if z is not None:
         _chk(z, torch.float32, "z")
         if z.numel() < (rows - 1) * ldz + z_off + width:
             raise _lib.I64HError("gate_norm: gate smaller than the launch reads")
-    d = _lib.GateNorm(y=ptr(y) + 4 * y_off, ldy=ldy, z=(ptr(z) + 4 * z_off) if z is not None else 0, ldz=ldz, w=ptr(w), width=width, groups=groups, eps=float(eps),
+    d = _lib.GateNorm(y=ptr(y), ldy=width, z=(ptr(z) + 4 * z_off) if z is not None else 0, ldz=ldz, w=ptr(w), width=width, groups=groups, eps=float(eps),
                       out=ptr(out), ldo=width, n=rows, gate_after=int(bool(gate_after)), w_len=w_len if w_len != width else 0, gate_act=int(bool(sigmoid)))
     call_dense("i64h_gate_norm", _ref(d), _stream())
     return out
